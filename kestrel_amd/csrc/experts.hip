@@ -5,6 +5,7 @@
 // A pair is p = token * top + choice. chosen[p] names the router's output that the token chose there: a number below
 // n_experts is an expert with weights, a number from n_experts on an identity expert whose output is the token's input.
 #include "ka_common.h"
+#include "ka_rows.h"
 
 constexpr int EX_MAX_OUTPUTS = 512;             // router outputs a wave can hold (8 a lane)
 constexpr int EX_PER_LANE = EX_MAX_OUTPUTS / KA_WAVE;
@@ -30,11 +31,13 @@ __device__ __forceinline__ void ex_wave_argmax(float& v, int& i) {
 //       and only outputs of the `keep` best groups can be chosen;
 //     the `top` outputs with the largest choice scores are chosen (the lower index wins a tie);
 //     weights: their s divided by the sum of the chosen s (+ 1e-20), times scale.
+// by_logits: the choice goes by the logits themselves (no correction, no groups); the weights are the softmax over the chosen
+// logits, times scale.
 // chosen int32 [n, top], weights fp32 [n, top].
 // ----------------------------------------------------------------------------
 __global__ void __launch_bounds__(KA_WAVE)
 route_kernel(const float* __restrict__ logits, long stride, const float* __restrict__ correction, int R, int top, int n_groups,
-             int keep, float scale, int* __restrict__ chosen, float* __restrict__ weights) {
+             int keep, float scale, int by_logits, int* __restrict__ chosen, float* __restrict__ weights) {
     __shared__ float choice_s[EX_MAX_OUTPUTS];
     __shared__ float group_s[EX_MAX_GROUPS];
     __shared__ int allowed_s[EX_MAX_GROUPS];
@@ -52,6 +55,7 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
     float total = 0.f;
 #pragma unroll
     for (int q = 0; q < EX_PER_LANE; ++q) {
+        c[q] = s[q];
         s[q] = lane + q * KA_WAVE < R ? expf(s[q] - top_z) : 0.f;
         total += s[q];
     }
@@ -59,6 +63,7 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
 #pragma unroll
     for (int q = 0; q < EX_PER_LANE; ++q) {
         const int r = lane + q * KA_WAVE;
+        if (by_logits) continue;      // (the largest logit is among the chosen: e^(z - top) over their sum is their softmax)
         s[q] = s[q] / total;
         c[q] = r < R ? s[q] + (correction ? correction[r] : 0.f) : -INFINITY;
         if (r < R) choice_s[r] = c[q];
@@ -120,13 +125,14 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
     }
     if (lane < top) {
         chosen[(size_t)t * top + lane] = mine_i;
-        weights[(size_t)t * top + lane] = mine_w / (sum + 1e-20f) * scale;
+        weights[(size_t)t * top + lane] = mine_w / (by_logits ? sum : sum + 1e-20f) * scale;
     }
 }
 
 KA_API int ka_route(const float* logits, long stride, const float* correction, int n, int R, int top, int n_groups, int keep,
-                    float scale, int* chosen, float* weights, hipStream_t stream) {
+                    float scale, int by_logits, int* chosen, float* weights, hipStream_t stream) {
     const char* who = "ka_route";
+    KA_CHECK(!by_logits || (n_groups == 0 && correction == nullptr), "%s: a choice by the logits alone has no groups and no correction", who);
     KA_CHECK(n >= 0 && R > 0 && R <= EX_MAX_OUTPUTS && stride >= R, "%s: %d router outputs (at most %d)", who, R, EX_MAX_OUTPUTS);
     KA_CHECK(top > 0 && top <= R && top <= KA_WAVE, "%s: %d choices of %d", who, top, R);
     KA_CHECK(n_groups >= 0 && n_groups <= EX_MAX_GROUPS && (n_groups == 0 || (R % n_groups == 0 && keep > 0 && keep <= n_groups)),
@@ -134,7 +140,7 @@ KA_API int ka_route(const float* logits, long stride, const float* correction, i
     KA_CHECK(n_groups == 0 || keep * (R / n_groups) >= top, "%s: %d kept groups hold fewer than %d outputs", who, keep, top);
     if (n == 0) return 0;
     hipLaunchKernelGGL(route_kernel, dim3(n), dim3(KA_WAVE), 0, stream, logits, stride, correction, R, top, n_groups, keep, scale,
-                       chosen, weights);
+                       by_logits, chosen, weights);
     KA_LAUNCH_CHECK();
     return 0;
 }
@@ -258,6 +264,86 @@ KA_API int ka_experts_combine(const float* y, const void* h, long h_stride, int 
     else
         hipLaunchKernelGGL(experts_combine_kernel<bf16_t>, dim3(n), dim3(256), 0, stream, y, (const bf16_t*)h, h_stride, chosen, weights,
                            top, E, shared, shared_gate, gate_stride, out, dim, accumulate);
+    KA_LAUNCH_CHECK();
+    return 0;
+}
+
+// ----------------------------------------------------------------------------
+// The weighted sum of ka_experts_combine as the output of a sublayer whose norm stands behind it: it is normalised and
+// added into the fp32 stream x, and the norm of the new rows is computed, in the same launch (ka_rows.h). A workgroup
+// per token; the sums are those of ka_experts_combine, in its order.
+// ----------------------------------------------------------------------------
+template <typename T, int PIECES>
+__global__ void __launch_bounds__(KA_ROW_THREADS)
+experts_combine_normed_kernel(const float* __restrict__ y, const T* __restrict__ h_in, long h_stride, const int* __restrict__ chosen,
+                              const float* __restrict__ weights, int top, int E, const float* __restrict__ shared,
+                              const float* __restrict__ shared_gate, long gate_stride, float* __restrict__ x, int dim, KaRowNorms a) {
+    __shared__ float smem[KA_ROW_WAVES];
+    const int t = blockIdx.x;
+    const float sg = shared ? (shared_gate ? 1.0f / (1.0f + expf(-shared_gate[(size_t)t * gate_stride])) : 1.f) : 0.f;
+    auto one = [&](int c) {
+        float acc = 0.f;
+        for (int k = 0; k < top; ++k) {
+            const int e = chosen[(size_t)t * top + k];
+            const float v = e < E ? y[((size_t)t * top + k) * dim + c] : ka_to_float(h_in[(size_t)t * h_stride + c]);
+            acc = fmaf(weights[(size_t)t * top + k], v, acc);
+        }
+        return shared ? fmaf(sg, shared[(size_t)t * dim + c], acc) : acc;
+    };
+    auto piece = [&](int c) {
+        float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+        for (int k = 0; k < top; ++k) {
+            const int e = chosen[(size_t)t * top + k];
+            const float w = weights[(size_t)t * top + k];
+            float4 v;
+            if (e < E) {
+                v = *reinterpret_cast<const float4*>(y + ((size_t)t * top + k) * dim + c);
+            } else {
+                const T* hp = h_in + (size_t)t * h_stride + c;
+                v = make_float4(ka_to_float(hp[0]), ka_to_float(hp[1]), ka_to_float(hp[2]), ka_to_float(hp[3]));
+            }
+            acc.x = fmaf(w, v.x, acc.x);
+            acc.y = fmaf(w, v.y, acc.y);
+            acc.z = fmaf(w, v.z, acc.z);
+            acc.w = fmaf(w, v.w, acc.w);
+        }
+        if (shared) {
+            const float4 v = *reinterpret_cast<const float4*>(shared + (size_t)t * dim + c);
+            acc.x = fmaf(sg, v.x, acc.x);
+            acc.y = fmaf(sg, v.y, acc.y);
+            acc.z = fmaf(sg, v.z, acc.z);
+            acc.w = fmaf(sg, v.w, acc.w);
+        }
+        return acc;
+    };
+    ka_finish_row<PIECES>(x, t, dim, a, piece, one, smem);
+}
+
+KA_API int ka_experts_combine_normed(const float* y, const void* h_in, long h_stride, int dtype, const int* chosen, const float* weights,
+                                     int n, int top, int E, const float* shared, const float* shared_gate, long gate_stride, float* x,
+                                     int dim, const float* gain, float eps, const float* gain2, float eps2, void* h, hipStream_t stream) {
+    const char* who = "ka_experts_combine_normed";
+    KA_CHECK(n >= 0 && top > 0 && dim > 0 && h_stride >= dim && eps >= 0.f && eps2 >= 0.f && gain != nullptr, "%s: bad sizes", who);
+    KA_CHECK(dtype == KA_F32 || dtype == KA_BF16, "%s: unsupported dtype %d", who, dtype);
+    KA_CHECK((gain2 == nullptr) == (h == nullptr), "%s: the second norm needs gains and rows", who);
+    if (n == 0) return 0;
+    const KaRowNorms a{gain, eps, gain2, eps2, h, dtype == KA_BF16};
+    const dim3 grid(n), block(KA_ROW_THREADS);
+    const int pieces = (uintptr_t)shared % 16 == 0 ? ka_row_pieces(dim, x, y, a) : 0;
+#define EX_COMBINE(T, P)                                                                                                            \
+    hipLaunchKernelGGL((experts_combine_normed_kernel<T, P>), grid, block, 0, stream, y, (const T*)h_in, h_stride, chosen, weights, top, E, \
+                       shared, shared_gate, gate_stride, x, dim, a)
+#define EX_COMBINE_ALL(T)                   \
+    switch (pieces) {                       \
+        case 1: EX_COMBINE(T, 1); break;    \
+        case 2: EX_COMBINE(T, 2); break;    \
+        case 4: EX_COMBINE(T, 4); break;    \
+        case 8: EX_COMBINE(T, 8); break;    \
+        default: EX_COMBINE(T, 0); break;   \
+    }
+    if (dtype == KA_F32) { EX_COMBINE_ALL(float) } else { EX_COMBINE_ALL(bf16_t) }
+#undef EX_COMBINE_ALL
+#undef EX_COMBINE
     KA_LAUNCH_CHECK();
     return 0;
 }

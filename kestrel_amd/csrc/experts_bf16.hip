@@ -137,9 +137,16 @@ experts_gemm_kernel(const bf16_t* __restrict__ a, long lda, int gather_div, cons
                     }
                 } else {
                     bf16_t* op = reinterpret_cast<bf16_t*>(out) + row * ldo + o;
+                    eb_bf16x4 y;
 #pragma unroll
-                    for (int x = 0; x < 4; ++x)
-                        if (o + x < N) op[x] = (bf16_t)(ka_act_base(act) ? ka_activate_fast(act, acc_here[g4 * 4 + x]) : acc_here[g4 * 4 + x]);
+                    for (int x = 0; x < 4; ++x) y[x] = (bf16_t)(ka_act_base(act) ? ka_activate_fast(act, acc_here[g4 * 4 + x]) : acc_here[g4 * 4 + x]);
+                    if (o + 3 < N && ldo % 4 == 0) {
+                        *reinterpret_cast<eb_bf16x4*>(op) = y;
+                    } else {
+#pragma unroll
+                        for (int x = 0; x < 4; ++x)
+                            if (o + x < N) op[x] = y[x];
+                    }
                 }
             }
         }
@@ -273,9 +280,16 @@ experts_gemm_lds_kernel(const bf16_t* __restrict__ a, long lda, int gather_div, 
                     }
                 } else {
                     bf16_t* op = reinterpret_cast<bf16_t*>(out) + row * ldo + o;
+                    eb_bf16x4 y;
 #pragma unroll
-                    for (int x = 0; x < 4; ++x)
-                        if (o + x < N) op[x] = (bf16_t)(ka_act_base(act) ? ka_activate_fast(act, acc_here[g4 * 4 + x]) : acc_here[g4 * 4 + x]);
+                    for (int x = 0; x < 4; ++x) y[x] = (bf16_t)(ka_act_base(act) ? ka_activate_fast(act, acc_here[g4 * 4 + x]) : acc_here[g4 * 4 + x]);
+                    if (o + 3 < N && ldo % 4 == 0) {
+                        *reinterpret_cast<eb_bf16x4*>(op) = y;
+                    } else {
+#pragma unroll
+                        for (int x = 0; x < 4; ++x)
+                            if (o + x < N) op[x] = y[x];
+                    }
                 }
             }
         }

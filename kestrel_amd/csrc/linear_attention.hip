@@ -1,0 +1,288 @@
+// Kernels of attention without a softmax, run as a recurrence: the walk over a row's tokens one by one, and the norm of
+// what it reads. fp32 or bf16 storage of what the projections made; activations, the state and all sums are fp32.
+#include "ka_common.h"
+
+constexpr int LA_THREADS = 256;
+
+// ----------------------------------------------------------------------------
+// Per request and head a state S [dv, d] (value channel by key channel), fp32. For every token of a row, in order,
+//     S <- decay_h S + v k^T,    o = S q,         q, k, v = act(projected)
+// and o [dv] is left in `raw` in fp32. A value channel's row of S is independent of the others: a head is dealt out over
+// workgroups by slices of value channels (blockIdx.z) and over groups of LI lanes, a lane holding four key channels (NV
+// times) of NJ value channels in registers; a read-out is a sum over the LI lanes of a group inside the vector unit.
+// Nothing passes between waves. One launch takes whatever a step holds: a prompt, a portion, single tokens. The next
+// token's numbers are asked for before the current token's sums. A row without a request (slot < 0) gets zeros.
+// ----------------------------------------------------------------------------
+struct LinearAttentionArgs {
+    const void* q;
+    const void* k;
+    const void* v;
+    long stride;            // of the rows of q, k and v
+    const float* decay;     // [H]
+    float* state;           // [slots, state_stride]: S [H, dv, d]
+    long state_stride;
+    const int* cu_q;
+    const int* row_slot;
+    float* raw;             // [n, H dv]
+    int H, d, dv, act, vectors;
+};
+
+template <typename T>
+__device__ __forceinline__ float4 la_four(const T* p, int c, int d, bool vectors) {
+    typedef __attribute__((ext_vector_type(4))) T vec;
+    if (vectors) {
+        if (c >= d) return make_float4(0.f, 0.f, 0.f, 0.f);
+        const vec x = *reinterpret_cast<const vec*>(p + c);
+        return make_float4(ka_to_float(x[0]), ka_to_float(x[1]), ka_to_float(x[2]), ka_to_float(x[3]));
+    }
+    return make_float4(c < d ? ka_to_float(p[c]) : 0.f, c + 1 < d ? ka_to_float(p[c + 1]) : 0.f, c + 2 < d ? ka_to_float(p[c + 2]) : 0.f,
+                       c + 3 < d ? ka_to_float(p[c + 3]) : 0.f);
+}
+
+// (every activation of the table maps 0 to 0: channels behind the last stay out of the sums)
+template <typename T>
+__device__ __forceinline__ float la_act(int act, float x) {
+    return sizeof(T) == 2 ? ka_activate_fast(act, x) : ka_activate(act, x);
+}
+template <typename T>
+__device__ __forceinline__ float4 la_act4(int act, float4 x) {
+    return make_float4(la_act<T>(act, x.x), la_act<T>(act, x.y), la_act<T>(act, x.z), la_act<T>(act, x.w));
+}
+
+template <typename T, int LI, int NV, int NJ>
+__global__ void __launch_bounds__(LA_THREADS) linear_attention_kernel(LinearAttentionArgs a) {
+    constexpr int JW = LA_THREADS / LI;
+    const int head = blockIdx.x, row = blockIdx.y, tid = threadIdx.x;
+    const int li = tid % LI, jr = tid / LI;
+    const int d = a.d, dv = a.dv;
+    const int j0 = blockIdx.z * (JW * NJ);
+    const int t0 = a.cu_q[row], t1 = a.cu_q[row + 1];
+    if (t0 >= t1) return;
+    const int slot = a.row_slot[row];
+    const size_t out_at = (size_t)head * dv, out_row = (size_t)a.H * dv;
+    if (slot < 0) {
+        for (int t = t0; t < t1; ++t)
+#pragma unroll
+            for (int m = 0; m < NJ; ++m) {
+                const int j = j0 + m * JW + jr;
+                if (li == 0 && j < dv) a.raw[(size_t)t * out_row + out_at + j] = 0.f;
+            }
+        return;
+    }
+    const bool vectors = a.vectors != 0;
+    float* S_mem = a.state + (size_t)slot * a.state_stride + (size_t)head * dv * d;
+    const T* qp = reinterpret_cast<const T*>(a.q) + (size_t)head * d;
+    const T* kp = reinterpret_cast<const T*>(a.k) + (size_t)head * d;
+    const T* vp = reinterpret_cast<const T*>(a.v) + (size_t)head * dv;
+    const float keep = a.decay[head];
+    float4 S[NJ][NV];
+    int jc[NJ];             // (value channels behind the last are clamped for the loads and not stored)
+#pragma unroll
+    for (int m = 0; m < NJ; ++m) {
+        const int j = j0 + m * JW + jr;
+        jc[m] = min(j, dv - 1);
+#pragma unroll
+        for (int u = 0; u < NV; ++u) S[m][u] = la_four(S_mem + (size_t)jc[m] * d, (u * LI + li) * 4, d, d % 4 == 0);
+    }
+    float4 qn[NV], kn[NV];
+    float vn[NJ];
+    auto fetch = [&](int t) {
+        const size_t at = (size_t)t * a.stride;
+#pragma unroll
+        for (int u = 0; u < NV; ++u) {
+            qn[u] = la_four(qp + at, (u * LI + li) * 4, d, vectors);
+            kn[u] = la_four(kp + at, (u * LI + li) * 4, d, vectors);
+        }
+#pragma unroll
+        for (int m = 0; m < NJ; ++m) vn[m] = ka_to_float(vp[at + jc[m]]);
+    };
+    fetch(t0);
+    for (int t = t0; t < t1; ++t) {
+        float4 q[NV], k[NV];
+        float v[NJ];
+#pragma unroll
+        for (int u = 0; u < NV; ++u) {
+            q[u] = la_act4<T>(a.act, qn[u]);
+            k[u] = la_act4<T>(a.act, kn[u]);
+        }
+#pragma unroll
+        for (int m = 0; m < NJ; ++m) v[m] = la_act<T>(a.act, vn[m]);
+        if (t + 1 < t1) fetch(t + 1);
+#pragma unroll
+        for (int m = 0; m < NJ; ++m) {
+            float acc = 0.f;
+#pragma unroll
+            for (int u = 0; u < NV; ++u) {
+                float4& s = S[m][u];
+                s.x = fmaf(keep, s.x, k[u].x * v[m]);
+                s.y = fmaf(keep, s.y, k[u].y * v[m]);
+                s.z = fmaf(keep, s.z, k[u].z * v[m]);
+                s.w = fmaf(keep, s.w, k[u].w * v[m]);
+                acc = fmaf(q[u].x, s.x, acc);
+                acc = fmaf(q[u].y, s.y, acc);
+                acc = fmaf(q[u].z, s.z, acc);
+                acc = fmaf(q[u].w, s.w, acc);
+            }
+            acc = ka_lanes_reduce<1, LI>(acc, KaSum{});
+            const int j = j0 + m * JW + jr;
+            if (li == 0 && j < dv) a.raw[(size_t)t * out_row + out_at + j] = acc;
+        }
+    }
+#pragma unroll
+    for (int m = 0; m < NJ; ++m) {
+        const int j = j0 + m * JW + jr;
+        if (j >= dv) continue;
+#pragma unroll
+        for (int u = 0; u < NV; ++u) {
+            const int c = (u * LI + li) * 4;
+            float* p = S_mem + (size_t)j * d + c;
+            if (d % 4 == 0) {
+                if (c < d) *reinterpret_cast<float4*>(p) = S[m][u];
+            } else {
+                if (c < d) p[0] = S[m][u].x;
+                if (c + 1 < d) p[1] = S[m][u].y;
+                if (c + 2 < d) p[2] = S[m][u].z;
+                if (c + 3 < d) p[3] = S[m][u].w;
+            }
+        }
+    }
+}
+
+constexpr int LA_MAX_D = 512;
+
+KA_API int ka_linear_attention_supported(int d, int dv) { return d > 0 && d <= LA_MAX_D && dv > 0 ? 1 : 0; }
+
+KA_API int ka_linear_attention(const void* q, const void* k, const void* v, long stride, int dtype, const float* decay, float* state,
+                               long state_stride, const int* cu_q, const int* row_slot, float* raw, int n, int n_rows, int H, int d,
+                               int dv, int act, hipStream_t stream) {
+    const char* who = "ka_linear_attention";
+    KA_CHECK(n >= 0 && n_rows >= 0 && H > 0 && ka_linear_attention_supported(d, dv), "%s: heads of %d x %d channels are not covered (keys up to %d)", who, d, dv, LA_MAX_D);
+    KA_CHECK(dtype == KA_F32 || dtype == KA_BF16, "%s: unsupported dtype %d", who, dtype);
+    KA_CHECK(ka_act_known(act) && !ka_act_gated(act), "%s: unknown activation %d", who, act);
+    KA_CHECK(state_stride >= (long)H * d * dv && (uintptr_t)state % 16 == 0 && (d % 4 != 0 || state_stride % 4 == 0), "%s: the state rows are too short or not aligned", who);
+    KA_CHECK(stride >= (long)H * d && stride >= (long)H * dv, "%s: rows are shorter than their heads", who);
+    KA_CHECK(H <= 65535 && n_rows <= 65535, "%s: too many heads or rows", who);
+    if (n == 0 || n_rows == 0) return 0;
+    const size_t align = dtype == KA_F32 ? 16 : 8;
+    const int vectors = d % 4 == 0 && stride % 4 == 0 && (uintptr_t)q % align == 0 && (uintptr_t)k % align == 0;
+    LinearAttentionArgs a{q, k, v, stride, decay, state, state_stride, cu_q, row_slot, raw, H, d, dv, act, vectors};
+    const int lanes = d <= 32 ? 8 : d <= 64 ? 16 : d <= 128 ? 32 : 64;
+    // (few workgroups: a value channel a group of lanes; many: four, so that a token's keys and queries serve four)
+    const int jw = LA_THREADS / lanes;
+    const int nj = (long)H * n_rows * ka_cdiv(dv, jw) >= 8L * ka_compute_units() ? 4 : 1;
+    const dim3 grid(H, n_rows, ka_cdiv(dv, jw * nj));
+#define LA_LAUNCH(T, LI, NV, NJ) hipLaunchKernelGGL((linear_attention_kernel<T, LI, NV, NJ>), grid, dim3(LA_THREADS), 0, stream, a)
+#define LA_LAUNCH_NJ(T, LI, NV)          \
+    if (nj == 4) LA_LAUNCH(T, LI, NV, 4); \
+    else LA_LAUNCH(T, LI, NV, 1)
+#define LA_LAUNCH_ALL(T)                                \
+    if (lanes == 8) { LA_LAUNCH_NJ(T, 8, 1); }          \
+    else if (lanes == 16) { LA_LAUNCH_NJ(T, 16, 1); }   \
+    else if (lanes == 32) { LA_LAUNCH_NJ(T, 32, 1); }   \
+    else if (d <= 256) { LA_LAUNCH_NJ(T, 64, 1); }      \
+    else { LA_LAUNCH_NJ(T, 64, 2); }
+    if (dtype == KA_F32) { LA_LAUNCH_ALL(float) } else { LA_LAUNCH_ALL(bf16_t) }
+#undef LA_LAUNCH_ALL
+#undef LA_LAUNCH_NJ
+#undef LA_LAUNCH
+    KA_LAUNCH_CHECK();
+    return 0;
+}
+
+// ----------------------------------------------------------------------------
+// out[t] = x[t] / sqrt(mean(x[t]^2) + eps) * gain * sigmoid(gate[t]) over whole fp32 rows x [n, dim] (gain, gate optional):
+// a workgroup per row, which stays in registers where it has up to 4 PIECES LA_THREADS channels in pieces of four.
+// ----------------------------------------------------------------------------
+__device__ __forceinline__ float la_block_sum(float v, float* smem) {
+    v = ka_wave_sum(v);
+    if (threadIdx.x % KA_WAVE == 0) smem[threadIdx.x / KA_WAVE] = v;
+    __syncthreads();
+    float total = 0.f;
+#pragma unroll
+    for (int w = 0; w < LA_THREADS / KA_WAVE; ++w) total += smem[w];
+    return total;
+}
+
+template <typename T>
+__device__ __forceinline__ float la_sigmoid(float x) {
+    return sizeof(T) == 2 ? __fdividef(1.0f, 1.0f + __expf(-x)) : 1.0f / (1.0f + expf(-x));
+}
+
+template <typename T, int PIECES>
+__global__ void __launch_bounds__(LA_THREADS)
+gated_rmsnorm_kernel(const float* __restrict__ x, const float* __restrict__ gain, const T* __restrict__ gate, long gate_stride,
+                     T* __restrict__ out, int dim, float eps) {
+    __shared__ float smem[LA_THREADS / KA_WAVE];
+    typedef __attribute__((ext_vector_type(4))) T vec;
+    const int t = blockIdx.x, tid = threadIdx.x;
+    const float* row = x + (size_t)t * dim;
+    const T* g = gate ? gate + (size_t)t * gate_stride : nullptr;
+    T* o = out + (size_t)t * dim;
+    if constexpr (PIECES > 0) {
+        float4 v[PIECES];
+        vec gt[PIECES];
+        float s = 0.f;
+#pragma unroll
+        for (int p = 0; p < PIECES; ++p) {
+            const int c = (p * LA_THREADS + tid) * 4;
+            if (c < dim) {
+                v[p] = *reinterpret_cast<const float4*>(row + c);
+                if (g) gt[p] = *reinterpret_cast<const vec*>(g + c);
+                s += v[p].x * v[p].x + v[p].y * v[p].y + v[p].z * v[p].z + v[p].w * v[p].w;
+            }
+        }
+        const float r = 1.0f / sqrtf(la_block_sum(s, smem) / (float)dim + eps);
+#pragma unroll
+        for (int p = 0; p < PIECES; ++p) {
+            const int c = (p * LA_THREADS + tid) * 4;
+            if (c < dim) {
+                float y[4] = {v[p].x * r, v[p].y * r, v[p].z * r, v[p].w * r};
+                vec b;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    if (gain) y[e] *= gain[c + e];
+                    if (g) y[e] *= la_sigmoid<T>(ka_to_float(gt[p][e]));
+                    b[e] = ka_from_float<T>(y[e]);
+                }
+                *reinterpret_cast<vec*>(o + c) = b;
+            }
+        }
+    } else {
+        float s = 0.f;
+        for (int c = tid; c < dim; c += LA_THREADS) s += row[c] * row[c];
+        const float r = 1.0f / sqrtf(la_block_sum(s, smem) / (float)dim + eps);
+        for (int c = tid; c < dim; c += LA_THREADS) {
+            float y = row[c] * r * (gain ? gain[c] : 1.f);
+            if (g) y *= la_sigmoid<T>(ka_to_float(g[c]));
+            o[c] = ka_from_float<T>(y);
+        }
+    }
+}
+
+KA_API int ka_gated_rmsnorm(const float* x, const float* gain, const void* gate, long gate_stride, void* out, int dtype, int n, int dim,
+                            float eps, hipStream_t stream) {
+    const char* who = "ka_gated_rmsnorm";
+    KA_CHECK(n >= 0 && dim > 0 && eps >= 0.f && (gate == nullptr || gate_stride >= dim), "%s: bad sizes", who);
+    KA_CHECK(dtype == KA_F32 || dtype == KA_BF16, "%s: unsupported dtype %d", who, dtype);
+    if (n == 0) return 0;
+    const size_t align = dtype == KA_F32 ? 16 : 8;
+    const bool vectors = dim % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)out % align == 0 &&
+                         (gate == nullptr || ((uintptr_t)gate % align == 0 && gate_stride % 4 == 0));
+    const int need = ka_cdiv(dim, 4 * LA_THREADS);
+    const int pieces = !vectors || need > 8 ? 0 : need <= 1 ? 1 : need <= 2 ? 2 : need <= 4 ? 4 : 8;
+#define LA_NORM(T, P) \
+    hipLaunchKernelGGL((gated_rmsnorm_kernel<T, P>), dim3(n), dim3(LA_THREADS), 0, stream, x, gain, (const T*)gate, gate_stride, (T*)out, dim, eps)
+#define LA_NORM_ALL(T)                   \
+    switch (pieces) {                    \
+        case 1: LA_NORM(T, 1); break;    \
+        case 2: LA_NORM(T, 2); break;    \
+        case 4: LA_NORM(T, 4); break;    \
+        case 8: LA_NORM(T, 8); break;    \
+        default: LA_NORM(T, 0); break;   \
+    }
+    if (dtype == KA_F32) { LA_NORM_ALL(float) } else { LA_NORM_ALL(bf16_t) }
+#undef LA_NORM_ALL
+#undef LA_NORM
+    KA_LAUNCH_CHECK();
+    return 0;
+}

@@ -4,6 +4,7 @@
 // layer, the paged cache write), an output gate, the sum of normalised branches, and a gated matrix memory
 // (a recurrent mixer with a state of fixed size per request). fp32 or bf16 storage, all arithmetic in fp32.
 #include "ka_common.h"
+#include "ka_rows.h"
 
 constexpr int MP_THREADS = 256;
 constexpr int MP_WAVES = MP_THREADS / KA_WAVE;
@@ -442,6 +443,36 @@ KA_API int ka_branches_sum(float* x, const float* a, const float* gain_a, float 
     else
         hipLaunchKernelGGL(branches_sum_kernel<float>, dim3(n), dim3(MP_THREADS), 0, stream, x, a, gain_a, ca, b, gain_b, cb, eps, dim,
                            (float*)rounded);
+    KA_LAUNCH_CHECK();
+    return 0;
+}
+
+// ----------------------------------------------------------------------------
+// x += d / rms(d) * gain for fp32 rows d and, of the new rows, h = x / rms(x) * gain2 (h optional): ka_rows.h.
+// ----------------------------------------------------------------------------
+template <int PIECES>
+__global__ void __launch_bounds__(KA_ROW_THREADS)
+add_normed_kernel(float* __restrict__ x, const float* __restrict__ d, KaRowNorms a, int dim) {
+    __shared__ float smem[KA_ROW_WAVES];
+    const float* row = d + (size_t)blockIdx.x * dim;
+    ka_finish_row<PIECES>(x, blockIdx.x, dim, a, [&](int c) { return *reinterpret_cast<const float4*>(row + c); },
+                          [&](int c) { return row[c]; }, smem);
+}
+
+KA_API int ka_add_normed(float* x, const float* d, const float* gain, float eps, const float* gain2, float eps2, void* h, int h_dtype,
+                         int n, int dim, hipStream_t stream) {
+    KA_CHECK(n >= 0 && dim > 0 && eps >= 0.f && eps2 >= 0.f && gain != nullptr, "ka_add_normed: bad sizes or no gain");
+    KA_CHECK((gain2 == nullptr) == (h == nullptr) && (h_dtype == KA_F32 || h_dtype == KA_BF16), "ka_add_normed: the second norm needs gains and rows");
+    if (n == 0) return 0;
+    const KaRowNorms a{gain, eps, gain2, eps2, h, h_dtype == KA_BF16};
+    const dim3 grid(n), block(KA_ROW_THREADS);
+    switch (ka_row_pieces(dim, x, d, a)) {
+        case 1: hipLaunchKernelGGL(add_normed_kernel<1>, grid, block, 0, stream, x, d, a, dim); break;
+        case 2: hipLaunchKernelGGL(add_normed_kernel<2>, grid, block, 0, stream, x, d, a, dim); break;
+        case 4: hipLaunchKernelGGL(add_normed_kernel<4>, grid, block, 0, stream, x, d, a, dim); break;
+        case 8: hipLaunchKernelGGL(add_normed_kernel<8>, grid, block, 0, stream, x, d, a, dim); break;
+        default: hipLaunchKernelGGL(add_normed_kernel<0>, grid, block, 0, stream, x, d, a, dim); break;
+    }
     KA_LAUNCH_CHECK();
     return 0;
 }

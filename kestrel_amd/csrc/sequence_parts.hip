@@ -436,22 +436,27 @@ KA_API int ka_clamped_pairs(const void* x, long x_stride, void* out, long out_st
 }
 
 // ----------------------------------------------------------------------------
-// x[t] += v for every row of fp32 x [n, dim] (a learned vector that enters the stream at a junction).
+// x[t] += v (+ other[t]) for every row of fp32 x [n, dim] (a learned vector that enters the stream at a junction, with or
+// without another fp32 stream of the same tokens).
 // ----------------------------------------------------------------------------
 template <typename T>
-__global__ void add_vector_kernel(float* __restrict__ x, const T* __restrict__ v, long count, int dim) {
+__global__ void add_vector_kernel(float* __restrict__ x, const T* __restrict__ v, const float* __restrict__ other, long count, int dim) {
     const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
-    if (i < count) x[i] += ka_to_float(v[i % dim]);
+    if (i < count) {
+        float y = x[i];
+        if (other) y += other[i];
+        x[i] = y + ka_to_float(v[i % dim]);
+    }
 }
 
-KA_API int ka_add_vector(float* x, const void* v, int v_dtype, int n, int dim, hipStream_t stream) {
+KA_API int ka_add_vector(float* x, const void* v, int v_dtype, const float* other, int n, int dim, hipStream_t stream) {
     KA_CHECK(n >= 0 && dim > 0, "ka_add_vector: bad sizes");
     KA_CHECK(v_dtype == KA_F32 || v_dtype == KA_BF16, "ka_add_vector: unsupported dtype %d", v_dtype);
     const long count = (long)n * dim;
     if (count == 0) return 0;
     const unsigned blocks = (unsigned)((count + 255) / 256);
-    if (v_dtype == KA_F32) hipLaunchKernelGGL(add_vector_kernel<float>, dim3(blocks), dim3(256), 0, stream, x, (const float*)v, count, dim);
-    else hipLaunchKernelGGL(add_vector_kernel<bf16_t>, dim3(blocks), dim3(256), 0, stream, x, (const bf16_t*)v, count, dim);
+    if (v_dtype == KA_F32) hipLaunchKernelGGL(add_vector_kernel<float>, dim3(blocks), dim3(256), 0, stream, x, (const float*)v, other, count, dim);
+    else hipLaunchKernelGGL(add_vector_kernel<bf16_t>, dim3(blocks), dim3(256), 0, stream, x, (const bf16_t*)v, other, count, dim);
     KA_LAUNCH_CHECK();
     return 0;
 }

@@ -25,6 +25,8 @@ class DecoderModel:
         self.blocks: List[Block] = [Block(layer) for layer in plan.layers]
         self.final_norm = build_part("norm", plan.final_norm)
         self.position = build_part("position", plan.position) if plan.position is not None else None
+        embedding_norm = getattr(plan, "embedding_norm", None)
+        self.embedding_norm = build_part("norm", embedding_norm) if embedding_norm is not None else None
         self.junctions = {name: build_part("junction", spec) for name, spec in dict(getattr(plan, "junctions", None) or {}).items()}
         for index, entry in enumerate(plan.schedule):
             before = getattr(entry, "before", None)
@@ -53,6 +55,9 @@ class DecoderModel:
             out.update(block.params())
         for local, pspec in self.final_norm.params().items():
             out[plan.names[f"final_norm.{local}"]] = pspec
+        if self.embedding_norm is not None:
+            for local, pspec in self.embedding_norm.params().items():
+                out[plan.names[f"embedding_norm.{local}"]] = pspec
         if self.position is not None:
             for local, pspec in self.position.params().items():
                 out[plan.names[f"position.{local}"]] = pspec
@@ -73,6 +78,8 @@ class DecoderModel:
             block.bind(tensors, dtype, device)
         self.final_norm.bind({k: tensors[plan.names[f"final_norm.{k}"]] for k in self.final_norm.params()}, dtype,
                              device)
+        if self.embedding_norm is not None:
+            self.embedding_norm.bind({k: tensors[plan.names[f"embedding_norm.{k}"]] for k in self.embedding_norm.params()}, dtype, device)
         if self.position is not None:
             self.position.bind({k: tensors[plan.names[f"position.{k}"]] for k in self.position.params()}, dtype, device)
         for name, junction in self.junctions.items():
@@ -102,7 +109,7 @@ class DecoderModel:
     def replays_every_step(self) -> bool:
         """Whether steps of every shape may be captured and replayed: every part of the model says so
         (``Part.replays_every_step``)."""
-        parts = [self.final_norm, self.position] + list(self.junctions.values())
+        parts = [self.final_norm, self.embedding_norm, self.position] + list(self.junctions.values())
         for block in self.blocks:
             parts += list(block.parts().values()) + [getattr(block.mixer, "position", None)]
         return all(bool(getattr(part, "replays_every_step", False)) for part in parts if part is not None)
@@ -130,9 +137,13 @@ class DecoderModel:
         plan = self.plan
         ws = batch.workspace
         x = ws.get("model.x", (batch.n_tokens, plan.dim), torch.float32)
-        core.embed(self.embedding, batch.token_ids, x, batch.pending, plan.embedding_scale)
+        # (a norm of the embedded tokens reads them from a buffer of their own)
+        looked_up = x if self.embedding_norm is None else ws.get("model.looked_up", (batch.n_tokens, plan.dim), torch.float32)
+        core.embed(self.embedding, batch.token_ids, looked_up, batch.pending, plan.embedding_scale)
         if batch.given_embeds is not None:
-            core.scatter_rows(batch.given_embeds, batch.given_rows, x)
+            core.scatter_rows(batch.given_embeds, batch.given_rows, looked_up)
+        if self.embedding_norm is not None:
+            self.embedding_norm.forward(looked_up, x)
         if self.position is not None:
             position_state = getattr(self.position, "state_spec", None)
             if callable(position_state) and position_state() is not None:

@@ -49,7 +49,13 @@ _SIGNATURES = {
     "ka_rotate_tail": [_c_void_p, _c_int, _c_long, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_int,
                        _c_int, _c_void_p, _c_void_p],
     "ka_clamped_pairs": [_c_void_p, _c_long, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void_p],
-    "ka_add_vector": [_c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
+    "ka_add_vector": [_c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_void_p],
+    "ka_add_normed": [_c_void_p, _c_void_p, _c_void_p, _c_float, _c_void_p, _c_float, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
+    "ka_experts_combine_normed": [_c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p,
+                                  _c_long, _c_void_p, _c_int, _c_void_p, _c_float, _c_void_p, _c_float, _c_void_p, _c_void_p],
+    "ka_linear_attention": [_c_void_p, _c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_void_p, _c_void_p,
+                            _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+    "ka_gated_rmsnorm": [_c_void_p, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_int, _c_int, _c_int, _c_float, _c_void_p],
     "ka_gate_mul": [_c_void_p, _c_long, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_void_p],
     "ka_branches_sum": [_c_void_p, _c_void_p, _c_void_p, _c_float, _c_void_p, _c_void_p, _c_float, _c_float, _c_int, _c_int,
                         _c_void_p, _c_int, _c_void_p],
@@ -61,7 +67,7 @@ _SIGNATURES = {
     "ka_decayed_memory": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                           _c_long, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_float,
                           _c_void_p, _c_void_p],
-    "ka_route": [_c_void_p, _c_long, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void_p, _c_void_p, _c_void_p],
+    "ka_route": [_c_void_p, _c_long, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_void_p, _c_void_p, _c_void_p],
     "ka_experts_linear": [_c_void_p, _c_long, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p,
                           _c_long, _c_int, _c_void_p],
     "ka_experts_combine": [_c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p,
@@ -445,13 +451,79 @@ def clamped_pairs(x: torch.Tensor, out: torch.Tensor, limit: float, slope: float
                                   code_of(x.dtype), n, n_out, float(limit), float(slope), float(shift), stream_ptr()))
 
 
-def add_vector(x: torch.Tensor, vector: torch.Tensor) -> None:
-    """``x[t] += vector`` for every row of fp32 ``x`` ``[n, dim]``."""
-    _dev(x, vector)
+def add_vector(x: torch.Tensor, vector: torch.Tensor, other: Optional[torch.Tensor] = None) -> None:
+    """``x[t] += vector`` for every row of fp32 ``x`` ``[n, dim]``; with ``other`` (fp32, the shape of ``x``) ``x += other`` first."""
+    _dev(x, vector, other)
     n, dim = x.shape
     _need(x.dtype == torch.float32 and x.is_contiguous() and vector.numel() == dim and vector.is_contiguous(),
           "add_vector: x must be contiguous fp32 [n, dim] and the vector [dim]")
-    _check(lib().ka_add_vector(x.data_ptr(), vector.data_ptr(), code_of(vector.dtype), n, dim, stream_ptr()))
+    _need(other is None or (other.dtype == torch.float32 and other.is_contiguous() and other.shape == x.shape),
+          "add_vector: other must be contiguous fp32 of the shape of x")
+    _check(lib().ka_add_vector(x.data_ptr(), vector.data_ptr(), code_of(vector.dtype), _ptr(other), n, dim, stream_ptr()))
+
+
+def _norm_pair(who: str, x, norm, then, rows):
+    """The operands of "add a normalised row into the stream, then norm the new row": both norms ``(gain fp32 [dim], eps)``."""
+    n, dim = x.shape
+    _need(x.dtype == torch.float32 and x.is_contiguous(), f"{who}: the stream must be contiguous fp32 [n, dim]")
+    for pair in (norm,) + ((then,) if then is not None else ()):
+        gain = pair[0]
+        _need(gain.is_cuda and gain.dtype == torch.float32 and gain.is_contiguous() and gain.numel() == dim, f"{who}: gains fp32 [dim]")
+    _need((then is None) == (rows is None), f"{who}: the second norm needs its rows")
+    _need(rows is None or (rows.is_cuda and rows.is_contiguous() and tuple(rows.shape) == (n, dim)), f"{who}: rows must be [n, dim]")
+    return (norm[0].data_ptr(), float(norm[1]), None if then is None else then[0].data_ptr(), 0.0 if then is None else float(then[1]),
+            _ptr(rows))
+
+
+def add_normed(x: torch.Tensor, delta: torch.Tensor, norm, then=None, rows: Optional[torch.Tensor] = None) -> None:
+    """``x += delta / rms(delta) * gain`` for fp32 rows ``delta`` into the fp32 stream ``x``, with ``norm = (gain, eps)`` and
+    ``rms(y) = sqrt(mean(y^2) + eps)``; with ``then`` (the same form) also ``rows = x / rms(x) * gain`` of the new rows."""
+    _dev(x, delta, rows)
+    n, dim = x.shape
+    _need(delta.dtype == torch.float32 and delta.is_contiguous() and delta.shape == x.shape, "add_normed: delta must be fp32 of the shape of x")
+    _check(lib().ka_add_normed(x.data_ptr(), delta.data_ptr(), *_norm_pair("add_normed", x, norm, then, rows),
+                               code_of(rows.dtype) if rows is not None else KA_F32, n, dim, stream_ptr()))
+
+
+def linear_attention_supported(head_dim: int, value_dim: int) -> bool:
+    return 0 < head_dim <= 512 and value_dim > 0
+
+
+def linear_attention(projected: torch.Tensor, offsets, decay: torch.Tensor, state: torch.Tensor, cu_q: torch.Tensor,
+                     row_slot: torch.Tensor, raw: torch.Tensor, n_heads: int, head_dim: int, value_dim: int, act: int) -> None:
+    """``S <- decay_h S + v k^T, o = S q`` over every row's tokens in order, with ``q, k, v = act(.)`` of the columns of ``projected``
+    that begin at ``offsets`` (``H head_dim``, ``H head_dim``, ``H value_dim`` of them). ``state`` fp32 ``[slots + 1, H value_dim
+    head_dim]`` is read and advanced, ``raw`` fp32 ``[n, H value_dim]`` gets the read-outs; rows without a request (``row_slot`` -1)
+    get zeros."""
+    _dev(projected, decay, state, cu_q, row_slot, raw)
+    n = projected.shape[0]
+    _need(linear_attention_supported(head_dim, value_dim), "linear_attention: head sizes not covered")
+    oq, ok, ov = (int(o) for o in offsets)
+    _need(projected.dim() == 2 and projected.stride(1) == 1 and max(oq + n_heads * head_dim, ok + n_heads * head_dim, ov + n_heads * value_dim)
+          <= projected.shape[1], "linear_attention: the projected rows are too short")
+    _need(decay.dtype == torch.float32 and decay.numel() == n_heads and decay.is_contiguous(), "linear_attention: decay fp32 [H]")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] == n_heads * head_dim * value_dim,
+          "linear_attention: state fp32 [slots, H dv d]")
+    n_rows = row_slot.numel()
+    _need(cu_q.dtype == torch.int32 and cu_q.numel() == n_rows + 1 and row_slot.dtype == torch.int32, "linear_attention: cu_q int32 [rows + 1]")
+    _need(raw.dtype == torch.float32 and raw.is_contiguous() and tuple(raw.shape) == (n, n_heads * value_dim), "linear_attention: raw fp32 [n, H dv]")
+    size, base = projected.element_size(), projected.data_ptr()
+    _check(lib().ka_linear_attention(base + oq * size, base + ok * size, base + ov * size, projected.stride(0) if n > 1 else projected.shape[1],
+                                     code_of(projected.dtype), decay.data_ptr(), state.data_ptr(), state.stride(0), cu_q.data_ptr(),
+                                     row_slot.data_ptr(), raw.data_ptr(), n, n_rows, n_heads, head_dim, value_dim, int(act), stream_ptr()))
+
+
+def gated_rmsnorm(x: torch.Tensor, gain: Optional[torch.Tensor], eps: float, gate: Optional[torch.Tensor], out: torch.Tensor) -> None:
+    """``out = x / sqrt(mean(x^2) + eps) * gain * sigmoid(gate)`` over whole fp32 rows of ``x`` ``[n, dim]``; ``gate`` (``[n, dim]`` of ``out``'s
+    type, rows may lie in a wider buffer) and ``gain`` may be ``None``."""
+    _dev(x, gain, gate, out)
+    n, dim = x.shape
+    _need(x.dtype == torch.float32 and x.is_contiguous() and out.is_contiguous() and out.shape == x.shape, "gated_rmsnorm: x fp32 and out [n, dim]")
+    _need(gain is None or (gain.dtype == torch.float32 and gain.numel() == dim and gain.is_contiguous()), "gated_rmsnorm: gain fp32 [dim]")
+    _need(gate is None or (gate.dtype == out.dtype and gate.dim() == 2 and gate.stride(1) == 1 and gate.shape == x.shape),
+          "gated_rmsnorm: the gate must be [n, dim] of the output's type")
+    _check(lib().ka_gated_rmsnorm(x.data_ptr(), _ptr(gain), _ptr(gate), (gate.stride(0) if n > 1 else dim) if gate is not None else 0,
+                                  out.data_ptr(), code_of(out.dtype), n, dim, float(eps), stream_ptr()))
 
 
 def pair_embed(table: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor, token_row: torch.Tensor, cu_q: torch.Tensor,
@@ -716,12 +788,14 @@ def decayed_memory(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torc
 
 
 def route(logits: torch.Tensor, n_outputs: int, correction: Optional[torch.Tensor], top: int, n_groups: int, keep_groups: int,
-          scale: float, chosen: torch.Tensor, weights: torch.Tensor) -> None:
+          scale: float, chosen: torch.Tensor, weights: torch.Tensor, weigh_chosen: bool = False) -> None:
     """A router's choice per token from fp32 ``logits`` ``[n, >= n_outputs]``: scores = softmax over the first ``n_outputs``
     columns; the choice goes by scores + ``correction`` among the outputs of the ``keep_groups`` best of ``n_groups`` equal
     groups of neighbours (0 groups: among all); ``chosen`` int32 ``[n, top]``, ``weights`` fp32 ``[n, top]`` = the chosen scores
-    over their sum (+ 1e-20), times ``scale``."""
+    over their sum (+ 1e-20), times ``scale``. ``weigh_chosen``: the choice goes by the logits alone and the weights are the softmax
+    over the chosen logits, times ``scale`` (no groups, no correction)."""
     _dev(logits, correction, chosen, weights)
+    _need(not weigh_chosen or (n_groups == 0 and correction is None), "route: a choice by the logits alone has no groups and no correction")
     n = logits.shape[0]
     _need(logits.dtype == torch.float32 and logits.dim() == 2 and logits.stride(1) == 1 and logits.shape[1] >= n_outputs, "route: logits fp32 [n, >= outputs]")
     _need(correction is None or (correction.dtype == torch.float32 and correction.is_contiguous() and correction.numel() == n_outputs),
@@ -729,7 +803,7 @@ def route(logits: torch.Tensor, n_outputs: int, correction: Optional[torch.Tenso
     _need(chosen.dtype == torch.int32 and chosen.is_contiguous() and tuple(chosen.shape) == (n, top) and weights.dtype == torch.float32
           and weights.is_contiguous() and tuple(weights.shape) == (n, top), "route: chosen int32 and weights fp32 [n, top]")
     _check(lib().ka_route(logits.data_ptr(), logits.stride(0) if n > 1 else logits.shape[1], _ptr(correction), n, int(n_outputs), int(top),
-                          int(n_groups), int(keep_groups), float(scale), chosen.data_ptr(), weights.data_ptr(), stream_ptr()))
+                          int(n_groups), int(keep_groups), float(scale), int(bool(weigh_chosen)), chosen.data_ptr(), weights.data_ptr(), stream_ptr()))
 
 
 def experts_linear(a: torch.Tensor, per_token: int, weights: torch.Tensor, chosen: torch.Tensor, out: torch.Tensor, act: int = 0) -> None:
@@ -767,6 +841,26 @@ def experts_combine(y: torch.Tensor, h: torch.Tensor, chosen: torch.Tensor, weig
                                     weights.data_ptr(), n, top, int(n_experts), _ptr(shared), _ptr(shared_gate),
                                     (shared_gate.stride(0) if n > 1 else 1) if shared_gate is not None else 0, out.data_ptr(), dim,
                                     int(bool(accumulate)), stream_ptr()))
+
+
+def experts_combine_normed(y: torch.Tensor, h: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor, n_experts: int,
+                           shared: Optional[torch.Tensor], shared_gate: Optional[torch.Tensor], x: torch.Tensor, norm, then=None,
+                           rows: Optional[torch.Tensor] = None) -> None:
+    """The weighted sum of ``experts_combine`` as a ``delta`` of ``add_normed``: normalised and added into the fp32 stream ``x``, with
+    the norm ``then`` of the new rows into ``rows`` (of ``h``'s type), in one launch."""
+    _dev(y, h, chosen, weights, shared, shared_gate, x, rows)
+    n, dim = x.shape
+    top = chosen.shape[1]
+    who = "experts_combine_normed"
+    _need(y.dtype == torch.float32 and y.is_contiguous() and tuple(y.shape) == (n * top, dim), f"{who}: y fp32 [n top, dim]")
+    _need(h.dim() == 2 and tuple(h.shape) == (n, dim) and h.stride(1) == 1, f"{who}: h [n, dim]")
+    _need(shared is None or (shared.dtype == torch.float32 and shared.is_contiguous() and tuple(shared.shape) == (n, dim)), f"{who}: shared fp32 [n, dim]")
+    _need(shared_gate is None or (shared_gate.dtype == torch.float32 and shared_gate.dim() == 1 and shared_gate.numel() == n), f"{who}: the gate is an fp32 column")
+    _need(rows is None or rows.dtype == h.dtype, f"{who}: rows must be of the type of h")
+    _check(lib().ka_experts_combine_normed(y.data_ptr(), h.data_ptr(), h.stride(0) if n > 1 else dim, code_of(h.dtype), chosen.data_ptr(),
+                                           weights.data_ptr(), n, top, int(n_experts), _ptr(shared), _ptr(shared_gate),
+                                           (shared_gate.stride(0) if n > 1 else 1) if shared_gate is not None else 0, x.data_ptr(), dim,
+                                           *_norm_pair(who, x, norm, then, rows), stream_ptr()))
 
 
 def experts_sort(chosen: torch.Tensor, n_experts: int, tile: int, sorted_pairs: torch.Tensor, tile_expert: torch.Tensor) -> None:

@@ -68,6 +68,8 @@ _SIGNATURES = {
     "ka_matrix_memory_chunks_bf16": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                                      _c_void_p, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float,
                                      _c_void_p, _c_int, _c_void_p],
+    "ka_linear_chunks_bf16": [_c_void_p, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_void_p, _c_void_p,
+                              _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
     "ka_linear_skinny_norm_store": [_c_void_p, _c_void_p, _c_void_p, _c_float, _c_int, _c_void_p, _c_long, _c_void_p, _c_void_p,
                                     _c_int, _c_long, _c_int, _c_int, _c_int, _c_void_p, _c_long, _c_void_p],
 }
@@ -712,12 +714,15 @@ def attention_maps_bf16(q, k_cache, v_cache, block_table, token_row, kv_lo, kv_h
                                  head_dim, value_dim, None, None, None, batch, keep_first=keep_first, maps=maps)
 
 
-def attention_latent_bf16(q, cache, block_table, token_row, kv_hi, out, scale, n_heads, row_dim, rank, sinks, batch) -> bool:
+def attention_latent_bf16(q, cache, block_table, token_row, kv_hi, out, scale, n_heads, row_dim, rank, sinks, batch, kv_lo=None,
+                          head_gate=None) -> bool:
     """``n_heads`` query heads of ``row_dim`` channels over one cached row per key whose first ``rank`` channels are its
-    value, with a sink score per head, on the matrix cores (rows above 128 channels: the kernel's wide form). False: not
+    value, with a sink score per head (``sinks`` ``None``: no sinks), behind a window (``kv_lo``), times the sigmoid of one number
+    per head (``head_gate`` ``[n, H]``), on the matrix cores (rows above 128 channels: the kernel's wide form). False: not
     covered (rows that are no multiple of 16 channels among others)."""
-    return attention_biased_bf16(q, cache, None, block_table, token_row, None, kv_hi, out, scale, n_heads, 1, row_dim, rank,
-                                 None, None, None, batch, sinks=sinks, values_in_keys=True)
+    return attention_biased_bf16(q, cache, None, block_table, token_row, kv_lo, kv_hi, out, scale, n_heads, 1, row_dim, rank,
+                                 None, None, None, batch, sinks=sinks, values_in_keys=True, gate=head_gate,
+                                 gate_per_head=head_gate is not None)
 
 
 def heads_linear_bf16(a, a_head: int, k: int, weights, out, out_head: int, n_out: int, gate=None) -> bool:
@@ -785,11 +790,52 @@ def matrix_memory_chunks_bf16(projected, offsets, pre, state, cu_q, row_slot, ga
     return True
 
 
+def linear_attention_chunks_scratch(n: int, n_rows: int, n_heads: int, head_dim: int, value_dim: int) -> int:
+    """fp32 numbers of scratch that ``linear_attention_chunks_bf16`` needs for a step of ``n`` tokens in ``n_rows`` rows; 0: the
+    kernels do not cover the head sizes."""
+    handle = lib()
+    handle.ka_linear_chunks_scratch.restype = ctypes.c_long
+    if not handle.ka_linear_chunks_supported(int(head_dim), int(value_dim)):
+        return 0
+    return int(handle.ka_linear_chunks_scratch(int(n), int(n_rows), int(n_heads), int(head_dim), int(value_dim)))
+
+
+def linear_attention_chunks_bf16(projected, offsets, log2_decay, state, cu_q, row_slot, raw, n_heads, head_dim, value_dim, act, scratch) -> bool:
+    """``ops.core.linear_attention`` for prompt portions on the matrix cores: the recurrence unrolled over chunks of 64 tokens, all
+    chunks at once in three launches (operands as there, with the decays' logarithms to base 2; ``scratch``: contiguous fp32 of
+    at least ``linear_attention_chunks_scratch`` numbers). False: sizes or alignment not covered, nothing was run."""
+    handle = lib()
+    n = projected.shape[0]
+    if n == 0:
+        return True
+    n_rows = int(row_slot.numel())
+    if projected.dtype != torch.bfloat16 or not handle.ka_linear_chunks_supported(int(head_dim), int(value_dim)):
+        return False
+    oq, ok, ov = (int(o) for o in offsets)
+    size, base = projected.element_size(), projected.data_ptr()
+    stride = projected.stride(0) if n > 1 else projected.shape[1]
+    if base % 16 or stride % 8 or any(o % 8 for o in (oq, ok, ov)) or projected.stride(1) != 1 or state.stride(0) % 4 \
+            or n // 64 + n_rows > 65535:
+        return False
+    need = linear_attention_chunks_scratch(n, n_rows, n_heads, head_dim, value_dim)
+    for t, numbers, what in ((scratch, need, "scratch"), (raw, n * n_heads * value_dim, "read-outs"), (log2_decay, n_heads, "decays")):
+        if t.dtype != torch.float32 or not t.is_contiguous() or t.numel() < numbers or not t.is_cuda:
+            raise KernelError(f"linear attention: the {what} must be contiguous fp32 of at least {numbers} numbers")
+    if max(oq + n_heads * head_dim, ok + n_heads * head_dim, ov + n_heads * value_dim) > projected.shape[1] \
+            or state.dtype != torch.float32 or state.shape[1] != n_heads * head_dim * value_dim \
+            or cu_q.dtype != torch.int32 or cu_q.numel() != n_rows + 1 or row_slot.dtype != torch.int32:
+        raise KernelError("linear attention: operands do not fit the head sizes")
+    _check(handle.ka_linear_chunks_bf16(base + oq * size, base + ok * size, base + ov * size, stride, log2_decay.data_ptr(), state.data_ptr(),
+                                        state.stride(0), cu_q.data_ptr(), row_slot.data_ptr(), raw.data_ptr(), scratch.data_ptr(), n, n_rows,
+                                        n_heads, head_dim, value_dim, int(act), stream_ptr()))
+    return True
+
+
 def experts_feed_forward_bf16(h, pairs, down, chosen, hidden, y, act, workspace) -> bool:
     """Both linears of the chosen experts for all pairs of a step on the matrix cores, an expert's pairs together: the pairs
-    are listed by expert (``ops.core.experts_sort``), the gated first linear gathers every pair's token from ``h`` ``[n, dim]`` and
+    are listed by expert (``ops.core.experts_sort``), the first linear (gated or not, as ``act`` says) gathers every pair's token from ``h`` ``[n, dim]`` and
     leaves the hidden rows in list order, the second writes fp32 ``y`` ``[n top, dim]`` at the pairs' own rows. ``pairs``
-    ``[E, 2 hidden, dim]``, ``down`` ``[E, dim, hidden]``, ``chosen`` int32 ``[n, top]``; ``hidden`` is not used (the list's hidden rows
+    ``[E, 2 hidden, dim]`` (not gated: ``[E, hidden, dim]``), ``down`` ``[E, dim, hidden]``, ``chosen`` int32 ``[n, top]``; ``hidden`` is not used (the list's hidden rows
     live in the workspace). False: not covered (sizes that are no multiple of 16, alignment), nothing was run."""
     from . import core
     n, top = chosen.shape
@@ -801,8 +847,10 @@ def experts_feed_forward_bf16(h, pairs, down, chosen, hidden, y, act, workspace)
             or h.data_ptr() % 16 or pairs.data_ptr() % 16 or down.data_ptr() % 16 or y.data_ptr() % 16:
         return False
     lda = h.stride(0) if n > 1 else dim
-    gated = int(act) | ACT_GATED
-    if not handle.ka_experts_gemm_supported(lda, n_pair_rows, dim, ff, gated, 0) or not handle.ka_experts_gemm_supported(ff, dim, ff, dim, 0, 1):
+    act = int(act)
+    if n_pair_rows != (2 * ff if act & ACT_GATED else ff):
+        raise KernelError("experts: the first linear's rows do not fit the hidden size")
+    if not handle.ka_experts_gemm_supported(lda, n_pair_rows, dim, ff, act, 0) or not handle.ka_experts_gemm_supported(ff, dim, ff, dim, 0, 1):
         return False
     tile = int(handle.ka_experts_gemm_tile())
     # (sized by the step's tokens alone: the same for every replay of a captured step)
@@ -814,7 +862,7 @@ def experts_feed_forward_bf16(h, pairs, down, chosen, hidden, y, act, workspace)
     rows = workspace.get("experts.hidden_listed", (capacity, ff), torch.bfloat16)
     core.experts_sort(chosen.view(-1), n_experts, tile, listed, tile_expert)
     _check(handle.ka_experts_gemm_bf16(h.data_ptr(), lda, top, pairs.data_ptr(), listed.data_ptr(), tile_expert.data_ptr(), capacity // tile,
-                                       n_pair_rows, dim, gated, rows.data_ptr(), ff, 0, 0, stream_ptr()))
+                                       n_pair_rows, dim, act, rows.data_ptr(), ff, 0, 0, stream_ptr()))
     _check(handle.ka_experts_gemm_bf16(rows.data_ptr(), ff, 0, down.data_ptr(), listed.data_ptr(), tile_expert.data_ptr(), capacity // tile,
                                        dim, ff, 0, y.data_ptr(), dim, 1, 1, stream_ptr()))
     return True

@@ -287,8 +287,70 @@ def _output_norms(block: "Block", x, batch, cache) -> None:
         add(block.norm2)
 
 
+def _add_normed(norm, delta, x, then, rows, ws) -> bool:
+    """``x += norm(delta)``, and the norm ``then`` of the new rows of the stream into ``rows``, in one launch where both are
+    root-mean-square norms (returns whether ``rows`` was written)."""
+    from ..ops import core
+
+    first = norm.rms_operands() if callable(getattr(norm, "rms_operands", None)) else None
+    if first is None:
+        if callable(getattr(norm, "add_normed", None)):
+            norm.add_normed(delta, x)
+        else:
+            normed = ws.get("block.normed", tuple(x.shape), torch.float32)
+            norm.forward(delta, normed)
+            core.add_scaled(x, normed, 1.0)
+        return False
+    second = then.rms_operands() if then is not None and callable(getattr(then, "rms_operands", None)) else None
+    core.add_normed(x, delta, first, second, rows if second is not None else None)
+    return second is not None
+
+
+def _norms_around(block: "Block", x, batch, cache, normed=None, then=None):
+    """``x += norm_after(mixer(norm(x))); x += norm2_after(ff(norm2(x)))``: a norm before and behind each sublayer.
+
+    A sublayer writes its output into an fp32 buffer (``mix``); one launch then normalises it, adds it into the stream
+    and computes the norm that the next reader of the stream begins with: ``norm2`` behind the mixer, and behind the
+    feed-forward the first norm of the block that follows (``then``), whose rows are handed over. A feed-forward that
+    offers ``mix_normed`` takes that launch's work into its own last one."""
+    ws = batch.workspace
+    ff = block.feed_forward
+    delta = ws.get("block.delta", tuple(x.shape), torch.float32)
+    h = normed
+    if h is None:
+        h = ws.get("block.h", tuple(x.shape), block.dtype)
+        block.norm.forward(x, h)
+
+    def into_delta(part, *operands):
+        if callable(getattr(part, "mix", None)):
+            part.mix(*operands, delta, False)
+        else:
+            delta.zero_()
+            part.forward(*operands, delta)
+
+    into_delta(block.mixer, h, batch, cache)
+    handed = ws.get("block.handed", tuple(x.shape), block.dtype)
+    if ff is None:
+        return handed if _add_normed(block.norm_after, delta, x, then, handed, ws) else None
+    h = ws.get("block.h2", tuple(x.shape), block.dtype)
+    if not _add_normed(block.norm_after, delta, x, block.norm2, h, ws):
+        block.norm2.forward(x, h)
+    if callable(getattr(ff, "mix_normed", None)):
+        first = block.norm2_after.rms_operands() if callable(getattr(block.norm2_after, "rms_operands", None)) else None
+        second = then.rms_operands() if then is not None and callable(getattr(then, "rms_operands", None)) else None
+        if first is not None:
+            ff.mix_normed(h, batch, x, first, second, handed if second is not None else None)
+            return handed if second is not None else None
+    into_delta(ff, h, batch)
+    return handed if _add_normed(block.norm2_after, delta, x, then, handed, ws) else None
+
+
+_norms_around.hands_over = True
+
+
 ARRANGEMENTS: Dict[str, Callable] = {"parallel": _parallel, "sequential": _sequential,
-                                     "parallel_two_norms": _parallel_two_norms, "output_norms": _output_norms}
+                                     "parallel_two_norms": _parallel_two_norms, "output_norms": _output_norms,
+                                     "norms_around": _norms_around}
 
 
 def register_arrangement(name: str, fn: Callable) -> None:
@@ -311,10 +373,16 @@ class Block:
         self.norm2 = build_part("norm", spec.norm2) if spec.norm2 is not None else None
         if spec.arrangement == "sequential" and self.norm2 is None and spec.feed_forward is not None:
             raise ValueError("the sequential arrangement needs norm2 for its feed-forward")
+        self.norm_after = build_part("norm", spec.norm_after) if getattr(spec, "norm_after", None) is not None else None
+        self.norm2_after = build_part("norm", spec.norm2_after) if getattr(spec, "norm2_after", None) is not None else None
+        if spec.arrangement == "norms_around" and (self.norm_after is None or (
+                spec.feed_forward is not None and (self.norm2 is None or self.norm2_after is None))):
+            raise ValueError("the norms_around arrangement needs norm_after, and norm2 and norm2_after for its feed-forward")
         self.mixer = build_part("mixer", spec.mixer)
         if spec.arrangement == "output_norms" and self.norm2 is None and spec.feed_forward is not None:
             raise ValueError("the output_norms arrangement needs norm2 for its feed-forward")
-        if spec.feed_forward is None and spec.arrangement not in ("parallel_two_norms", "parallel", "sequential", "output_norms"):
+        if spec.feed_forward is None and spec.arrangement not in ("parallel_two_norms", "parallel", "sequential", "output_norms",
+                                                                          "norms_around"):
             raise ValueError(f"the {spec.arrangement} arrangement needs a feed-forward")
         if spec.arrangement == "parallel_two_norms" and spec.feed_forward is not None and self.norm2 is None:
             raise ValueError("the parallel_two_norms arrangement needs norm2 for its feed-forward")
@@ -328,6 +396,10 @@ class Block:
             out["feed_forward"] = self.feed_forward
         if self.norm2 is not None:
             out["norm2"] = self.norm2
+        if self.norm_after is not None:
+            out["norm_after"] = self.norm_after
+        if self.norm2_after is not None:
+            out["norm2_after"] = self.norm2_after
         return out
 
     def params(self) -> Dict[str, ParamSpec]:

@@ -47,7 +47,8 @@ class ConcatLinear(Junction):
 
 class PassVector(Junction):
     """``x <- x + steps[passage]``: a learned vector per passage through the junction, ``steps`` ``[passages, dim]``, added
-    to every token's row of the fp32 stream."""
+    to every token's row of the fp32 stream; from the passage ``spec.embedding_from`` on, the embedding output as well
+    (kept in fp32 from the start of the step)."""
 
     replays_every_step = True
 
@@ -61,10 +62,19 @@ class PassVector(Junction):
     def bind(self, tensors, dtype, device) -> None:
         self.steps = tensors["steps"].to(device).contiguous()
 
+    def _kept(self, x, batch) -> torch.Tensor:
+        return batch.workspace.get("junction.embedding", tuple(x.shape), torch.float32)
+
+    def begin(self, x, batch) -> None:
+        start = getattr(self.spec, "embedding_from", None)
+        if start is not None and start < self.spec.passages:
+            core.cast_columns(x, self._kept(x, batch))
+
     def forward(self, x, batch, passage: int = 0) -> None:
         if not 0 <= passage < self.spec.passages:
             raise ValueError(f"passage {passage} through a junction of {self.spec.passages} vectors")
-        core.add_vector(x, self.steps[passage])
+        start = getattr(self.spec, "embedding_from", None)
+        core.add_vector(x, self.steps[passage], self._kept(x, batch) if start is not None and passage >= start else None)
 
 
 register_junction("concat_linear", ConcatLinear)

@@ -21,6 +21,10 @@ class LatentAttention(Mixer):
         score = scale * (q_plain . W_uk,h c + rot(q_rot) . rot(k_r)),   softmax over j <= i with exp(sink_h) in the denominator
         out = W_o (concat_h(sum_j w_j v_h,j) * sigmoid(W_g h))
 
+    Forms, each by its field of the specification: queries projected directly, ``q = W_q h`` (``q_rank`` ``None``); no rotated
+    part (``rot_dim`` 0); a window, so that ``j`` is seen while ``i - j < window`` and pages behind it go back; no sinks; no gate,
+    or a gate of one number per head (it rides in the attention kernel, where it multiplies the weighted latents).
+
     Only ``[c | rot(k_r)]`` is cached, one row of ``kv_rank + dr`` channels per token (``LatentCacheSpec``). The per-head
     up-projections are moved to the query's side: ``q_plain . W_uk,h c = (W_uk,h^T q_plain) . c``, so every head's query
     becomes ``[W_uk,h^T q_plain | rot(q_rot)]`` against the cached row, and ``sum_j w_j W_uv,h c_j = W_uv,h sum_j w_j c_j``,
@@ -38,7 +42,14 @@ class LatentAttention(Mixer):
         self.row_dim = spec.kv_rank + spec.rot_dim              # a cached row, and a query head as the kernel sees it
         self.out_dim = spec.n_heads * spec.value_dim
         self.gated = bool(spec.output_gate)
-        self.down_dim = spec.q_rank + self.row_dim + (self.out_dim if self.gated else 0)
+        self.gate_per_head = self.gated and bool(getattr(spec, "gate_per_head", False))
+        self.gate_dim = (spec.n_heads if self.gate_per_head else self.out_dim) if self.gated else 0
+        self.window = getattr(spec, "window", None)
+        self.q_latent = spec.q_rank is not None
+        self.q_cols = spec.q_rank if self.q_latent else self.q_dim      # columns of the first linear that the queries come from
+        used = self.q_cols + self.row_dim + self.gate_dim
+        # (rows of the projected buffer start on multiples of 16 bytes: what is missing is filled with weight rows of zeros)
+        self.down_dim = used if self.gate_dim == self.out_dim else -(-used // 8) * 8
         self.down_weight = self.uq_weight = self.absorb = self.lift = self.proj_weight = None
         self._q_gain = self._kv_gain = self._sinks = self._freqs = None
         self._pairing = "halves"
@@ -46,32 +57,41 @@ class LatentAttention(Mixer):
 
     def params(self) -> Dict[str, ParamSpec]:
         spec = self.spec
-        out = {"dq.weight": ParamSpec((spec.q_rank, spec.dim)), "dq_norm.weight": ParamSpec((spec.q_rank,), "vector", "gain"),
-               "uq.weight": ParamSpec((self.q_dim, spec.q_rank)), "dkv.weight": ParamSpec((self.row_dim, spec.dim)),
+        if self.q_latent:
+            out = {"dq.weight": ParamSpec((spec.q_rank, spec.dim)), "dq_norm.weight": ParamSpec((spec.q_rank,), "vector", "gain"),
+                   "uq.weight": ParamSpec((self.q_dim, spec.q_rank))}
+        else:
+            out = {"q.weight": ParamSpec((self.q_dim, spec.dim))}
+        out.update({"dkv.weight": ParamSpec((self.row_dim, spec.dim)),
                "dkv_norm.weight": ParamSpec((spec.kv_rank,), "vector", "gain"),
                "uk.weight": ParamSpec((spec.n_heads * spec.head_dim, spec.kv_rank)),
-               "uv.weight": ParamSpec((self.out_dim, spec.kv_rank)), "proj.weight": ParamSpec((spec.dim, self.out_dim))}
+               "uv.weight": ParamSpec((self.out_dim, spec.kv_rank)), "proj.weight": ParamSpec((spec.dim, self.out_dim))})
         if spec.head_sinks:
             out["sink"] = ParamSpec((spec.n_heads,), "vector", "bias")
         if self.gated:
-            out["gate.weight"] = ParamSpec((self.out_dim, spec.dim))
+            out["gate.weight"] = ParamSpec((self.gate_dim, spec.dim))
         return out
 
     def cache_spec(self) -> LatentCacheSpec:
-        return LatentCacheSpec(self.spec.kv_rank, self.spec.rot_dim)
+        return LatentCacheSpec(self.spec.kv_rank, self.spec.rot_dim, self.window)
 
     def bind(self, tensors, dtype, device) -> None:
         spec = self.spec
         self.dtype = dtype
-        names = ["dq.weight", "dkv.weight"] + (["gate.weight"] if self.gated else [])
-        # one launch projects the query latent, the key/value latent with the shared key part, and the gate
-        self.down_weight = torch.cat([tensors[name].to(device) for name in names], dim=0).contiguous()
-        self.uq_weight = tensors["uq.weight"].to(device).contiguous()
+        names = ["dq.weight" if self.q_latent else "q.weight", "dkv.weight"] + (["gate.weight"] if self.gated else [])
+        # one launch projects the queries or their latent, the key/value latent with the shared key part, and the gate
+        rows = [tensors[name].to(device) for name in names]
+        missing = self.down_dim - sum(r.shape[0] for r in rows)
+        if missing:
+            rows.append(torch.zeros((missing, spec.dim), dtype=rows[0].dtype, device=device))
+        self.down_weight = torch.cat(rows, dim=0).contiguous()
+        if self.q_latent:
+            self.uq_weight = tensors["uq.weight"].to(device).contiguous()
+            self._q_gain = tensors["dq_norm.weight"].to(device=device, dtype=torch.float32).contiguous()
         # W_uk per head, transposed: [H, kv_rank, hd] (a linear's weight for q_plain -> latent space)
         self.absorb = tensors["uk.weight"].to(device).view(spec.n_heads, spec.head_dim, spec.kv_rank).transpose(1, 2).contiguous()
         self.lift = tensors["uv.weight"].to(device).view(spec.n_heads, spec.value_dim, spec.kv_rank).contiguous()
         self.proj_weight = tensors["proj.weight"].to(device).contiguous()
-        self._q_gain = tensors["dq_norm.weight"].to(device=device, dtype=torch.float32).contiguous()
         self._kv_gain = tensors["dkv_norm.weight"].to(device=device, dtype=torch.float32).contiguous()
         if spec.head_sinks:
             self._sinks = tensors["sink"].to(device=device, dtype=torch.float32).contiguous()
@@ -98,32 +118,41 @@ class LatentAttention(Mixer):
         return self.proj_weight, None
 
     def attend(self, down, batch, cache: LayerCache, beside=None) -> torch.Tensor:
-        """From the projected row ``[c_q' | c' | k_r | gate]`` to the gated heads, the input of the output projection."""
+        """From the projected row ``[c_q' or q | c' | k_r | gate]`` to the gated heads, the input of the output projection."""
         spec = self.spec
         n = down.shape[0]
         ws = batch.workspace
         group = batch.groups[cache.group]
         slots = group.slots if cache.writes else None
-        cq = ws.get("latent.cq", (n, spec.q_rank), self.dtype)
-        core.latent_prepare(down, 0, spec.q_rank, self._q_gain, cq, spec.q_rank, spec.kv_rank, self._kv_gain, spec.rot_dim,
-                            self._freqs, self._pairing, batch.positions, slots, cache.k, spec.eps)
-        q = ws.get("latent.q", (n, self.q_dim), self.dtype)
-        linear(cq, self.uq_weight, None, q)
+        cq = ws.get("latent.cq", (n, spec.q_rank), self.dtype) if self.q_latent else None
+        core.latent_prepare(down, 0, spec.q_rank if self.q_latent else 0, self._q_gain, cq, self.q_cols, spec.kv_rank, self._kv_gain,
+                            spec.rot_dim, self._freqs, self._pairing, batch.positions, slots, cache.k, spec.eps)
+        if self.q_latent:
+            q = ws.get("latent.q", (n, self.q_dim), self.dtype)
+            linear(cq, self.uq_weight, None, q)
+        else:
+            q = down[:, :self.q_dim]
         full = ws.get("latent.q_full", (n, spec.n_heads * self.row_dim), self.dtype)
-        core.rotate_tail(q, full, spec.n_heads, spec.head_dim, spec.rot_dim, spec.kv_rank, self._freqs, self._pairing, batch.positions)
+        if spec.rot_dim:
+            core.rotate_tail(q, full, spec.n_heads, spec.head_dim, spec.rot_dim, spec.kv_rank, self._freqs, self._pairing, batch.positions)
         self._per_head(q, self.q_head, spec.head_dim, self.absorb, full, self.row_dim, spec.kv_rank)
         mixed = ws.get("latent.mixed", (n, spec.n_heads * spec.kv_rank), self.dtype)
-        gate = down[:, spec.q_rank + self.row_dim:] if self.gated else None
+        gate_at = self.q_cols + self.row_dim
+        gate = down[:, gate_at:gate_at + self.gate_dim] if self.gated else None
+        # (a number per head scales a head's weighted latents as well as its values: the attention kernel applies it)
+        inside = gate if self.gate_per_head else None
+        kv_lo = group.kv_lo if self.window is not None else None
         done = False
         if self.dtype == torch.bfloat16:
             from ..ops import fast
             done = fast.attention_latent_bf16(full, cache.k, group.block_table, batch.token_row, batch.kv_hi, mixed, float(spec.scale),
-                                              spec.n_heads, self.row_dim, spec.kv_rank, self._sinks, batch)
+                                              spec.n_heads, self.row_dim, spec.kv_rank, self._sinks, batch, kv_lo=kv_lo, head_gate=inside)
         if not done:
             core.attention_generic(full, cache.k, None, group.block_table, batch.token_row, group.kv_lo, batch.kv_hi, mixed,
                                    float(spec.scale), spec.n_heads, 1, self.row_dim, spec.kv_rank, sinks=self._sinks,
-                                   values_in_keys=True)
+                                   values_in_keys=True, gate=inside, gate_per_head=inside is not None)
         heads = ws.get("latent.heads", (n, self.out_dim), self.dtype)
+        gate = None if self.gate_per_head else gate
         if not self._per_head(mixed, spec.kv_rank, spec.kv_rank, self.lift, heads, spec.value_dim, spec.value_dim, gate) \
                 and gate is not None:
             core.gate_mul(heads, gate)

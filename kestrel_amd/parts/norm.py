@@ -46,7 +46,8 @@ class LayerNorm(Norm):
 class RMSNorm(Norm):
     """``x / sqrt(mean(x^2) + eps) * (offset + weight)`` over the last axis: no mean is taken off, no shift is added;
     ``spec.offset`` is 0 for a weight used as stored and 1 for one stored around zero (added once, in fp32, when the
-    weights are bound). It offers no ``layernorm_operands`` (it is no LayerNorm), but
+    weights are bound); with ``spec.scaled`` a second vector (tensor ``scale``) multiplies the result, folded into the
+    weight in fp32 when the weights are bound. It offers no ``layernorm_operands`` (it is no LayerNorm), but
     ``rms_operands``: the weight-streaming linears of a few rows take it into their launch as they take a LayerNorm."""
 
     replays_every_step = True
@@ -57,10 +58,16 @@ class RMSNorm(Norm):
 
     def params(self) -> Dict[str, ParamSpec]:
         around_zero = float(getattr(self.spec, "offset", 0.0)) != 0.0
-        return {"weight": ParamSpec((self.spec.dim,), "vector", "shift" if around_zero else "gain")}
+        out = {"weight": ParamSpec((self.spec.dim,), "vector", "shift" if around_zero else "gain")}
+        if getattr(self.spec, "scaled", False):
+            out["scale"] = ParamSpec((self.spec.dim,), "vector", "gain")
+        return out
 
     def bind(self, tensors, dtype, device) -> None:
-        self.weight = (tensors["weight"].to(device=device, dtype=torch.float32) + float(getattr(self.spec, "offset", 0.0))).contiguous()
+        weight = tensors["weight"].to(device=device, dtype=torch.float32) + float(getattr(self.spec, "offset", 0.0))
+        if getattr(self.spec, "scaled", False):
+            weight = weight * tensors["scale"].to(device=device, dtype=torch.float32)
+        self.weight = weight.contiguous()
 
     def forward(self, x, out, rows=None) -> None:
         core.rmsnorm(x, self.weight, self.spec.eps, out, rows)

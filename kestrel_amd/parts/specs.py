@@ -32,13 +32,16 @@ class ParamSpec:
 
 @dataclass(frozen=True)
 class NormSpec:
-    """``offset``: what is added to the stored weight before it multiplies (1.0 for a weight stored around zero)."""
+    """``offset``: what is added to the stored weight before it multiplies (1.0 for a weight stored around zero).
+    ``scaled``: a second vector (tensor ``scale``) multiplies the result channel by channel: the layer scale of a sublayer
+    whose output this norm stands behind."""
 
     kind: str
     dim: int
     eps: float
     bias: bool = True
     offset: float = 0.0
+    scaled: bool = False
 
 
 @dataclass(frozen=True)
@@ -333,11 +336,14 @@ class DifferentialAttentionSpec:
 @dataclass(frozen=True)
 class LatentAttentionSpec:
     """Attention whose queries, keys and values come from low-rank latents: ``c_q = rms(W_dq h) g_q`` (``q_rank``),
-    ``q = W_uq c_q`` laid out per head as ``[head_dim plain, rot_dim rotated]``; ``W_dkv h`` gives the latent ``c`` (``kv_rank``,
-    normalised with gains) and ``rot_dim`` channels of one rotated key part shared by all heads; a head's plain keys are
-    ``W_uk c`` and its values ``W_uv c``. Every ``j <= i`` is seen. ``head_sinks``: one learned score per head that enters the
+    ``q = W_uq c_q`` laid out per head as ``[head_dim plain, rot_dim rotated]`` (``q_rank`` ``None``: ``q = W_q h``, no latent of
+    queries); ``W_dkv h`` gives the latent ``c`` (``kv_rank``,
+    normalised with gains) and ``rot_dim`` channels of one rotated key part shared by all heads (0: there is none, and
+    nothing knows a position); a head's plain keys are
+    ``W_uk c`` and its values ``W_uv c``. ``window`` ``None``: every ``j <= i`` is seen, else the ``window`` latest.
+    ``head_sinks``: one learned score per head that enters the
     softmax's denominator without a value. ``output_gate``: the heads times ``sigmoid(W_g h)`` before the output
-    projection. ``position`` turns the ``rot_dim`` part."""
+    projection (``gate_per_head``: one number per head instead of one per channel). ``position`` turns the ``rot_dim`` part."""
 
     kind: str
     dim: int
@@ -345,13 +351,15 @@ class LatentAttentionSpec:
     head_dim: int
     rot_dim: int
     value_dim: int
-    q_rank: int
+    q_rank: Optional[int]
     kv_rank: int
     scale: float
     eps: float
     position: PositionSpec
     head_sinks: bool = True
     output_gate: bool = True
+    gate_per_head: bool = False
+    window: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -384,11 +392,13 @@ class PairEmbeddingSpec:
 @dataclass(frozen=True)
 class PassVectorSpec:
     """A junction that adds a learned vector to the stream, one vector per passage (``[passages, dim]``;
-    ``ScheduleEntry.passage`` says which)."""
+    ``ScheduleEntry.passage`` says which). ``embedding_from``: from this passage on the embedding output is added too
+    (``None``: never)."""
 
     kind: str
     dim: int
     passages: int
+    embedding_from: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -421,7 +431,10 @@ class RoutedExpertsSpec:
     neighbours, a group counts by its largest choice score, and only outputs of the ``keep_groups`` best groups can be
     chosen. The last ``n_identity`` outputs are experts without tensors whose output is the input itself.
     ``shared_hidden``: a further expert of that hidden size that every token uses, times ``sigmoid(shared.sg h)`` (one
-    number per token) if ``shared_gate``."""
+    number per token) if ``shared_gate``. ``gated`` ``False``: the experts are plain, ``down(act(up h))``.
+    ``weigh_chosen``: choice and weights go by the logits alone, ``router h`` plus a stored bias (tensor ``router.bias``): the
+    ``top`` largest are chosen and their weights are the softmax over the chosen logits (times ``scale``); there is no
+    ``correction``."""
 
     kind: str
     dim: int
@@ -435,6 +448,26 @@ class RoutedExpertsSpec:
     activation: str = "silu"
     shared_hidden: Optional[int] = None
     shared_gate: bool = True
+    gated: bool = True
+    weigh_chosen: bool = False
+
+
+@dataclass(frozen=True)
+class LinearAttentionSpec:
+    """Attention without a softmax, as a recurrence: per head a state ``S`` ``[head_dim, value_dim]``, ``S <- decay_h S + k v^T``,
+    read as ``S^T q``, with queries, keys and values through ``activation`` and ``decay`` one constant per head; the
+    concatenated heads are normalised together (``eps``, gains), times ``sigmoid(W_g h)`` if ``output_gate``
+    (``parts/linear_attention.py``)."""
+
+    kind: str
+    dim: int
+    n_heads: int
+    head_dim: int
+    value_dim: int
+    decay: Tuple[float, ...]
+    eps: float
+    activation: str = "silu"
+    output_gate: bool = True
 
 
 @dataclass(frozen=True)
@@ -488,8 +521,10 @@ class LayerSpec:
     (``feed_forward`` and ``norm2`` may be ``None`` there: a layer of a mixer alone).
     ``output_norms`` = ``x += norm(mixer(x)); x += norm2(ff(x))``: the parts read the stream itself and the norms stand
     behind them (``feed_forward`` and ``norm2`` may be ``None``).
-    ``names`` maps ``"<part>.<local tensor name>"`` (parts: ``norm``, ``norm2``, ``mixer``,
-    ``feed_forward``) to the tensor's name in the checkpoint.
+    ``norms_around`` = ``x += norm_after(mixer(norm(x))); x += norm2_after(ff(norm2(x)))`` (``feed_forward``, ``norm2`` and
+    ``norm2_after`` may be ``None``).
+    ``names`` maps ``"<part>.<local tensor name>"`` (parts: ``norm``, ``norm2``, ``norm_after``,
+    ``norm2_after``, ``mixer``, ``feed_forward``) to the tensor's name in the checkpoint.
     """
 
     arrangement: str
@@ -499,6 +534,8 @@ class LayerSpec:
     norm2: Optional[object] = None
     names: Mapping[str, str] = field(default_factory=dict)
     residual_scale: float = 1.0        # weight of the branches' sum in arrangements that have one
+    norm_after: Optional[object] = None
+    norm2_after: Optional[object] = None
 
 
 @dataclass(frozen=True)
@@ -539,6 +576,8 @@ class ModelPlan:
     # encoding): its ``add_to_embeddings`` runs on the embedded tokens before the first block; its tensors
     # are named by ``names["position.<local name>"]``. ``None``: positions are the mixers' business.
     position: Optional[object] = None
+    # a norm of the embedded tokens before anything else sees them (tensors ``names["embedding_norm.<local name>"]``)
+    embedding_norm: Optional[object] = None
     # junctions by name: specifications whose parts (registered as junctions) transform the residual stream between
     # runs of layers, where a schedule entry names one (``ScheduleEntry.before``); a junction named by several
     # entries runs with the same tensors each time; its tensors are named by ``names["junction.<name>.<local name>"]``

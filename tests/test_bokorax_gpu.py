@@ -285,7 +285,7 @@ def test_experts_linears_and_sum(dtype, n, dim, ff, n_experts, top):
     if dtype == torch.bfloat16 and dim % 16 == 0 and ff % 16 == 0:
         from kestrel_amd.engine.batch import Workspace
         y2 = torch.full((n * top, dim), float("nan"), device=DEV)
-        assert fast.experts_feed_forward_bf16(h.to(DEV), pairs, down.to(DEV), chosen.to(DEV), None, y2, act, Workspace(torch.device(DEV)))
+        assert fast.experts_feed_forward_bf16(h.to(DEV), pairs, down.to(DEV), chosen.to(DEV), None, y2, act | ACT_GATED, Workspace(torch.device(DEV)))
         live = (chosen < n_experts).view(-1)
         _near(y2[live.to(DEV)], y[live.to(DEV)], dtype, "by expert against pair by pair", atol=1e-2, rtol=2e-2)
 
