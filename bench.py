@@ -22,7 +22,9 @@ feed-forward, heads, head size, runs of layers, vocabulary; random weights): a p
 layer of chunked attention beside a matrix memory) at sizes of its own (``BOGIVIK_SIZES``), and
 ``--workload compare-bokorax`` for the Bokorax design (two kinds of attention, a decaying matrix memory, routed experts),
 ``--workload compare-letevik`` for the Letevik design (differential attention behind short convolutions and latent
-attention in a looped stretch of layers; ``LETEVIK_SIZES``).
+attention in a looped stretch of layers; ``LETEVIK_SIZES``), and ``--workload compare-vufolorn`` for the Vufolorn design (a
+linear recurrence with a decay per head, windowed latent attention, routed plain experts; ``VUFOLORN_SIZES``), which also
+has Bokorax, the design closest to it, beside it.
 """
 
 from __future__ import annotations
@@ -248,8 +250,9 @@ def design_facts(net):
         elif kind == "latent_attention":
             # per head a score over the plain and the rotated part and a value product; the cache holds the latent and
             # the shared rotated key part
-            attention.append((spec.n_heads * (spec.head_dim + spec.rot_dim + spec.value_dim), spec.kv_rank + spec.rot_dim, None, None, 0))
-        elif kind == "matrix_memory":
+            attention.append((spec.n_heads * (spec.head_dim + spec.rot_dim + spec.value_dim), spec.kv_rank + spec.rot_dim,
+                              getattr(spec, "window", None), None, 0))
+        elif kind in ("matrix_memory", "linear_attention"):
             memory.append((spec.n_heads, spec.head_dim, spec.value_dim))
         elif kind == "decayed_memory":
             memory.append((spec.n_heads, spec.head_dim, spec.head_dim))
@@ -263,7 +266,7 @@ def design_facts(net):
         if getattr(ff, "kind", None) == "routed_experts":
             # routed experts: a token multiplies with `top` of them, and a step reads those that its tokens chose; they are
             # counted apart from the weights that every token uses
-            size = 3 * ff.dim * ff.hidden_dim
+            size = (3 if getattr(ff, "gated", True) else 2) * ff.dim * ff.hidden_dim
             experts.append((ff.n_experts, ff.top, size))
             linear -= ff.n_experts * size
     return SimpleNamespace(linear=linear, attention=attention, memory=memory, experts=experts, width=plan.dim, vocab=plan.vocab_size)
@@ -389,6 +392,43 @@ def bokorax_models(size: dict, positions: int):
                           "max_context": positions, "n_heads": h, "n_kv_heads": g, "head_dim": d, "rotary_dim": d // 2,
                           "rope_theta": 10000.0, "prefix_attn": 0, "layer_norm_eps": 1e-5}}
     return {"bokorax": (bokorax, "bokorax"), "moondream2": (moondream, "moondream2")}
+
+
+# Sizes at which Vufolorn is measured beside Bokorax, the design that is closest to it (a recurrence, windowed attention,
+# routed experts), and beside the Moondream decoder: width, the recurrence's heads and head size (keys and values), the
+# latent layers' heads, head size (keys and values), latent size and window, the routed experts (how many, their hidden
+# size, choices per token, the shared expert) and the order of layers (r: recurrence, a: latent attention). Bokorax gets a
+# decaying memory of as many channels for every r and windowed attention over `kv_heads` kv heads for every a, and gated
+# experts of two thirds of the hidden size: the same weights.
+VUFOLORN_SIZES = {
+    "w2048": dict(width=2048, ff=5632, kv_heads=8, recurrence=(32, 64), latent=dict(heads=32, dim=64, kv_rank=512, window=1024),
+                  experts=dict(n=30, ff=1056, top=4, shared=4224), order="rara"),
+    "w4096": dict(width=4096, ff=7168, kv_heads=8, recurrence=(32, 128), latent=dict(heads=32, dim=128, kv_rank=512, window=2048),
+                  experts=dict(n=62, ff=1344, top=6, shared=2688), order="rra"),
+}
+
+
+def vufolorn_models(size: dict, positions: int):
+    """``{name: (config dict, registry name)}`` of Vufolorn, Bokorax and the Moondream decoder at one size."""
+    w, (heads, d), m, e = size["width"], size["recurrence"], size["latent"], size["experts"]
+    mlp = {"kind": "moe", "expert": {"ff": e["ff"]}, "router": {"experts": e["n"], "top": e["top"]}, "shared": {"ff": e["shared"]}}
+    recurrence = {"heads": heads, "dim": d, "vdim": d, "decay": [2.0 ** (-8.0 * (h + 1) / heads) for h in range(heads)]}
+    latent = {"heads": m["heads"], "dim": m["dim"], "vdim": m["dim"], "kv_rank": m["kv_rank"], "scale": m["dim"] ** -0.5,
+              "mask": {"size": m["window"]}}
+    layers = [{"type": "lightning", "mixer": dict(recurrence), "mlp": mlp} if kind == "r" else
+              {"type": "latent_attention", "mixer": dict(latent), "mlp": mlp} for kind in size["order"]]
+    vufolorn = {"architecture": "Vufolorn", "vocab": COMPARE_VOCAB, "width": w, "norm": {"eps": 1e-6}, "max_positions": positions, "layers": layers}
+    both = bokorax_models(dict(width=w, ff=size["ff"], heads=m["heads"], kv_heads=size["kv_heads"], head=m["dim"], window=m["window"],
+                               memory=(heads * d // 64, 64), rank=64,
+                               experts=dict(n=e["n"], ff=e["ff"] * 2 // 3, top=e["top"], identity=2, groups=(e["n"] // 2 + 1, e["n"] // 2 + 1),
+                                            shared=e["shared"] * 2 // 3),
+                               order=size["order"].replace("r", "w").replace("a", "1")), positions)
+    return {"vufolorn": (vufolorn, "vufolorn"), **both}
+
+
+def run_compare_vufolorn(args, dtype, device) -> dict:
+    """Vufolorn beside Bokorax and the Moondream decoder at equal sizes, through the same step function."""
+    return run_compare_design(args, dtype, device, "vufolorn", VUFOLORN_SIZES, vufolorn_models)
 
 
 def run_compare_bokorax(args, dtype, device) -> dict:
@@ -740,14 +780,15 @@ def main() -> int:
                         help="with --workload: RuntimeConfig.tune_linears (time the vendor library's algorithms at warm-up)")
     parser.add_argument("--check", type=int, default=0,
                         help="with --workload: compare this many greedy requests with the plain implementation (for --layers 2)")
-    parser.add_argument("--workload", default="decode", choices=["decode", "waves256", "mixed48", "compare-vimesun", "compare-bogivik", "compare-letevik", "compare-bokorax"],
+    parser.add_argument("--workload", default="decode", choices=["decode", "waves256", "mixed48", "compare-vimesun", "compare-bogivik", "compare-letevik", "compare-bokorax",
+                                                                     "compare-vufolorn"],
                         help="decode: the benchmark's decode step (default); waves256 and mixed48 run requests through "
                              "InferenceEngine; compare-vimesun, compare-bogivik and compare-letevik measure that design beside the Moondream "
                              "decoder at equal sizes")
     parser.add_argument("--compare-sizes", default=None,
                         help="with --workload compare-*: which of its sizes, with commas between them "
                              "(default: all of them)")
-    parser.add_argument("--compare-model", default="both", choices=["both", "vimesun", "bogivik", "letevik", "bokorax", "moondream2"],
+    parser.add_argument("--compare-model", default="both", choices=["both", "vimesun", "bogivik", "letevik", "bokorax", "vufolorn", "moondream2"],
                         help="with --workload compare-*: one of the two designs only (for profiling)")
     parser.add_argument("--compare-batches", default="1,8,64", help="with --workload compare-bogivik or compare-letevik: batch sizes of the decode steps")
     parser.add_argument("--skip-prefill", action="store_true", help="with --workload compare-bogivik or compare-letevik: decode steps only")
@@ -785,6 +826,9 @@ def main() -> int:
         return 0
     if args.workload == "compare-bokorax":
         print(json.dumps(run_compare_bokorax(args, dtype, device)))
+        return 0
+    if args.workload == "compare-vufolorn":
+        print(json.dumps(run_compare_vufolorn(args, dtype, device)))
         return 0
     if args.workload == "compare-letevik":
         print(json.dumps(run_compare_letevik(args, dtype, device)))

@@ -13,6 +13,7 @@ import torch
 from tests import helpers
 from tests import letevik_cases as cases
 from tests.helpers import Request
+from tests.packed import CUTS, PackedStep
 from tests.plain import letevik_plain as plain
 
 pytestmark = pytest.mark.gpu
@@ -618,68 +619,9 @@ def test_latent_rows_kernels(dtype):
 
 
 # ------------------------------------------------------------------------------------------------ the matrix-core attention's further forms
-class _Packed:
-    """Rows of keys in a paged cache with shuffled pages, and the packed queries of a step over them: row ``r`` has
-    ``lengths[r]`` keys, of which the last ``lengths[r] - starts[r]`` places are this step's queries. Pages that a window
-    has passed and that hold no kept key are given back (the table says -1 and the page holds NaN)."""
-
-    def __init__(self, lengths, starts, window, kept, seed):
-        from types import SimpleNamespace
-
-        self.lengths, self.starts, self.window, self.kept = lengths, starts, window, kept
-        gen = torch.Generator().manual_seed(seed)
-        self.gen = gen
-        n_pages = sum(-(-n // 16) for n in lengths) + 3
-        order = torch.randperm(n_pages, generator=gen).tolist()
-        self.n_pages = n_pages
-        table = torch.full((len(lengths), max(-(-n // 16) for n in lengths) + 1), -1, dtype=torch.int32)
-        for r, n in enumerate(lengths):
-            for p in range(-(-n // 16)):
-                table[r, p] = order.pop()
-        self.full_table = table.clone()
-        if window is not None:
-            for r, s in enumerate(starts):
-                for p in range(max(0, s + 1 - window) // 16):
-                    if p * 16 >= kept:
-                        table[r, p] = -1
-        token_row, kv_lo, kv_hi, cu_q, rows, first = [], [], [], [0], [], []
-        for r, (n, s) in enumerate(zip(lengths, starts)):
-            for b in range(0, n - s, 32):
-                rows.append(r)
-                first.append(len(token_row) + b)
-            for p in range(s, n):
-                token_row.append(r)
-                kv_hi.append(p + 1)
-                kv_lo.append(0 if window is None else max(0, p + 1 - window))
-            cu_q.append(len(token_row))
-        self.n = len(token_row)
-        self.token_row, self.kv_hi, self.cu_q = _i32(token_row), _i32(kv_hi), _i32(cu_q)
-        self.kv_lo = _i32(kv_lo) if window is not None else None
-        self.table = table.to(DEV)
-        from kestrel_amd.engine.batch import Workspace
-
-        # (with a workspace at hand a decode step of few rows deals a row's keys out over several workgroups)
-        self.batch = SimpleNamespace(decode_only=all(n - s == 1 for n, s in zip(lengths, starts)),
-                                     query_blocks={32: (_i32(rows), _i32(first))}, cu_q=self.cu_q,
-                                     workspace=Workspace(torch.device(DEV)))
-
-    def pages(self, per_row, transposed=False):
-        """``per_row[r]`` ``[length, heads, channels]`` into pages ``[pages, heads, 16, channels]`` (or ``[pages, heads, channels, 16]``);
-        pages given back hold NaN."""
-        heads, channels = per_row[0].shape[1:]
-        out = torch.full((self.n_pages, heads, 16, channels), float("nan"), dtype=per_row[0].dtype)
-        for r, rows in enumerate(per_row):
-            for p in range(-(-rows.shape[0] // 16)):
-                if self.table[r, p] >= 0:
-                    part = rows[p * 16:(p + 1) * 16]
-                    out[self.full_table[r, p], :, :part.shape[0]] = part.transpose(0, 1)
-        return (out.transpose(2, 3) if transposed else out).contiguous().to(DEV)
 
 
-_CUTS = {"mixed": ([70, 133, 9, 2, 101, 64, 300], [0, 100, 7, 0, 100, 63, 267]), "decode": ([70, 133, 9, 1, 300], [69, 132, 8, 0, 299])}
-
-
-@pytest.mark.parametrize("cut", list(_CUTS))
+@pytest.mark.parametrize("cut", list(CUTS))
 @pytest.mark.parametrize("window, kept", [(24, 4), (40, 0), (7, 9), (33, 17), (64, 40), (None, 0)])
 @pytest.mark.parametrize("hd, hdv", [(32, 64), (64, 32), (48, 20), (128, 128), (80, 96), (160, 192), (64, 132)])
 def test_two_maps_on_the_matrix_cores(hd, hdv, window, kept, cut):
@@ -688,8 +630,8 @@ def test_two_maps_on_the_matrix_cores(hd, hdv, window, kept, cut):
     in LDS and value channels in slices of 128.)"""
     from kestrel_amd.ops import fast
 
-    lengths, starts = _CUTS[cut]
-    case = _Packed(lengths, starts, window, kept, seed=hd + hdv)
+    lengths, starts = CUTS[cut]
+    case = PackedStep(lengths, starts, window, kept, seed=hd + hdv)
     H, G, scale = 4, 2, 1.7 / math.sqrt(hd)
     bf = torch.bfloat16
     k = [torch.randn(n, 2 * G, hd, generator=case.gen).to(bf) for n in lengths]
@@ -713,7 +655,7 @@ def test_two_maps_on_the_matrix_cores(hd, hdv, window, kept, cut):
     assert bool((err <= 3e-2 + 2e-2 * want.abs()).all()), f"max error {float(err.max()):.3g}"
 
 
-@pytest.mark.parametrize("cut", list(_CUTS))
+@pytest.mark.parametrize("cut", list(CUTS))
 @pytest.mark.parametrize("heads", [5, 40])
 @pytest.mark.parametrize("rank, dr", [(64, 16), (80, 16), (48, 32), (96, 32), (20, 12), (128, 32), (512, 64), (260, 28)])
 def test_latents_with_sinks_on_the_matrix_cores(rank, dr, heads, cut):
@@ -721,8 +663,8 @@ def test_latents_with_sinks_on_the_matrix_cores(rank, dr, heads, cut):
     than one workgroup's columns. (Rows above 128 numbers: the kernel's wide form.)"""
     from kestrel_amd.ops import fast
 
-    lengths, starts = _CUTS[cut]
-    case = _Packed(lengths, starts, None, 0, seed=rank + dr + heads)
+    lengths, starts = CUTS[cut]
+    case = PackedStep(lengths, starts, None, 0, seed=rank + dr + heads)
     scale = 1.5 / math.sqrt(rank + dr)
     bf = torch.bfloat16
     rows = [torch.randn(n, 1, rank + dr, generator=case.gen).to(bf) for n in lengths]
