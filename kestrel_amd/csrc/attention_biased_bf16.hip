@@ -24,7 +24,9 @@
 //    and values at once); the value operand is then gathered from the key page;
 //  * out_f32: outputs leave as fp32;
 //  * softcap > 0: scale * (q . k) passes through softcap * tanh(. / softcap) before the other terms are added;
-//  * gate_per_head: the output gate holds one number per head ([n, H]) instead of one per channel.
+//  * gate_per_head: the output gate holds one number per head ([n, H]) instead of one per channel;
+//  * rows_from, rows_below: of a step with blocks of queries, only rows that bring at least rows_from and less than rows_below
+//    tokens are taken; the others' outputs are left alone (they are another launch's business).
 //
 // A decode step of few rows has few workgroups. With n_splits > 1 a row's tiles of keys are dealt out over that many
 // workgroups in contiguous runs; each leaves its unnormalised outputs, reference point and sum in `partial`
@@ -86,7 +88,8 @@ attn_biased_kernel(const bf16_t* __restrict__ q, long q_row_stride, const bf16_t
                    long out_row_stride, float scale, int H, int Hkv, int hdv, int heads_per_block, int has_sink,
                    float sink_score, const float* __restrict__ bias_table, int bias_len, const bf16_t* __restrict__ gate,
                    long gate_row_stride, const float* __restrict__ sinks, int keep_first, int maps, int values_in_keys,
-                   int out_f32, int hd_wide, int n_splits, float* __restrict__ partial, float softcap, int gate_per_head) {
+                   int out_f32, int hd_wide, int n_splits, float* __restrict__ partial, float softcap, int gate_per_head,
+                   int rows_from, int rows_below) {
     constexpr bool WIDE = NK == 0;
     const int HD = WIDE ? hd_wide : NK * 16;
     const int v0 = WIDE ? blockIdx.z * (NV * 32) : 0;     // the first value channel of this workgroup's slice
@@ -115,8 +118,9 @@ attn_biased_kernel(const bf16_t* __restrict__ q, long q_row_stride, const bf16_t
         kvh = (head / maps / G) * maps + head % maps;
         const int blk = blockIdx.y;
         row = qblk_row[blk];
-        const int tok_end = cu_q[row + 1];
+        const int tok_end = cu_q[row + 1], brings = tok_end - cu_q[row];
         if (qblk_tok[blk] >= tok_end) return;          // (the unused end of a list of fixed length)
+        if (brings < rows_from || brings >= rows_below) return;
         tok = qblk_tok[blk] + col;
         live = tok < tok_end;
         if (!live) tok = tok_end - 1;
@@ -470,7 +474,7 @@ KA_API int ka_attention_biased_bf16(const void* q, long q_row_stride, const void
                                     int page_size, int waves, int has_sink, float sink_score, const float* bias_table,
                                     int bias_len, const void* gate, long gate_row_stride, const float* sinks, int keep_first,
                                     int maps, int values_in_keys, int out_f32, int n_splits, float* partial,
-                                    float softcap, int gate_per_head, hipStream_t stream) {
+                                    float softcap, int gate_per_head, int rows_from, int rows_below, hipStream_t stream) {
     const char* who = "ka_attention_biased_bf16";
     KA_CHECK(softcap >= 0.f, "%s: a cap on the scores must be positive", who);
     KA_CHECK(n >= 0 && n_blocks >= 0 && H > 0 && Hkv > 0 && H % Hkv == 0, "%s: bad sizes", who);
@@ -519,7 +523,8 @@ KA_API int ka_attention_biased_bf16(const void* q, long q_row_stride, const void
                            q_row_stride, (const bf16_t*)k_cache, (const bf16_t*)v_cache, block_table, max_pages, qblk_row, \
                            qblk_tok, cu_q, token_row, kv_lo, kv_hi, positions, slopes, (bf16_t*)out, out_row_stride, scale, \
                            H, Hkv, hdv, heads_per_block, has_sink, sink_score, bias_table, bias_len, (const bf16_t*)gate, \
-                           gate_row_stride, sinks, keep_first, maps, values_in_keys, out_f32, hd, n_splits, partial, softcap, gate_per_head); \
+                           gate_row_stride, sinks, keep_first, maps, values_in_keys, out_f32, hd, n_splits, partial, softcap, gate_per_head, \
+                           rows_from, rows_below);                                                                         \
     }
 #define AB_LAUNCH_NK(NK) AB_LAUNCH(NK, 1) AB_LAUNCH(NK, 2) AB_LAUNCH(NK, 3) AB_LAUNCH(NK, 4)
     AB_LAUNCH_NK(2) AB_LAUNCH_NK(3) AB_LAUNCH_NK(4) AB_LAUNCH_NK(5) AB_LAUNCH_NK(6) AB_LAUNCH_NK(7) AB_LAUNCH_NK(8)

@@ -1,7 +1,8 @@
 // A linear per head on the matrix cores: out[r, h, o] = sum_k a[r, h, k] * w[h, o, k] for every head h, with rows of `a`
 // that hold heads of `a_head` channels (the first k of each are read) and rows of `out` that hold heads of `out_head`
 // channels (the first n_out of each are written, the rest are left alone). bf16 in and out, sums in fp32. With `gate`
-// (rows laid out as those of `out`, a row stride of their own) every output is multiplied by the sigmoid of its gate.
+// (rows laid out as those of `out`, a row stride of their own) every output is multiplied by the sigmoid of its gate. With
+// `skip` (one number a row) the rows whose number is not 0 are left alone.
 //
 // What it is for: mixers that keep a low-rank latent per key and move the per-head up-projections to the query's side
 // (every head's query times its own key matrix, every head's weighted sum of latents times its own value matrix). One
@@ -21,12 +22,15 @@ constexpr int HL_TILE = 64;
 
 __global__ void __launch_bounds__(256)
 heads_linear_kernel(const bf16_t* __restrict__ a, long lda, int a_head, const bf16_t* __restrict__ w, bf16_t* __restrict__ out,
-                    long ldo, int out_head, int n, int n_out, int k, const bf16_t* __restrict__ gate, long ldg) {
+                    long ldo, int out_head, int n, int n_out, int k, const bf16_t* __restrict__ gate, long ldg,
+                    const int* __restrict__ skip) {
     const int wave = threadIdx.x / KA_WAVE, lane = threadIdx.x % KA_WAVE;
     const int col = lane % 32, half = lane / 32;
     const int head = blockIdx.z;
     const int o0 = blockIdx.x * HL_TILE + (wave & 1) * 32, r0 = blockIdx.y * HL_TILE + (wave >> 1) * 32;
     if (o0 >= n_out || r0 >= n) return;                  // (a whole wave; the kernel has no barrier)
+    const bool stores = r0 + col < n && !(skip && skip[r0 + col] != 0);
+    if (__builtin_amdgcn_ballot_w64(stores) == 0) return;
     // rows past the end are clamped for the loads and not stored
     const bf16_t* wp = w + ((size_t)head * n_out + min(o0 + col, n_out - 1)) * k + half * 8;
     const bf16_t* ap = a + (size_t)min(r0 + col, n - 1) * lda + (size_t)head * a_head + half * 8;
@@ -38,7 +42,7 @@ heads_linear_kernel(const bf16_t* __restrict__ a, long lda, int a_head, const bf
         acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const hl_bf16x8*>(wp + kk),
                                                       *reinterpret_cast<const hl_bf16x8*>(ap + kk), acc, 0, 0, 0);
     const int row = r0 + col;
-    if (row >= n) return;
+    if (!stores) return;
     // register i: output o0 + (i / 4) * 8 + half * 4 + i % 4 of the lane's row
     bf16_t* op = out + (size_t)row * ldo + (size_t)head * out_head;
     if (gate) {
@@ -72,7 +76,7 @@ KA_API int ka_heads_linear_supported(long lda, int a_head, long ldo, int out_hea
 }
 
 KA_API int ka_heads_linear_bf16(const void* a, long lda, int a_head, const void* w, void* out, long ldo, int out_head, int n,
-                                int heads, int n_out, int k, const void* gate, long ldg, hipStream_t stream) {
+                                int heads, int n_out, int k, const void* gate, long ldg, const int* skip, hipStream_t stream) {
     const char* who = "ka_heads_linear_bf16";
     KA_CHECK(n >= 0 && heads > 0 && heads <= 65535, "%s: bad sizes", who);
     KA_CHECK(ka_heads_linear_supported(lda, a_head, ldo, out_head, n_out, k), "%s: sizes k=%d n_out=%d heads of %d -> %d not covered", who, k, n_out, a_head, out_head);
@@ -82,7 +86,7 @@ KA_API int ka_heads_linear_bf16(const void* a, long lda, int a_head, const void*
     const dim3 grid((n_out + HL_TILE - 1) / HL_TILE, (n + HL_TILE - 1) / HL_TILE, heads);
     KA_CHECK(grid.y <= 65535, "%s: too many rows %d", who, n);
     hipLaunchKernelGGL(heads_linear_kernel, grid, dim3(256), 0, stream, (const bf16_t*)a, lda, a_head, (const bf16_t*)w,
-                       (bf16_t*)out, ldo, out_head, n, n_out, k, (const bf16_t*)gate, ldg);
+                       (bf16_t*)out, ldo, out_head, n, n_out, k, (const bf16_t*)gate, ldg, skip);
     KA_LAUNCH_CHECK();
     return 0;
 }

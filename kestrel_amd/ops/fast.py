@@ -58,9 +58,14 @@ _SIGNATURES = {
     "ka_attention_biased_bf16": [_c_void_p, _c_long, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_int,
                                  _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_long, _c_float,
                                  _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void_p, _c_int, _c_void_p, _c_long,
-                                 _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_float, _c_int, _c_void_p],
+                                 _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_float, _c_int, _c_int, _c_int, _c_void_p],
+    "ka_latent_expand_supported": [_c_int, _c_int, _c_int, _c_int, _c_long],
+    "ka_latent_expand_plan": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p,
+                              _c_void_p, _c_void_p, _c_void_p, _c_void_p],
+    "ka_latent_expand_bf16": [_c_void_p, _c_long, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p,
+                              _c_void_p, _c_void_p],
     "ka_heads_linear_bf16": [_c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p,
-                             _c_long, _c_void_p],
+                             _c_long, _c_void_p, _c_void_p],
     "ka_heads_linear_supported": [_c_long, _c_int, _c_long, _c_int, _c_int, _c_int],
     "ka_experts_gemm_supported": [_c_long, _c_int, _c_int, _c_long, _c_int, _c_int],
     "ka_experts_gemm_bf16": [_c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p,
@@ -632,12 +637,13 @@ def biased_query_block(head_dim: int, value_dim: int) -> Optional[int]:
 def attention_biased_bf16(q, k_cache, v_cache, block_table, token_row, kv_lo, kv_hi, out, scale, n_heads, n_kv_heads,
                           head_dim, value_dim, positions, slopes, sink, batch, bias_table=None, gate=None, sinks=None,
                           keep_first: int = 0, maps: int = 1, values_in_keys: bool = False, softcap: Optional[float] = None,
-                          gate_per_head: bool = False) -> bool:
+                          gate_per_head: bool = False, row_tokens=None) -> bool:
     """Attention with the further terms of ``ops.core.attention_generic`` (values of ``value_dim`` channels, ``slopes``
     times the distance taken off the scores, a ``sink`` in the softmax's denominator or one per head in ``sinks``, kept
     first keys before the window, several maps per head over shared values, values that are the first channels of the
     keys, fp32 outputs where ``out`` is fp32) on the matrix cores, for prompt portions, mixed steps and decode steps
-    alike. False: not covered (head sizes, page size, alignment, no list of blocks of 32 queries with the step),
+    alike. ``row_tokens`` ``(from, below)``: of a step that is no decode step, only rows of that many tokens are taken, the others'
+    outputs are left alone. False: not covered (head sizes, page size, alignment, no list of blocks of 32 queries with the step),
     nothing was run."""
     n = q.shape[0]
     page_size = k_cache.shape[2]
@@ -702,7 +708,8 @@ def attention_biased_bf16(q, k_cache, v_cache, block_table, token_row, kv_lo, kv
         value_dim, page_size, waves, int(sink is not None or sinks is not None), float(sink or 0.0), _ptr(bias_table),
         int(bias_table.shape[1]) if bias_table is not None else 0, _ptr(gate),
         (gate.stride(0) if n > 1 else gate_cols) if gate is not None else 0, _ptr(sinks), int(keep_first), int(maps),
-        int(bool(values_in_keys)), int(out_f32), n_splits, _ptr(partial), float(softcap or 0.0), int(bool(gate_per_head)), stream_ptr()))
+        int(bool(values_in_keys)), int(out_f32), n_splits, _ptr(partial), float(softcap or 0.0), int(bool(gate_per_head)),
+        *(row_tokens if row_tokens is not None else (0, 0x7fffffff)), stream_ptr()))
     return True
 
 
@@ -715,20 +722,76 @@ def attention_maps_bf16(q, k_cache, v_cache, block_table, token_row, kv_lo, kv_h
 
 
 def attention_latent_bf16(q, cache, block_table, token_row, kv_hi, out, scale, n_heads, row_dim, rank, sinks, batch, kv_lo=None,
-                          head_gate=None) -> bool:
+                          head_gate=None, row_tokens=None) -> bool:
     """``n_heads`` query heads of ``row_dim`` channels over one cached row per key whose first ``rank`` channels are its
     value, with a sink score per head (``sinks`` ``None``: no sinks), behind a window (``kv_lo``), times the sigmoid of one number
     per head (``head_gate`` ``[n, H]``), on the matrix cores (rows above 128 channels: the kernel's wide form). False: not
     covered (rows that are no multiple of 16 channels among others)."""
     return attention_biased_bf16(q, cache, None, block_table, token_row, kv_lo, kv_hi, out, scale, n_heads, 1, row_dim, rank,
                                  None, None, None, batch, sinks=sinks, values_in_keys=True, gate=head_gate,
-                                 gate_per_head=head_gate is not None)
+                                 gate_per_head=head_gate is not None, row_tokens=row_tokens)
 
 
-def heads_linear_bf16(a, a_head: int, k: int, weights, out, out_head: int, n_out: int, gate=None) -> bool:
+class LiftPlan(NamedTuple):
+    """What of a step's cached latents is lifted to keys and values per head (``latent_expand_plan``)."""
+
+    capacity: int               # lifted pages there is room for
+    list: torch.Tensor          # int32 [capacity * 16]: place in the cache of every lifted place, -1: none
+    table: torch.Tensor         # int32 [rows, max_pages]: lifted page of a row's logical page
+    used: torch.Tensor          # int32 [1]: lifted places in use
+    lifted: torch.Tensor        # int32 [tokens]: 1 for the tokens of a lifted row
+    row_tokens: int             # rows of at least this many tokens are lifted
+
+
+def latent_expand_supported(n_heads: int, head_dim: int, value_dim: int, rank: int, row_dim: int) -> bool:
+    """Whether latents of ``rank`` channels (in cached rows of ``row_dim``) can be lifted to keys and values of these heads and
+    attended to on the matrix cores with keys and values in registers."""
+    handle = lib()
+    return bool(handle.ka_latent_expand_supported(int(n_heads), int(head_dim), int(value_dim), int(rank), int(row_dim))) \
+        and head_dim <= 128 and value_dim <= 128 and bool(handle.ka_attention_biased_supported(int(head_dim), int(value_dim), 16))
+
+
+def latent_expand_plan(batch, group, name: str, window: int, row_tokens: int, pool_pages: int) -> Optional[LiftPlan]:
+    """Which rows of the step are lifted (those of at least ``row_tokens`` tokens), made by one launch from what the step holds. The
+    room it is made for follows from the step's numbers of tokens and rows alone. ``None``: too many rows or pages."""
+    handle = lib()
+    n, rows = batch.n_tokens, batch.n_rows
+    if rows > int(handle.ka_latent_expand_max_rows()) or batch.workspace is None:
+        return None
+    # a row of q tokens behind a window of w reads at most w - 1 + q keys, which touch one page more at either end
+    most = n // 16 + min(rows, n // row_tokens) * (window // 16 + 3)
+    capacity = -(-min(most, pool_pages) // 8) * 8
+    if capacity <= 0 or capacity // 8 > 65535:
+        return None
+    ws = batch.workspace
+    max_pages = group.block_table.shape[1]
+    plan = LiftPlan(capacity, ws.get(f"latent.lift_list.{name}", (capacity * 16,), torch.int32),
+                    ws.get(f"latent.lift_table.{name}", (rows, max_pages), torch.int32),
+                    ws.get(f"latent.lift_used.{name}", (1,), torch.int32), ws.get(f"latent.lifted.{name}", (n,), torch.int32), int(row_tokens))
+    _check(handle.ka_latent_expand_plan(batch.cu_q.data_ptr(), batch.kv_len.data_ptr(), _ptr(group.kv_lo), batch.token_row.data_ptr(),
+                                        group.block_table.data_ptr(), max_pages, n, rows, int(row_tokens), capacity, plan.list.data_ptr(),
+                                        plan.table.data_ptr(), plan.used.data_ptr(), plan.lifted.data_ptr(), stream_ptr()))
+    return plan
+
+
+def latent_expand_bf16(cache, weights, plan: LiftPlan, n_heads: int, head_dim: int, value_dim: int, rank: int, workspace):
+    """The latents that ``plan`` lists lifted by ``weights`` ``[H head_dim + H value_dim, rank]``: keys ``[pages, H, 16, head_dim]`` and
+    values ``[pages, H, value_dim, 16]`` of the workspace."""
+    if cache.dtype != torch.bfloat16 or not cache.is_contiguous() or cache.dim() != 4 or cache.shape[1] != 1 or cache.shape[2] != 16 \
+            or weights.dtype != torch.bfloat16 or not weights.is_contiguous() \
+            or tuple(weights.shape) != (n_heads * (head_dim + value_dim), rank) or cache.shape[3] < rank:
+        raise KernelError("latents to lift: cache bf16 [pages, 1, 16, >= rank], weights bf16 [H (d + dv), rank]")
+    keys = workspace.get("latent.lift_keys", (plan.capacity, n_heads, 16, head_dim), torch.bfloat16)
+    values = workspace.get("latent.lift_values", (plan.capacity, n_heads, value_dim, 16), torch.bfloat16)
+    _check(lib().ka_latent_expand_bf16(cache.data_ptr(), cache.shape[3], weights.data_ptr(), plan.list.data_ptr(), plan.used.data_ptr(),
+                                       plan.capacity, n_heads, head_dim, value_dim, rank, keys.data_ptr(), values.data_ptr(), stream_ptr()))
+    return keys, values
+
+
+def heads_linear_bf16(a, a_head: int, k: int, weights, out, out_head: int, n_out: int, gate=None, skip=None) -> bool:
     """``out[:, h, :n_out] = a[:, h, :k] @ weights[h].T`` for every head in one launch on the matrix cores: ``a`` ``[n, H a_head]``,
     ``weights`` ``[H, n_out, k]``, ``out`` ``[n, H out_head]``, all bf16; with ``gate`` (bf16, laid out as ``out``) times the
-    sigmoid of it. False: not covered (``k`` no multiple of 16, heads that are not aligned), nothing was run."""
+    sigmoid of it. ``skip`` (int32 ``[n]``): rows whose number is not 0 are left alone. False: not covered (``k`` no multiple of 16, heads that are not aligned), nothing was run."""
     n = a.shape[0]
     if n == 0:
         return True
@@ -747,7 +810,7 @@ def heads_linear_bf16(a, a_head: int, k: int, weights, out, out_head: int, n_out
         return False
     _check(handle.ka_heads_linear_bf16(a.data_ptr(), lda, a_head, weights.data_ptr(), out.data_ptr(), ldo, out_head, n, heads,
                                        n_out, k, _ptr(gate), (gate.stride(0) if n > 1 else heads * out_head) if gate is not None else 0,
-                                       stream_ptr()))
+                                       _ptr(skip), stream_ptr()))
     return True
 
 

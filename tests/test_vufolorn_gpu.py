@@ -288,7 +288,7 @@ def test_choice_by_logits_kernel(outputs, top):
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=DTYPE_IDS)
-@pytest.mark.parametrize("n, dim, ff, n_experts, top", [(3, 100, 36, 5, 2), (70, 128, 48, 6, 3), (200, 64, 96, 4, 1), (150, 192, 80, 33, 4)])
+@pytest.mark.parametrize("n, dim, ff, n_experts, top", [(3, 100, 36, 5, 2), (70, 128, 48, 6, 3), (200, 64, 96, 4, 1), (150, 192, 80, 33, 4), (90, 16, 176, 3, 2)])
 def test_plain_experts_and_the_weighted_sum_kernels(n, dim, ff, n_experts, top, dtype):
     """Experts of two linears with the square of relu between, pair by pair and (bfloat16) listed by expert; the weighted
     sum with a gated shared expert, normalised, added into the stream and followed by the next norm."""
@@ -380,6 +380,61 @@ def test_windowed_latents_and_a_gate_per_head(rank, heads, window, cut, kernel, 
     _near(out.view(case.n, heads, rank), want, dtype, "latents")
 
 
+@pytest.mark.parametrize("host_knows", [True, False], ids=["launched", "captured"])
+@pytest.mark.parametrize("lengths, starts", [([70, 300, 9, 101, 64, 200, 129], [0, 100, 7, 100, 0, 137, 0]), ([500], [300]), ([40, 64], [0, 1])],
+                         ids=["mixed", "one portion", "none long enough"])
+@pytest.mark.parametrize("rank, heads, d, dv, window", [(64, 4, 32, 24, 24), (48, 2, 64, 64, 7), (144, 3, 32, 80, 33), (128, 1, 128, 128, 64), (80, 6, 48, 4, 200)])
+def test_latents_lifted_for_long_portions(rank, heads, d, dv, window, lengths, starts, host_knows):
+    """The mixer's core on a step whose long portions are lifted to keys and values per head while its short portions and
+    single tokens stay with the latents; one key stands out at the window's edge; pages given back hold NaN. ``captured``: the
+    host does not know what the step brings (as when it was captured), both halves are launched."""
+    from kestrel_amd.engine.batch import GroupBatch
+    from kestrel_amd.parts.base import LayerCache
+    from kestrel_amd.parts.latent_attention import LatentAttention
+    from kestrel_amd.parts.specs import LatentAttentionSpec, PositionSpec
+
+    bf = torch.bfloat16
+    case = PackedStep(lengths, starts, window, 0, seed=rank + d)
+    gen = case.gen
+    scale = 1.0 / math.sqrt(d)
+    mixer = LatentAttention(LatentAttentionSpec("latent_attention", 32, heads, d, 0, dv, None, rank, scale, 1e-5, PositionSpec("none"),
+                                                head_sinks=False, gate_per_head=True, window=window))
+    w = {name: (torch.randn(spec.shape, generator=gen) * 0.2).to(bf) for name, spec in mixer.params().items()}
+    mixer.bind({k: v.to(DEV) for k, v in w.items()}, bf, torch.device(DEV))
+    assert mixer.lift_weight is not None
+    uk, uv = w["uk.weight"].double(), w["uv.weight"].double()
+    rows, q = [], []
+    for n, s in zip(lengths, starts):
+        c = torch.randn(n, 1, rank, generator=gen)
+        lean = torch.randn(rank, generator=gen)
+        lean = lean / lean.norm() * math.sqrt(rank)
+        c[n % window::window, 0] = lean
+        key = (uk @ lean.double()).reshape(heads, d)
+        queries = 0.2 * torch.randn(n - s, heads, d, generator=gen).double() + key * (9.0 / (scale * key.pow(2).sum(dim=1, keepdim=True)))
+        rows.append(c.to(bf))
+        q.append(queries.float().to(bf))
+    down = torch.zeros(case.n, mixer.down_dim, dtype=bf)
+    down[:, :heads * d] = torch.cat(q).reshape(case.n, -1)
+    gate = (torch.randn(case.n, heads, generator=gen) * 3).to(bf)
+    down[:, heads * d + rank:heads * d + rank + heads] = gate
+    batch = case.batch
+    batch.n_tokens, batch.n_rows, batch.token_row, batch.kv_hi = case.n, len(lengths), case.token_row, case.kv_hi
+    batch.kv_len, batch.positions = _i32(lengths), _i32([0] * case.n)
+    batch.host = {"q_lens": [n - s for n, s in zip(lengths, starts)] if host_knows else []}
+    pages = case.pages(rows)
+    batch.groups = {0: GroupBatch(block_table=case.table, slots=_i32([-1] * case.n), kv_lo=case.kv_lo, page_size=16)}
+    got = mixer.attend(down.to(DEV), batch, LayerCache(group=0, tensors={"k": pages}))
+    want = []
+    for r, (n, s) in enumerate(zip(lengths, starts)):
+        c = rows[r].double()[:, 0]
+        k, v = (c @ uk.T).reshape(n, heads, d), (c @ uv.T).reshape(n, heads, dv)
+        seen = plain.window_mask(n, window)[s:]
+        want.append(torch.stack([plain.softmax_over((q[r].double()[:, h] @ k[:, h].T) * scale, seen) @ v[:, h] for h in range(heads)], dim=1))
+    want = torch.cat(want) * torch.sigmoid(gate.double())[:, :, None]
+    spread = float(want.std())
+    _near(got.view(case.n, heads, dv), want, bf, "heads", atol=3e-2 * max(1.0, 2 * spread), rtol=2e-2)
+
+
 def test_latents_made_ready_without_a_rotated_part():
     """Only the latent is normalised and cached: rows of ``[q | latent | gate]`` with no latent of queries and no shared part."""
     from kestrel_amd.ops import core
@@ -406,7 +461,7 @@ def test_the_matrix_core_kernels_run_where_sizes_allow():
     from kestrel_amd.ops import fast
 
     calls = {}
-    names = ("attention_biased_bf16", "linear_attention_chunks_bf16", "experts_feed_forward_bf16", "heads_linear_bf16")
+    names = ("attention_biased_bf16", "linear_attention_chunks_bf16", "experts_feed_forward_bf16", "heads_linear_bf16", "latent_expand_bf16")
     originals = {name: getattr(fast, name) for name in names}
 
     def spy(name):
@@ -422,8 +477,9 @@ def test_the_matrix_core_kernels_run_where_sizes_allow():
         for model in ("P", "R"):
             calls.clear()
             folder = cases.model_dir(model)
-            helpers.replay(_runner(folder, torch.bfloat16), {"r": Request("r", _ids(folder, 900, 80))}, [[("r", 80)]])
-            assert set(calls) == set(names) and all(all(done) for done in calls.values()), (model, calls)
+            for length in (50, 80):              # (too short for its latents to be lifted, and long enough)
+                helpers.replay(_runner(folder, torch.bfloat16), {"r": Request("r", _ids(folder, 900, length))}, [[("r", length)]])
+            assert set(calls) == set(names) and all(bool(d) for done in calls.values() for d in done), (model, calls)
     finally:
         for name in names:
             setattr(fast, name, originals[name])
