@@ -225,8 +225,18 @@ attn_biased_kernel(const bf16_t* __restrict__ q, long q_row_stride, const bf16_t
 #pragma unroll
             for (int i = 0; i < 16; ++i) s[i] = 0.f;
             if constexpr (WIDE) {
-
-                for (int c = 0; c < HD / 16; ++c)
+                // (eight steps' keys are asked for before the first is multiplied: one trip to memory for all of them)
+                constexpr int AHEAD = 8;
+                int c = 0;
+                for (; c + AHEAD <= HD / 16; c += AHEAD) {
+                    ab_bf16x8 kw[AHEAD];
+#pragma unroll
+                    for (int u = 0; u < AHEAD; ++u) kw[u] = *reinterpret_cast<const ab_bf16x8*>(kp + (c + u) * 16);
+#pragma unroll
+                    for (int u = 0; u < AHEAD; ++u)
+                        s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kw[u], q_lds[(c + u) * KA_WAVE + lane], s, 0, 0, 0);
+                }
+                for (; c < HD / 16; ++c)
                     s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const ab_bf16x8*>(kp + c * 16),
                                                                 q_lds[c * KA_WAVE + lane], s, 0, 0, 0);
             } else {
@@ -414,32 +424,52 @@ attn_biased_kernel(const bf16_t* __restrict__ q, long q_row_stride, const bf16_t
         }
 }
 
-// Merges the partial results of a decode step whose rows' keys were split over workgroups: a wave per (token, head).
-__global__ void __launch_bounds__(KA_WAVE)
+// Merges the partial results of a decode step whose rows' keys were split over workgroups (at most 64 of them): a workgroup
+// per (token, head). A lane of every wave works out one run's weight, so that the runs are looked up once and side by
+// side; a thread then sums its channels over the runs in their order, four runs' numbers asked for at a time.
+constexpr int AB_FINISH_THREADS = 256;
+__global__ void __launch_bounds__(AB_FINISH_THREADS)
 attn_biased_finish_kernel(const float* __restrict__ partial, int n_splits, int H, int hdv, void* __restrict__ out,
                           long out_row_stride, int out_f32, int has_sink, float sink_score, const float* __restrict__ sinks,
                           const bf16_t* __restrict__ gate, long gate_row_stride, int gate_per_head) {
-    const int tok = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
-    const float* pp = partial + ((size_t)tok * H + head) * n_splits * (hdv + 2);
+    __shared__ float weight_s[KA_WAVE];
+    const int tok = blockIdx.x, head = blockIdx.y, lane = threadIdx.x % KA_WAVE;
+    const size_t record = hdv + 2;
+    const float* pp = partial + ((size_t)tok * H + head) * n_splits * record;
     const float sink2 = (sinks ? sinks[head] : sink_score) * AB_LOG2E;
-    float top = has_sink ? sink2 : -INFINITY;
-    for (int s = 0; s < n_splits; ++s) top = fmaxf(top, pp[(size_t)s * (hdv + 2) + hdv]);
-    float total = has_sink ? __builtin_amdgcn_exp2f(sink2 - top) : 0.f;
-    for (int s = 0; s < n_splits; ++s) {
-        const float ms = pp[(size_t)s * (hdv + 2) + hdv], ls = pp[(size_t)s * (hdv + 2) + hdv + 1];
-        if (ls > 0.f) total += ls * __builtin_amdgcn_exp2f(ms - top);
+    float m = -INFINITY, l = 0.f;
+    if (lane < n_splits) {
+        m = pp[lane * record + hdv];
+        l = pp[lane * record + hdv + 1];
     }
+    if (!(l > 0.f)) m = -INFINITY;              // (a run that saw no key left nothing to add, and its outputs may be anything)
+    float top = ka_wave_max(m);
+    if (has_sink) top = fmaxf(top, sink2);
+    const float scale = l > 0.f ? __builtin_amdgcn_exp2f(m - top) : 0.f;
+    const float total = ka_wave_sum(scale > 0.f ? l * scale : 0.f) + (has_sink ? __builtin_amdgcn_exp2f(sink2 - top) : 0.f);
     const float inv = total > 0.f ? 1.0f / total : 0.f;
+    if (threadIdx.x < KA_WAVE) weight_s[lane] = scale * inv;
+    __syncthreads();
     const size_t out_at = (size_t)tok * out_row_stride + (size_t)head * hdv;
-    for (int ch = lane; ch < hdv; ch += KA_WAVE) {
+    float head_gate = 1.f;
+    if (gate && gate_per_head) head_gate = 1.0f / (1.0f + __expf(-(float)gate[(size_t)tok * gate_row_stride + head]));
+    for (int ch = threadIdx.x; ch < hdv; ch += AB_FINISH_THREADS) {
         float acc = 0.f;
-        for (int s = 0; s < n_splits; ++s) {
-            const float ls = pp[(size_t)s * (hdv + 2) + hdv + 1];
-            // (a split that saw no key left nothing to add, and its outputs may be anything)
-            if (ls > 0.f) acc += pp[(size_t)s * (hdv + 2) + ch] * __builtin_amdgcn_exp2f(pp[(size_t)s * (hdv + 2) + hdv] - top);
+        for (int s0 = 0; s0 < n_splits; s0 += 4) {
+            float x[4], w[4];
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const int sp = min(s0 + u, n_splits - 1);
+                x[u] = pp[sp * record + ch];
+                w[u] = s0 + u < n_splits ? weight_s[sp] : 0.f;
+            }
+#pragma unroll
+            for (int u = 0; u < 4; ++u)
+                if (w[u] > 0.f) acc = fmaf(x[u], w[u], acc);
         }
-        float y = acc * inv;
-        if (gate) y *= 1.0f / (1.0f + __expf(-(float)gate[(size_t)tok * gate_row_stride + (gate_per_head ? (size_t)head : (size_t)head * hdv + ch)]));
+        float y = acc;
+        if (gate && gate_per_head) y *= head_gate;
+        else if (gate) y *= 1.0f / (1.0f + __expf(-(float)gate[(size_t)tok * gate_row_stride + (size_t)head * hdv + ch]));
         if (out_f32) reinterpret_cast<float*>(out)[out_at + ch] = y;
         else reinterpret_cast<bf16_t*>(out)[out_at + ch] = (bf16_t)y;
     }
@@ -534,7 +564,7 @@ KA_API int ka_attention_biased_bf16(const void* q, long q_row_stride, const void
     KA_LAUNCH_CHECK();
     if (n_splits > 1) {
         KA_CHECK(H <= 65535, "%s: too many heads %d", who, H);
-        hipLaunchKernelGGL(attn_biased_finish_kernel, dim3(n, H), dim3(KA_WAVE), 0, stream, partial, n_splits, H, hdv, out,
+        hipLaunchKernelGGL(attn_biased_finish_kernel, dim3(n, H), dim3(AB_FINISH_THREADS), 0, stream, partial, n_splits, H, hdv, out,
                            out_row_stride, out_f32, has_sink, sink_score, sinks, (const bf16_t*)gate, gate_row_stride, gate_per_head);
         KA_LAUNCH_CHECK();
     }

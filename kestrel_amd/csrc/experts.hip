@@ -153,21 +153,35 @@ KA_API int ka_route(const float* logits, long stride, const float* correction, i
 // ----------------------------------------------------------------------------
 constexpr int EX_COLS = 16;
 
-template <typename T>
-__device__ __forceinline__ float ex_dot(const T* __restrict__ w, const float* __restrict__ a, int K, int lane, bool vectors) {
-    float acc = 0.f;
+// R rows of weights against one row of inputs: the rows' loads are in flight together and share the input's. A row's sum is
+// made in the order it would be made in alone.
+template <typename T, int R>
+__device__ __forceinline__ void ex_dots(const T* const (&w)[R], const float* __restrict__ a, int K, int lane, bool vectors, float (&y)[R]) {
+    float acc[R];
+#pragma unroll
+    for (int r = 0; r < R; ++r) acc[r] = 0.f;
     if (vectors) {
         constexpr int V = 16 / sizeof(T);
         typedef __attribute__((ext_vector_type(V))) T vec;
+#pragma unroll 2
         for (int c = lane * V; c < K; c += KA_WAVE * V) {
-            const vec x = *reinterpret_cast<const vec*>(w + c);
+            vec x[R];
 #pragma unroll
-            for (int e = 0; e < V; ++e) acc = fmaf(ka_to_float(x[e]), a[c + e], acc);
+            for (int r = 0; r < R; ++r) x[r] = *reinterpret_cast<const vec*>(w[r] + c);
+#pragma unroll
+            for (int e = 0; e < V; ++e) {
+                const float h = a[c + e];
+#pragma unroll
+                for (int r = 0; r < R; ++r) acc[r] = fmaf(ka_to_float(x[r][e]), h, acc[r]);
+            }
         }
     } else {
-        for (int c = lane; c < K; c += KA_WAVE) acc = fmaf(ka_to_float(w[c]), a[c], acc);
+        for (int c = lane; c < K; c += KA_WAVE)
+#pragma unroll
+            for (int r = 0; r < R; ++r) acc[r] = fmaf(ka_to_float(w[r][c]), a[c], acc[r]);
     }
-    return ka_wave_sum(acc);
+#pragma unroll
+    for (int r = 0; r < R; ++r) y[r] = ka_wave_sum(acc[r]);
 }
 
 template <typename T>
@@ -186,21 +200,36 @@ experts_linear_kernel(const T* __restrict__ a, long a_stride, int a_div, const T
     const int n_out = gated ? N / 2 : N;
     const T* We = W + (size_t)e * N * K;
     const bool vectors = K % (16 / sizeof(T)) == 0 && reinterpret_cast<uintptr_t>(W) % 16 == 0;
-    for (int q = wave; q < EX_COLS; q += 4) {
-        const int j = blockIdx.x * EX_COLS + q;
-        if (j >= n_out) break;
-        float y;
-        if (gated) {
-            const float g = ex_dot(We + (size_t)(2 * j) * K, row, K, lane, vectors);
-            const float v = ex_dot(We + (size_t)(2 * j + 1) * K, row, K, lane, vectors);
-            y = ka_activate(act, g) * v;
-        } else {
-            y = ex_dot(We + (size_t)j * K, row, K, lane, vectors);
-            if (ka_act_base(act)) y = ka_activate(act, y);
+    constexpr int ROWS = EX_COLS / 4;           // outputs of a wave: four neighbours, or (gated) two pairs at a time
+    const int j0 = blockIdx.x * EX_COLS + wave * ROWS;
+    if (j0 >= n_out) return;
+    float y[ROWS];
+    if (gated) {
+#pragma unroll
+        for (int q = 0; q < ROWS; q += 2) {
+            const T* w[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) w[r] = We + (size_t)min(2 * (j0 + q) + r, N - 1) * K;     // (rows past the end: not stored)
+            float s[4];
+            ex_dots<T, 4>(w, row, K, lane, vectors, s);
+            y[q] = ka_activate(act, s[0]) * s[1];
+            y[q + 1] = ka_activate(act, s[2]) * s[3];
         }
-        if (lane == 0) {
-            if (out_f32) reinterpret_cast<float*>(out)[(size_t)p * out_stride + j] = y;
-            else reinterpret_cast<T*>(out)[(size_t)p * out_stride + j] = ka_from_float<T>(y);
+    } else {
+        const T* w[ROWS];
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r) w[r] = We + (size_t)min(j0 + r, N - 1) * K;
+        ex_dots<T, ROWS>(w, row, K, lane, vectors, y);
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r)
+            if (ka_act_base(act)) y[r] = ka_activate(act, y[r]);
+    }
+    if (lane == 0) {
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r) {
+            if (j0 + r >= n_out) break;
+            if (out_f32) reinterpret_cast<float*>(out)[(size_t)p * out_stride + j0 + r] = y[r];
+            else reinterpret_cast<T*>(out)[(size_t)p * out_stride + j0 + r] = ka_from_float<T>(y[r]);
         }
     }
 }
