@@ -740,3 +740,27 @@ KA_API int ka_unit_norm_cache(void* qkv, int dtype, long row_stride, const int* 
     KA_LAUNCH_CHECK();
     return 0;
 }
+
+// ----------------------------------------------------------------------------
+// x = act(x) in place over bf16 rows of n numbers (n a multiple of 8, rows 16-byte aligned): the second half of a linear whose
+// activation the kernel that multiplied has no epilogue for.
+// ----------------------------------------------------------------------------
+__global__ void __launch_bounds__(256) activate_rows_kernel(bf16_t* __restrict__ x, long stride, int n, int act) {
+    typedef __attribute__((ext_vector_type(8))) __bf16 vec8;
+    bf16_t* row = x + (size_t)blockIdx.y * stride;
+    const int c = (blockIdx.x * 256 + threadIdx.x) * 8;
+    if (c >= n) return;
+    vec8 v = *reinterpret_cast<const vec8*>(row + c);
+#pragma unroll
+    for (int u = 0; u < 8; ++u) v[u] = (bf16_t)ka_activate_fast(act, (float)v[u]);
+    *reinterpret_cast<vec8*>(row + c) = v;
+}
+
+KA_API int ka_activate_rows(void* x, long stride, int m, int n, int act, hipStream_t stream) {
+    KA_CHECK(m >= 0 && m <= 65535 && n > 0 && n % 8 == 0 && stride >= n && stride % 8 == 0 && (uintptr_t)x % 16 == 0, "ka_activate_rows: bad sizes or alignment");
+    KA_CHECK(ka_act_known(act) && !ka_act_gated(act), "ka_activate_rows: unknown activation %d", act);
+    if (m == 0) return 0;
+    hipLaunchKernelGGL(activate_rows_kernel, dim3(ka_cdiv(n, 2048), m), dim3(256), 0, stream, (bf16_t*)x, stride, n, act);
+    KA_LAUNCH_CHECK();
+    return 0;
+}

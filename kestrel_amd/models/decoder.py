@@ -136,6 +136,9 @@ class DecoderModel:
         """Run the packed tokens of ``batch``; returns fp32 logits ``[wanted, vocab]``."""
         plan = self.plan
         ws = batch.workspace
+        if getattr(batch, "host", None) is not None:
+            # what parts make once a step for all layers: made anew by every run (a captured run must launch it itself)
+            batch.host["made_once"] = {}
         x = ws.get("model.x", (batch.n_tokens, plan.dim), torch.float32)
         # (a norm of the embedded tokens reads them from a buffer of their own)
         looked_up = x if self.embedding_norm is None else ws.get("model.looked_up", (batch.n_tokens, plan.dim), torch.float32)

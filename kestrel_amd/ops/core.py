@@ -50,6 +50,7 @@ _SIGNATURES = {
                        _c_int, _c_void_p, _c_void_p],
     "ka_clamped_pairs": [_c_void_p, _c_long, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void_p],
     "ka_add_vector": [_c_void_p, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_void_p],
+    "ka_activate_rows": [_c_void_p, _c_long, _c_int, _c_int, _c_int, _c_void_p],
     "ka_add_normed": [_c_void_p, _c_void_p, _c_void_p, _c_float, _c_void_p, _c_float, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
     "ka_experts_combine_normed": [_c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p,
                                   _c_long, _c_void_p, _c_int, _c_void_p, _c_float, _c_void_p, _c_float, _c_void_p, _c_void_p],
@@ -460,6 +461,13 @@ def add_vector(x: torch.Tensor, vector: torch.Tensor, other: Optional[torch.Tens
     _need(other is None or (other.dtype == torch.float32 and other.is_contiguous() and other.shape == x.shape),
           "add_vector: other must be contiguous fp32 of the shape of x")
     _check(lib().ka_add_vector(x.data_ptr(), vector.data_ptr(), code_of(vector.dtype), _ptr(other), n, dim, stream_ptr()))
+
+
+def activate_rows(x: torch.Tensor, act: int) -> None:
+    """``x = act(x)`` in place for bf16 rows ``x`` ``[m, n]`` (``n`` and the row stride multiples of 8)."""
+    _dev(x)
+    _need(x.dtype == torch.bfloat16 and x.dim() == 2 and x.stride(1) == 1, "activate_rows: x must be bf16 rows")
+    _check(lib().ka_activate_rows(x.data_ptr(), x.stride(0) if x.shape[0] > 1 else x.shape[1], x.shape[0], x.shape[1], int(act), stream_ptr()))
 
 
 def _norm_pair(who: str, x, norm, then, rows):

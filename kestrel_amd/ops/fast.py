@@ -12,6 +12,7 @@ from typing import Dict, NamedTuple, Optional
 import torch
 
 from ..csrc import build as _build
+from . import core
 from .core import KA_BF16, KA_F32, KernelError, _ptr, stream_ptr
 
 _c_void_p, _c_int, _c_long, _c_float = ctypes.c_void_p, ctypes.c_int, ctypes.c_long, ctypes.c_float
@@ -108,6 +109,12 @@ TILED_CONFIG = 0
 # four linears: 201 against 242 us a layer at 2,048 rows, 112 against 151 at 730, 64 against 72 at 96.
 LIBRARY_LINEAR = True
 LIBRARY_WORKSPACE_BYTES = 128 << 20
+# Activations that the library has no epilogue for (relu squared: ops.linear.ACT_RELU_SQUARED), and the size of an output from
+# which the library's product and a pass over it are faster than this package's tiled kernel with the activation in its
+# epilogue (2,048 rows of 2,048 by 4,224: 75 us).
+_ACTIVATIONS_APART = (4,)
+ACTIVATION_APART_FROM_ROWS = 256
+ACTIVATION_APART_FROM_COLUMNS = 1024
 _library_space = {}
 SCRATCH_FLOATS = 8 << 20
 WIDE_FLOATS = 8 << 20              # 32 MB of partial sums for the wide skinny kernel
@@ -315,10 +322,15 @@ def linear_bf16(a, weight, bias, out, act, accumulate) -> bool:
     else:
         if LIBRARY_LINEAR and TILED_CONFIG == 0:
             space = _library_workspace(a.device)
+            # (an activation the library has no epilogue for: a pass of its own over the products)
+            apart = act in _ACTIVATIONS_APART and m >= ACTIVATION_APART_FROM_ROWS and n >= ACTIVATION_APART_FROM_COLUMNS \
+                and out.dtype == torch.bfloat16 and n % 8 == 0 and out.stride(0) % 8 == 0 and m <= 65535
             status = handle.ka_linear_library_bf16(a.data_ptr(), a.stride(0), weight.data_ptr(), weight.stride(0),
                                                    _ptr(bias), out.data_ptr(), _OUT_CODE[out.dtype], out.stride(0), m, n, k,
-                                                   act, int(accumulate), space.data_ptr(), space.numel(), stream_ptr())
+                                                   0 if apart else act, int(accumulate), space.data_ptr(), space.numel(), stream_ptr())
             if status == 0:
+                if apart:
+                    core.activate_rows(out, act)
                 return True
             if status < 0:
                 _check(status)
@@ -900,7 +912,6 @@ def experts_feed_forward_bf16(h, pairs, down, chosen, hidden, y, act, workspace)
     leaves the hidden rows in list order, the second writes fp32 ``y`` ``[n top, dim]`` at the pairs' own rows. ``pairs``
     ``[E, 2 hidden, dim]`` (not gated: ``[E, hidden, dim]``), ``down`` ``[E, dim, hidden]``, ``chosen`` int32 ``[n, top]``; ``hidden`` is not used (the list's hidden rows
     live in the workspace). False: not covered (sizes that are no multiple of 16, alignment), nothing was run."""
-    from . import core
     n, top = chosen.shape
     n_experts, n_pair_rows, dim = pairs.shape
     ff = down.shape[2]

@@ -193,12 +193,12 @@ class LatentAttention(Mixer):
         if brings and max(brings) < self.LIFT_FROM_TOKENS:
             return None, True
         some_stay = not brings or min(brings) < self.LIFT_FROM_TOKENS
-        key = f"latent.lift_plan.{cache.group}"
-        if key not in batch.host:
+        made, key = batch.host.setdefault("made_once", {}), f"latent.lift_plan.{cache.group}"
+        if key not in made:
             from ..ops import fast
-            batch.host[key] = fast.latent_expand_plan(batch, group, str(cache.group), int(self.window), self.LIFT_FROM_TOKENS,
-                                                      int(cache.k.shape[0]))
-        return batch.host[key], some_stay
+            made[key] = fast.latent_expand_plan(batch, group, str(cache.group), int(self.window), self.LIFT_FROM_TOKENS,
+                                                int(cache.k.shape[0]))
+        return made[key], some_stay
 
     def _stays_in_fast_kernels(self, batch) -> bool:
         """Whether the rows that are not lifted run in kernels that pass over the lifted ones: a list of blocks of queries of

@@ -455,6 +455,20 @@ def test_latents_made_ready_without_a_rotated_part():
         assert float(got[[0, 1, 2, 6, 7, 8, 9, 10, 11, 13, 14, 15]].abs().max()) == 0.0
 
 
+@pytest.mark.parametrize("rows, columns", [(1, 40), (9, 40), (70, 1024), (255, 1024), (256, 1024), (300, 1048), (300, 1020)])
+def test_relu_squared_in_every_linear_kernel(rows, columns):
+    """In the epilogue of this package's kernels, and as a pass over the vendor library's product for large outputs; columns
+    behind the output's in its buffer are left alone."""
+    from kestrel_amd.ops.linear import activation_code, linear
+
+    gen = torch.Generator().manual_seed(rows)
+    a, w = torch.randn(rows, 64, generator=gen).bfloat16(), (torch.randn(columns, 64, generator=gen) * 0.2).bfloat16()
+    buffer = torch.full((rows, columns + 8), 7.0, dtype=torch.bfloat16, device=DEV)
+    linear(a.to(DEV), w.to(DEV), None, buffer[:, :columns], act=activation_code("relu_squared"))
+    _near(buffer[:, :columns], plain.relu_squared(a.double() @ w.double().T), torch.bfloat16, "relu squared", atol=1e-4)
+    assert bool((buffer[:, columns:] == 7.0).all())
+
+
 def test_the_matrix_core_kernels_run_where_sizes_allow():
     """In bfloat16 the models whose sizes the matrix-core kernels take run them for prompts, and the model of odd sizes the
     generic ones where they do not fit."""
@@ -575,6 +589,42 @@ def test_mixed_batches_in_reused_pages_and_slots(name, dtype, graphs):
     assert runner.cache.free_slots == 4
 
 
+@pytest.mark.parametrize("dtype", DTYPES, ids=DTYPE_IDS)
+@pytest.mark.parametrize("name", NAMES)
+def test_replayed_steps_of_any_shape(name, dtype):
+    """Steps replayed as graphs, one graph serving steps of different make-up in turn: long portions (whose latents are
+    lifted) alone, beside short ones and single tokens, and steps of the same number of tokens without a long one; in
+    pages that were given back and hold NaN."""
+    from tests.test_mixed_graphs_gpu import replay_last_places
+
+    folder = cases.folder_for(name, dtype)
+    runner = _runner(folder, dtype, n_pages=40, max_requests=8, graphs=True)
+    assert runner.mixed_graphs
+    lengths = {"a": 190, "b": 112, "c": 150, "d": 75, "e": 128, "f": 120, "g": 70, "h": 66}
+    steps = [[("a", 100), ("b", 20)],                              # all but the last: 65 to 128 tokens, the same graph
+             [("a", 1), ("b", 60), ("c", 50)],                     # no portion long enough
+             [("a", 64), ("b", 1), ("c", 2), ("d", 60)],           # one just long enough
+             [("a", 1), ("c", 98), ("d", 15)],
+             [("a", 24), ("b", 31), ("e", 63)],                    # a, b end; one token short of long
+             [("e", 65), ("f", 55)],
+             [("f", 65), ("g", 2)],
+             [("g", 68)],
+             [("h", 66)]]
+    reqs = {tag: Request(tag, _ids(folder, 800 + i, n)) for i, (tag, n) in enumerate(lengths.items())}
+    got = replay_last_places(runner, reqs, steps, wanted=2)
+    assert runner.mixed_graph_replays == len(steps) and len(runner._mixed) == 1, sorted(runner._mixed)
+    for tag, req in reqs.items():
+        places = sorted(got[tag])
+        want = _expected(folder, req.ids)
+        bound = None
+        if dtype == torch.bfloat16:
+            bound = torch.clamp(_what_rounding_does(folder, req.ids)[places], min=0.04)
+        diff = torch.stack([got[tag][p] for p in places]).double().cpu() - want[places]
+        diff = diff - diff.mean(dim=-1, keepdim=True)
+        rms = diff.pow(2).mean(dim=-1).sqrt() / want[places].std(dim=-1, unbiased=False)
+        assert bool((rms <= (5e-5 if bound is None else bound)).all()), (name, tag, places, rms)
+
+
 def test_a_slot_used_again_starts_from_nothing():
     """The cache manager clears a slot's state at admission: the second request in a slot must not see the first's."""
     folder = cases.model_dir("P")
@@ -632,13 +682,13 @@ def test_greedy_generation_through_the_entry_point(name, dtype):
 
     folder = cases.folder_for(name, dtype)
     config, weights = cases.config_of(folder), cases.stored_weights(folder)
-    prompts = [_ids(folder, 600 + i, n) for i, n in enumerate([5, 17, 33, 70])]
+    prompts = [_ids(folder, 600 + i, n) for i, n in enumerate([5, 17, 33, 120])]
     n_new = 24
     slack = 1e-4 if dtype == "float32" else 8e-2
     for graphs, depth in ((False, 1), (True, 2)):
         engine = InferenceEngine.create_sync(RuntimeConfig(model_path=folder, dtype=dtype, max_batch_size=4, kv_cache_pages=40,
-                                                           max_num_batched_tokens=48, enable_graphs=graphs, pipeline_depth=depth,
-                                                           max_seq_len=128))
+                                                           max_num_batched_tokens=96, enable_graphs=graphs, pipeline_depth=depth,
+                                                           max_seq_len=160))
         try:
             results = engine.generate_batch_sync(prompts, max_new_tokens=n_new, temperature=0.0, stop_ids=())
         finally:
