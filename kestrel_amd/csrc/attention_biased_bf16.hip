@@ -37,7 +37,10 @@
 // the head size is a run-time number, the queries of the workgroup's 32 columns lie in LDS instead of registers (every
 // wave reads them from there, 16 bytes a lane and step), keys are streamed step by step, and a workgroup owns a slice of
 // 128 value channels (blockIdx.z counts the slices; every slice computes the scores again, which costs little where
-// the keys are what is waited for).
+// the keys are what is waited for). Where values lie in the keys, a wave takes its tile's key rows through a piece of LDS of its
+// own, 128 channels at a time: loads of whole lines (four keys' 256 bytes an instruction, where the product's own operand
+// layout would ask for a piece of each of 32 rows), the operands of the scores from LDS, and, the slice's own channels
+// being taken last, the values of the slice from the same piece, eight keys of a channel a lane.
 //
 // A workgroup owns 32 columns of the score product and one kv head. In a step with prompt portions a
 // column is a query of a block of 32 consecutive tokens of one row and one query head (the host lists the
@@ -60,6 +63,8 @@ constexpr int AB_PAGE = 16;
 constexpr int AB_TILE = 32;                 // keys per tile: two pages
 constexpr int AB_COLS = 32;                 // columns (queries) per workgroup
 constexpr float AB_SLACK = 8.0f;            // powers of two a maximum may grow before the outputs are rescaled
+constexpr int AB_STRIP = 128;               // channels of a key row that the wide form stages at a time
+constexpr int AB_STRIP_PITCH = AB_STRIP + 8;
 constexpr float AB_LOG2E = 1.4426950408889634f;
 
 __device__ __forceinline__ float ab_max_halves(float x) {
@@ -139,7 +144,11 @@ attn_biased_kernel(const bf16_t* __restrict__ q, long q_row_stride, const bf16_t
 
     // queries: the column operand of the score product, held for the whole loop
     ab_bf16x8 qreg[WIDE ? 1 : NK];
-    ab_bf16x8* q_lds = reinterpret_cast<ab_bf16x8*>(mrg + (size_t)(n_waves / 2) * REC * KA_WAVE);     // [hd / 16][64]
+    // (the wide form: the waves' strips of keys, which the merge area lies over, then the queries)
+    constexpr int STRIP_FLOATS = AB_TILE * AB_STRIP_PITCH / 2;
+    const int over = WIDE && values_in_keys ? max((n_waves / 2) * REC * KA_WAVE, n_waves * STRIP_FLOATS) : (n_waves / 2) * REC * KA_WAVE;
+    ab_bf16x8* q_lds = reinterpret_cast<ab_bf16x8*>(mrg + over);                                      // [hd / 16][64]
+    bf16_t* strip = reinterpret_cast<bf16_t*>(mrg + (size_t)wave * STRIP_FLOATS);                     // [32][AB_STRIP_PITCH]
     {
         const bf16_t* qp = q + (size_t)tok * q_row_stride + (size_t)head * HD + half * 8;
         if constexpr (WIDE) {
@@ -203,7 +212,9 @@ attn_biased_kernel(const bf16_t* __restrict__ q, long q_row_stride, const bf16_t
                 for (int c = 0; c < NK; ++c) kr[c] = *reinterpret_cast<const ab_bf16x8*>(kp + c * 16);
             }
             ab_bf16x8 vr[2][NV];
-            if (values_in_keys) {
+            if (WIDE && values_in_keys) {
+                // (from the wave's strip, below)
+            } else if (values_in_keys) {
                 // eight consecutive keys of one channel: a column of the row-major key page
 #pragma unroll
                 for (int p = 0; p < 2; ++p) {
@@ -224,7 +235,51 @@ attn_biased_kernel(const bf16_t* __restrict__ q, long q_row_stride, const bf16_t
             ab_floatx16 s;
 #pragma unroll
             for (int i = 0; i < 16; ++i) s[i] = 0.f;
-            if constexpr (WIDE) {
+            if (WIDE && values_in_keys) {
+                const int strips = (HD + AB_STRIP - 1) / AB_STRIP, own = v0 / AB_STRIP;
+                const bf16_t* rows[8];                 // what this lane fetches of a strip: 16 bytes of eight keys
+                ab_bf16x8 st[8];
+                const int piece = lane % 16;
+#pragma unroll
+                for (int u = 0; u < 8; ++u) {
+                    const int key = u * 4 + lane / 16;
+                    rows[u] = k_cache + (size_t)pg[u / 4] * k_page + k_head + (size_t)(key & 15) * HD;
+                }
+                auto strip_at = [&](int turn_of) { return turn_of < own ? turn_of : (turn_of + 1 < strips ? turn_of + 1 : own); };
+                auto fetch = [&](int x) {
+                    const int ch = min(x * AB_STRIP + piece * 8, HD - 8);       // (behind the last channel: not multiplied)
+#pragma unroll
+                    for (int u = 0; u < 8; ++u) st[u] = *reinterpret_cast<const ab_bf16x8*>(rows[u] + ch);
+                };
+                fetch(strip_at(0));
+                for (int turn_of = 0; turn_of < strips; ++turn_of) {
+                    const int x = strip_at(turn_of);
+                    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+                    for (int u = 0; u < 8; ++u)
+                        *reinterpret_cast<ab_bf16x8*>(strip + (u * 4 + lane / 16) * AB_STRIP_PITCH + piece * 8) = st[u];
+                    if (turn_of + 1 < strips) fetch(strip_at(turn_of + 1));
+                    __builtin_amdgcn_wave_barrier();
+                    const int steps = min(AB_STRIP / 16, HD / 16 - x * (AB_STRIP / 16));
+                    if (steps == AB_STRIP / 16) {
+#pragma unroll
+                        for (int c = 0; c < AB_STRIP / 16; ++c)
+                            s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const ab_bf16x8*>(strip + krow * AB_STRIP_PITCH + c * 16 + half * 8),
+                                                                        q_lds[(x * (AB_STRIP / 16) + c) * KA_WAVE + lane], s, 0, 0, 0);
+                    } else {
+                        for (int c = 0; c < steps; ++c)
+                            s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const ab_bf16x8*>(strip + krow * AB_STRIP_PITCH + c * 16 + half * 8),
+                                                                        q_lds[(x * (AB_STRIP / 16) + c) * KA_WAVE + lane], s, 0, 0, 0);
+                    }
+                }
+                // the strip holds the slice's own channels now: eight consecutive keys of one channel a lane
+#pragma unroll
+                for (int p = 0; p < 2; ++p)
+#pragma unroll
+                    for (int b = 0; b < NV; ++b)
+#pragma unroll
+                        for (int e = 0; e < 8; ++e) vr[p][b][e] = strip[(p * AB_PAGE + half * 8 + e) * AB_STRIP_PITCH + vch[b] - v0];
+            } else if constexpr (WIDE) {
                 // (eight steps' keys are asked for before the first is multiplied: one trip to memory for all of them)
                 constexpr int AHEAD = 8;
                 int c = 0;
@@ -315,6 +370,7 @@ attn_biased_kernel(const bf16_t* __restrict__ q, long q_row_stride, const bf16_t
     }
     l = ab_sum_halves(l);                       // the column's whole sum, in both of its lanes
 
+    if (WIDE && values_in_keys) __syncthreads();        // (every wave is done with its strip)
     // merge the waves in a tree: at step s the waves with bit s set hand over to the wave 2^s below
     for (int step = 1; step < n_waves; step <<= 1) {
         const bool gives = (wave & (2 * step - 1)) == step, takes = (wave & (2 * step - 1)) == 0 && wave + step < n_waves;
@@ -541,7 +597,9 @@ KA_API int ka_attention_biased_bf16(const void* q, long q_row_stride, const void
     const int nk = wide ? 0 : hd / 16, nv = wide ? 4 : (hdv + 31) / 32;
     if (wide) grid.z = (hdv + 127) / 128;
     // the merge area of the waves and, in the wide form, the queries of the 32 columns
-    const size_t lds = (size_t)(waves / 2) * (16 * nv + 2) * KA_WAVE * sizeof(float) + (wide ? (size_t)hd * 32 * sizeof(bf16_t) : 0);
+    const size_t merge = (size_t)(waves / 2) * (16 * nv + 2) * KA_WAVE * sizeof(float), strips = (size_t)waves * AB_TILE * AB_STRIP_PITCH * sizeof(bf16_t);
+    const size_t lds = (wide && values_in_keys && strips > merge ? strips : merge) + (wide ? (size_t)hd * 32 * sizeof(bf16_t) : 0);
+    KA_CHECK(lds <= 160 * 1024, "%s: heads of %d channels do not fit in LDS", who, hd);
 #define AB_LAUNCH(NK, NV)                                                                                                  \
     if (nk == NK && nv == NV) {                                                                                            \
         static bool sized = false;                                                                                         \
