@@ -227,13 +227,15 @@ def bogivik_models(size: dict, positions: int):
 
 def design_facts(net):
     """What the roofline of any model of the package needs, read off its plan: the weights of its linears (every matrix
-    but the embedding table), and per layer of its attention ``(multiply-adds a query spends per key it sees, numbers
+    but the embedding table, unless that is the head), and per layer of its attention ``(multiply-adds a query spends per key it sees, numbers
     the cache holds per key, window, chunk, kept first keys)`` and the sizes of its matrix memory (heads, key and value size)."""
     from types import SimpleNamespace
 
     plan = net.plan
     embedding = plan.names["embedding"]
     linear = sum(int(__import__("math").prod(p.shape)) for name, p in net.params().items() if p.role == "matrix" and name != embedding)
+    if plan.tied_head:
+        linear += plan.dim * plan.vocab_size         # (the embedding table is the head's weight)
     attention, memory, experts = [], [], []
 
     def walk(spec):

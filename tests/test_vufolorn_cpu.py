@@ -59,7 +59,7 @@ def test_what_the_configuration_reader_refuses(edit, message):
 def test_tensor_names_and_shapes():
     params = DecoderModel(_plan("P")).params()
     assert params["embed"].shape == (300, 128) and params["embed.norm"].shape == (128,) and params["final.norm"].shape == (128,)
-    assert params["loop.step"].shape == (3, 128) and "head" not in params
+    assert params["loop.step"].shape == (2, 128) and "head" not in params
     for name in ("norm1", "norm1b", "ls1", "norm2", "norm2b", "ls2"):
         assert params["l0." + name].shape == (128,)
     # latent attention: queries directly, one gate number per head
@@ -81,13 +81,13 @@ def test_tensor_names_and_shapes():
 def test_schedule_junction_cache_groups_and_state():
     plan = _plan("P")
     assert [(e.layer, e.before, e.passage) for e in plan.schedule] == [
-        (0, None, 0), (1, "loop_step", 0), (2, None, 0), (1, "loop_step", 1), (2, None, 1), (1, "loop_step", 2), (2, None, 2), (3, None, 0)]
+        (0, None, 0), (1, "loop_step", 0), (2, None, 0), (1, "loop_step", 1), (2, None, 1), (3, None, 0)]
     assert plan.tied_head and plan.junctions["loop_step"].embedding_from == 1 and plan.embedding_norm is not None
     needs = DecoderModel(plan).cache_needs()
     manager = CacheManager(needs, 16, 40, 3)
     assert len(manager.groups) == 2                       # one per window and latent size; every pass has pages of its own
-    assert sorted(len(g.entries) for g in manager.groups) == [1, 3]
-    assert [s is not None for _c, s, _r in needs] == [False, True, False, True, False, True, False, True]
+    assert sorted(len(g.entries) for g in manager.groups) == [1, 2]
+    assert [s is not None for _c, s, _r in needs] == [False, True, False, True, False, True]
     assert needs[1][1].shape == (4 * 40 * 32,) and needs[1][1].dtype == "float32"
     assert _plan("R").junctions == {} and "loop.step" in _plan("R").ignored_prefixes
     plan = _plan("S")

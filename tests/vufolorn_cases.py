@@ -38,22 +38,22 @@ def _config(vocab, width, eps, layers, loop=None):
 
 
 CONFIGS: Dict[str, dict] = {
-    # sizes the matrix-core kernels take; a loop over both kinds, run three times; two windows, of two and a half pages and of
+    # sizes the matrix-core kernels take; a loop over both kinds, run twice; two windows, of two and a half pages and of
     # one and a half, so two cache groups
     "P": _config(300, 128, 1e-5, [
         latent(4, 16, 24, 64, 0.3, 40, experts(6, 48, 2, 32)),
         lightning(32, 40, (0.3, 0.9, 0.99, 0.9995), experts(6, 48, 2, 32)),
         latent(2, 32, 64, 48, 0.25, 24, experts(5, 64, 3, 80)),
         lightning(48, 64, (1.0, 0.7), None),
-    ], (1, 3, 3)),
+    ], (1, 3, 2)),
     # sizes that fit none of the fast kernels' alignments: a window shorter than a page, a layer that sees every key, layers
-    # without a feed-forward, no shared expert, one choice, a loop of one layer, heads of one channel
+    # without a feed-forward, no shared expert, one choice, a loop of one layer run three times, heads of one channel
     "Q": _config(211, 100, 1e-6, [
         lightning(10, 7, (0.95, 0.2, 0.999, 0.5, 0.98), experts(5, 20, 1)),
         latent(3, 12, 10, 36, 0.35, 7, experts(3, 24, 2, 20)),
         latent(5, 20, 6, 20, 0.25, None, None),
         lightning(1, 33, (0.9, 0.99, 0.8), experts(4, 24, 4, 36)),
-    ], (1, 2, 2)),
+    ], (1, 2, 3)),
     # the largest heads; latents wider than the attention kernel keeps in registers; windows of whole pages; more than 64
     # choices' worth of experts; no loop
     "R": _config(190, 256, 1e-3, [
