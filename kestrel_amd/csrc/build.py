@@ -29,12 +29,12 @@ ARCH = "gfx950"
 # library name -> its sources. "core" is all a float32 run needs; "fast" holds the
 # bf16 MFMA kernels of serving.
 LIBRARIES: Dict[str, List[str]] = {
-    "core": ["ka_error.hip", "elementwise.hip", "gemm_generic.hip", "attention_generic.hip", "mixer_parts.hip", "sequence_parts.hip", "recurrent_parts.hip", "linear_attention.hip", "experts.hip",
+    "core": ["ka_error.hip", "elementwise.hip", "gemm_generic.hip", "attention_generic.hip", "mixer_parts.hip", "sequence_parts.hip", "recurrent_parts.hip", "linear_attention.hip", "stream_parts.hip", "experts.hip",
              "sampling.hip", "peaks.hip"],
     "fast": ["ka_error.hip", "gemm_bf16.hip", "gemv_bf16.hip", "attention_bf16.hip", "attention_biased_bf16.hip", "heads_linear_bf16.hip", "matrix_memory_bf16.hip", "linear_attention_bf16.hip", "latent_expand_bf16.hip", "decode_beside.hip", "experts_bf16.hip",
              "gemm_library.hip"],
 }
-HEADERS = ["ka_common.h", "ka_partials.h", "ka_no_alloc.h", "ka_attention_decode.h", "ka_skinny.h", "ka_rows.h", "ka_listed_tiles.h"]
+HEADERS = ["ka_common.h", "ka_partials.h", "ka_no_alloc.h", "ka_attention_decode.h", "ka_skinny.h", "ka_rows.h", "ka_decay.h", "ka_listed_tiles.h"]
 
 # Libraries of the ROCm installation that a library of ours is linked against.
 LINK_LIBRARIES: Dict[str, List[str]] = {"fast": ["hipblaslt"]}

@@ -26,22 +26,24 @@ __device__ __forceinline__ void ex_wave_argmax(float& v, int& i) {
 
 // ----------------------------------------------------------------------------
 // The router's choice, a wave per token. logits fp32 [n, >= R] (rows `stride` apart), R router outputs.
-//     s = softmax(logits);  choice = s + correction (correction optional)
-//     n_groups > 0: the outputs form n_groups equal groups of neighbours, a group's score is its largest choice score,
-//       and only outputs of the `keep` best groups can be chosen;
+//     s = softmax(logits), or sigmoid(logits) one by one;  choice = s + correction (correction optional)
+//     n_groups > 0: the outputs form n_groups equal groups of neighbours, a group's score is its largest choice score, or the
+//       sum of its two largest (group_best 2), and only outputs of the `keep` best groups can be chosen;
 //     the `top` outputs with the largest choice scores are chosen (the lower index wins a tie);
 //     weights: their s divided by the sum of the chosen s (+ 1e-20), times scale.
-// by_logits: the choice goes by the logits themselves (no correction, no groups); the weights are the softmax over the chosen
+// mode 0: softmax scores, 2: sigmoid scores; 1 (by the logits): the choice goes by the logits themselves (no correction, no groups); the weights are the softmax over the chosen
 // logits, times scale.
-// chosen int32 [n, top], weights fp32 [n, top].
+// chosen int32 [n, top], weights fp32 [n, top]; always >= 0: the rows are one longer and end in that output with weight 1 (a
+// feed-forward that every token uses, laid behind the experts).
 // ----------------------------------------------------------------------------
 __global__ void __launch_bounds__(KA_WAVE)
 route_kernel(const float* __restrict__ logits, long stride, const float* __restrict__ correction, int R, int top, int n_groups,
-             int keep, float scale, int by_logits, int* __restrict__ chosen, float* __restrict__ weights) {
+             int keep, int group_best, float scale, int mode, int always, int* __restrict__ chosen, float* __restrict__ weights) {
     __shared__ float choice_s[EX_MAX_OUTPUTS];
     __shared__ float group_s[EX_MAX_GROUPS];
     __shared__ int allowed_s[EX_MAX_GROUPS];
     const int t = blockIdx.x, lane = threadIdx.x;
+    const bool by_logits = mode == 1, sigmoids = mode == 2;
     const float* z = logits + (size_t)t * stride;
     float s[EX_PER_LANE], c[EX_PER_LANE];
     float top_z = -INFINITY;
@@ -56,7 +58,8 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
 #pragma unroll
     for (int q = 0; q < EX_PER_LANE; ++q) {
         c[q] = s[q];
-        s[q] = lane + q * KA_WAVE < R ? expf(s[q] - top_z) : 0.f;
+        if (sigmoids) s[q] = lane + q * KA_WAVE < R ? 1.0f / (1.0f + expf(-s[q])) : 0.f;
+        else s[q] = lane + q * KA_WAVE < R ? expf(s[q] - top_z) : 0.f;
         total += s[q];
     }
     total = ka_wave_sum(total);
@@ -64,7 +67,7 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
     for (int q = 0; q < EX_PER_LANE; ++q) {
         const int r = lane + q * KA_WAVE;
         if (by_logits) continue;      // (the largest logit is among the chosen: e^(z - top) over their sum is their softmax)
-        s[q] = s[q] / total;
+        if (!sigmoids) s[q] = s[q] / total;
         c[q] = r < R ? s[q] + (correction ? correction[r] : 0.f) : -INFINITY;
         if (r < R) choice_s[r] = c[q];
     }
@@ -72,9 +75,13 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
         const int per = R / n_groups;
         __syncthreads();
         if (lane < n_groups) {
-            float best = -INFINITY;
-            for (int m = 0; m < per; ++m) best = fmaxf(best, choice_s[lane * per + m]);
-            group_s[lane] = best;
+            float best = -INFINITY, second = -INFINITY;
+            for (int m = 0; m < per; ++m) {
+                const float v = choice_s[lane * per + m];
+                second = fmaxf(second, fminf(v, best));
+                best = fmaxf(best, v);
+            }
+            group_s[lane] = group_best == 2 && per > 1 ? best + second : best;
             allowed_s[lane] = 0;
         }
         __syncthreads();
@@ -123,24 +130,30 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
             mine_i = i;
         }
     }
+    const size_t at = (size_t)t * (always >= 0 ? top + 1 : top);
     if (lane < top) {
-        chosen[(size_t)t * top + lane] = mine_i;
-        weights[(size_t)t * top + lane] = mine_w / (by_logits ? sum : sum + 1e-20f) * scale;
+        chosen[at + lane] = mine_i;
+        weights[at + lane] = mine_w / (by_logits ? sum : sum + 1e-20f) * scale;
+    }
+    if (always >= 0 && lane == 0) {
+        chosen[at + top] = always;
+        weights[at + top] = 1.f;
     }
 }
 
 KA_API int ka_route(const float* logits, long stride, const float* correction, int n, int R, int top, int n_groups, int keep,
-                    float scale, int by_logits, int* chosen, float* weights, hipStream_t stream) {
+                    int group_best, float scale, int mode, int always, int* chosen, float* weights, hipStream_t stream) {
     const char* who = "ka_route";
-    KA_CHECK(!by_logits || (n_groups == 0 && correction == nullptr), "%s: a choice by the logits alone has no groups and no correction", who);
+    KA_CHECK(mode >= 0 && mode <= 2 && (group_best == 1 || group_best == 2), "%s: unknown mode %d or group score %d", who, mode, group_best);
+    KA_CHECK(mode != 1 || (n_groups == 0 && correction == nullptr), "%s: a choice by the logits alone has no groups and no correction", who);
     KA_CHECK(n >= 0 && R > 0 && R <= EX_MAX_OUTPUTS && stride >= R, "%s: %d router outputs (at most %d)", who, R, EX_MAX_OUTPUTS);
     KA_CHECK(top > 0 && top <= R && top <= KA_WAVE, "%s: %d choices of %d", who, top, R);
     KA_CHECK(n_groups >= 0 && n_groups <= EX_MAX_GROUPS && (n_groups == 0 || (R % n_groups == 0 && keep > 0 && keep <= n_groups)),
              "%s: %d groups of which %d are kept do not divide %d outputs", who, n_groups, keep, R);
     KA_CHECK(n_groups == 0 || keep * (R / n_groups) >= top, "%s: %d kept groups hold fewer than %d outputs", who, keep, top);
     if (n == 0) return 0;
-    hipLaunchKernelGGL(route_kernel, dim3(n), dim3(KA_WAVE), 0, stream, logits, stride, correction, R, top, n_groups, keep, scale,
-                       by_logits, chosen, weights);
+    hipLaunchKernelGGL(route_kernel, dim3(n), dim3(KA_WAVE), 0, stream, logits, stride, correction, R, top, n_groups, keep, group_best,
+                       scale, mode, always, chosen, weights);
     KA_LAUNCH_CHECK();
     return 0;
 }
@@ -187,7 +200,7 @@ __device__ __forceinline__ void ex_dots(const T* const (&w)[R], const float* __r
 template <typename T>
 __global__ void __launch_bounds__(256)
 experts_linear_kernel(const T* __restrict__ a, long a_stride, int a_div, const T* __restrict__ W, const int* __restrict__ chosen,
-                      int E, int N, int K, int act, void* __restrict__ out, long out_stride, int out_f32) {
+                      int E, int N, int K, int act, KaGateClamp clamp, void* __restrict__ out, long out_stride, int out_f32) {
     extern __shared__ float row[];
     const int p = blockIdx.y;
     const int e = chosen[p];
@@ -212,8 +225,8 @@ experts_linear_kernel(const T* __restrict__ a, long a_stride, int a_div, const T
             for (int r = 0; r < 4; ++r) w[r] = We + (size_t)min(2 * (j0 + q) + r, N - 1) * K;     // (rows past the end: not stored)
             float s[4];
             ex_dots<T, 4>(w, row, K, lane, vectors, s);
-            y[q] = ka_activate(act, s[0]) * s[1];
-            y[q + 1] = ka_activate(act, s[2]) * s[3];
+            y[q] = ka_gate_product<false>(act, clamp, s[0], s[1]);
+            y[q + 1] = ka_gate_product<false>(act, clamp, s[2], s[3]);
         }
     } else {
         const T* w[ROWS];
@@ -235,8 +248,11 @@ experts_linear_kernel(const T* __restrict__ a, long a_stride, int a_div, const T
 }
 
 KA_API int ka_experts_linear(const void* a, long a_stride, int a_div, const void* W, int dtype, const int* chosen, int n_pairs,
-                             int E, int N, int K, int act, void* out, long out_stride, int out_f32, hipStream_t stream) {
+                             int E, int N, int K, int act, int clamped, float limit, float slope, float shift, void* out,
+                             long out_stride, int out_f32, hipStream_t stream) {
     const char* who = "ka_experts_linear";
+    KA_CHECK(!clamped || ka_act_gated(act), "%s: clamps are a gated linear's", who);
+    const KaGateClamp clamp{clamped, limit, slope, shift};
     KA_CHECK(n_pairs >= 0 && E > 0 && N > 0 && K > 0 && a_div > 0, "%s: bad sizes", who);
     KA_CHECK(ka_act_known(act) && (!ka_act_gated(act) || N % 2 == 0), "%s: unknown activation %d, or a gated linear of %d rows", who, act, N);
     KA_CHECK(dtype == KA_F32 || dtype == KA_BF16, "%s: unsupported dtype %d", who, dtype);
@@ -248,10 +264,10 @@ KA_API int ka_experts_linear(const void* a, long a_stride, int a_div, const void
     const size_t lds = (size_t)K * sizeof(float);
     if (dtype == KA_F32)
         hipLaunchKernelGGL(experts_linear_kernel<float>, grid, dim3(256), lds, stream, (const float*)a, a_stride, a_div, (const float*)W,
-                           chosen, E, N, K, act, out, out_stride, out_f32);
+                           chosen, E, N, K, act, clamp, out, out_stride, out_f32);
     else
         hipLaunchKernelGGL(experts_linear_kernel<bf16_t>, grid, dim3(256), lds, stream, (const bf16_t*)a, a_stride, a_div, (const bf16_t*)W,
-                           chosen, E, N, K, act, out, out_stride, out_f32);
+                           chosen, E, N, K, act, clamp, out, out_stride, out_f32);
     KA_LAUNCH_CHECK();
     return 0;
 }

@@ -5,7 +5,8 @@
 //  * the first linear gathers: list row i holds pair p = sorted[i] (-1: an unused row), whose input is row p / gather_div
 //    of `a`; its output goes to row i of `out` (the hidden rows stay in list order);
 //  * the second linear scatters: its input is row i of `a`, its output goes to row p of `out`;
-//  * gated (KA_ACT_GATED): weight rows 2j and 2j + 1 are gate and value of output j, as in every gated linear here.
+//  * gated (KA_ACT_GATED): weight rows 2j and 2j + 1 are gate and value of output j, as in every gated linear here, with or
+//    without clamps (KaGateClamp).
 //
 // The weights are the row operand: a lane ends with outputs of ONE list row, four neighbours at a time, so the pair of a
 // gated output meets in a lane's registers.
@@ -17,8 +18,8 @@ typedef __attribute__((ext_vector_type(2))) __bf16 eb_bf16x2;
 template <bool TAIL>
 __global__ void __launch_bounds__(256)
 experts_gemm_kernel(const bf16_t* __restrict__ a, long lda, int gather_div, const bf16_t* __restrict__ W, const int* __restrict__ sorted,
-                    const int* __restrict__ tile_expert, int N, int K, int act, void* __restrict__ out, long ldo, int scatter,
-                    int out_f32) {
+                    const int* __restrict__ tile_expert, int N, int K, int act, KaGateClamp clamp, void* __restrict__ out, long ldo,
+                    int scatter, int out_f32) {
     extern __shared__ __attribute__((aligned(16))) bf16_t eb_lds[];
     const int tile = blockIdx.y;
     const int e = tile_expert[tile];
@@ -53,11 +54,11 @@ experts_gemm_kernel(const bf16_t* __restrict__ a, long lda, int gather_div, cons
                 if (gated) {
                     if (o + 3 < N) {
                         eb_bf16x2 y;
-                        y[0] = (bf16_t)(ka_activate_fast(act, acc_here[g4 * 4]) * acc_here[g4 * 4 + 1]);
-                        y[1] = (bf16_t)(ka_activate_fast(act, acc_here[g4 * 4 + 2]) * acc_here[g4 * 4 + 3]);
+                        y[0] = (bf16_t)ka_gate_product<true>(act, clamp, acc_here[g4 * 4], acc_here[g4 * 4 + 1]);
+                        y[1] = (bf16_t)ka_gate_product<true>(act, clamp, acc_here[g4 * 4 + 2], acc_here[g4 * 4 + 3]);
                         *reinterpret_cast<eb_bf16x2*>(reinterpret_cast<bf16_t*>(out) + row * ldo + o / 2) = y;
                     } else if (o + 1 < N) {
-                        reinterpret_cast<bf16_t*>(out)[row * ldo + o / 2] = (bf16_t)(ka_activate_fast(act, acc_here[g4 * 4]) * acc_here[g4 * 4 + 1]);
+                        reinterpret_cast<bf16_t*>(out)[row * ldo + o / 2] = (bf16_t)ka_gate_product<true>(act, clamp, acc_here[g4 * 4], acc_here[g4 * 4 + 1]);
                     }
                 } else if (out_f32) {
                     float* op = reinterpret_cast<float*>(out) + row * ldo + o;
@@ -96,9 +97,11 @@ KA_API int ka_experts_gemm_supported(long lda, int N, int K, long ldo, int act, 
 }
 
 KA_API int ka_experts_gemm_bf16(const void* a, long lda, int gather_div, const void* W, const int* sorted, const int* tile_expert,
-                                int n_tiles, int N, int K, int act, void* out, long ldo, int scatter, int out_f32,
-                                hipStream_t stream) {
+                                int n_tiles, int N, int K, int act, int clamped, float limit, float slope, float shift, void* out,
+                                long ldo, int scatter, int out_f32, hipStream_t stream) {
     const char* who = "ka_experts_gemm_bf16";
+    KA_CHECK(!clamped || ka_act_gated(act), "%s: clamps are a gated linear's", who);
+    const KaGateClamp clamp{clamped, limit, slope, shift};
     KA_CHECK(n_tiles >= 0 && n_tiles <= 65535 && gather_div >= 0, "%s: bad sizes (%d tiles)", who, n_tiles);
     KA_CHECK(ka_act_known(act) && ka_experts_gemm_supported(lda, N, K, ldo, act, out_f32), "%s: sizes N=%d K=%d not covered", who, N, K);
     KA_CHECK((uintptr_t)a % 16 == 0 && (uintptr_t)W % 16 == 0 && (uintptr_t)out % 16 == 0, "%s: operands must be 16-byte aligned", who);
@@ -112,10 +115,10 @@ KA_API int ka_experts_gemm_bf16(const void* a, long lda, int gather_div, const v
     }
     if (K % KL_SLAB == 0)
         hipLaunchKernelGGL(experts_gemm_kernel<false>, grid, dim3(256), KL_LDS_BYTES, stream, (const bf16_t*)a, lda, gather_div, (const bf16_t*)W,
-                           sorted, tile_expert, N, K, act, out, ldo, scatter, out_f32);
+                           sorted, tile_expert, N, K, act, clamp, out, ldo, scatter, out_f32);
     else
         hipLaunchKernelGGL(experts_gemm_kernel<true>, grid, dim3(256), KL_LDS_BYTES, stream, (const bf16_t*)a, lda, gather_div, (const bf16_t*)W,
-                           sorted, tile_expert, N, K, act, out, ldo, scatter, out_f32);
+                           sorted, tile_expert, N, K, act, clamp, out, ldo, scatter, out_f32);
     KA_LAUNCH_CHECK();
     return 0;
 }

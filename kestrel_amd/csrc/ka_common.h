@@ -192,6 +192,23 @@ __device__ __forceinline__ float ka_activate_fast(int act, float x) {
     }
 }
 
+// The pair of a gated linear with clamps, for the kernels that carry its constants: on, a pair (g, u) becomes
+// g' sigmoid(slope g') (u' + shift) with g' = min(g, limit) and u' = clamp(u, -limit, limit), whatever the activation's code.
+struct KaGateClamp {
+    int on;
+    float limit, slope, shift;
+};
+
+template <bool FAST>
+__device__ __forceinline__ float ka_gate_product(int act, const KaGateClamp& c, float g, float u) {
+    if (c.on) {
+        g = fminf(g, c.limit);
+        u = fminf(fmaxf(u, -c.limit), c.limit) + c.shift;
+        return FAST ? g * __fdividef(1.0f, 1.0f + __expf(-c.slope * g)) * u : g / (1.0f + expf(-c.slope * g)) * u;
+    }
+    return (FAST ? ka_activate_fast(act, g) : ka_activate(act, g)) * u;
+}
+
 // The epilogue of a gated linear layer for the sums (biases added) of the weight rows n .. n + COUNT - 1 of
 // output row m, n even: out[m][(n + 2p) / 2] = act(v[2p]) * v[2p + 1] for every pair inside N. FAST: the
 // activations on the hardware's exponential (the kernels that write bf16), else the library's.

@@ -1,6 +1,7 @@
 // Kernels of attention without a softmax, run as a recurrence: the walk over a row's tokens one by one, and the norm of
-// what it reads. fp32 or bf16 storage of what the projections made; activations, the state and all sums are fp32.
+// what it reads. fp32 or bf16 storage of what the projections made; activations, decays, the state and all sums are fp32.
 #include "ka_common.h"
+#include "ka_decay.h"
 
 constexpr int LA_THREADS = 256;
 
@@ -12,6 +13,9 @@ constexpr int LA_THREADS = 256;
 // times) of NJ value channels in registers; a read-out is a sum over the LI lanes of a group inside the vector unit.
 // Nothing passes between waves. One launch takes whatever a step holds: a prompt, a portion, single tokens. The next
 // token's numbers are asked for before the current token's sums. A row without a request (slot < 0) gets zeros.
+//
+// GATED: instead of one decay per head, a decay per key channel computed from the token, a_i = sigmoid(pre_i)^(1 / tau) with
+// fp32 pre [n, H d] (ka_decay.h), and queries times q_scale.
 // ----------------------------------------------------------------------------
 struct LinearAttentionArgs {
     const void* q;
@@ -25,6 +29,8 @@ struct LinearAttentionArgs {
     const int* row_slot;
     float* raw;             // [n, H dv]
     int H, d, dv, act, vectors;
+    const float* pre;       // GATED: [n, H d]
+    float per_tau, q_scale; // GATED: 1 / tau
 };
 
 template <typename T>
@@ -49,7 +55,7 @@ __device__ __forceinline__ float4 la_act4(int act, float4 x) {
     return make_float4(la_act<T>(act, x.x), la_act<T>(act, x.y), la_act<T>(act, x.z), la_act<T>(act, x.w));
 }
 
-template <typename T, int LI, int NV, int NJ>
+template <typename T, int LI, int NV, int NJ, bool GATED>
 __global__ void __launch_bounds__(LA_THREADS) linear_attention_kernel(LinearAttentionArgs a) {
     constexpr int JW = LA_THREADS / LI;
     const int head = blockIdx.x, row = blockIdx.y, tid = threadIdx.x;
@@ -74,7 +80,7 @@ __global__ void __launch_bounds__(LA_THREADS) linear_attention_kernel(LinearAtte
     const T* qp = reinterpret_cast<const T*>(a.q) + (size_t)head * d;
     const T* kp = reinterpret_cast<const T*>(a.k) + (size_t)head * d;
     const T* vp = reinterpret_cast<const T*>(a.v) + (size_t)head * dv;
-    const float keep = a.decay[head];
+    const float keep = GATED ? 1.f : a.decay[head];
     float4 S[NJ][NV];
     int jc[NJ];             // (value channels behind the last are clamped for the loads and not stored)
 #pragma unroll
@@ -84,7 +90,7 @@ __global__ void __launch_bounds__(LA_THREADS) linear_attention_kernel(LinearAtte
 #pragma unroll
         for (int u = 0; u < NV; ++u) S[m][u] = la_four(S_mem + (size_t)jc[m] * d, (u * LI + li) * 4, d, d % 4 == 0);
     }
-    float4 qn[NV], kn[NV];
+    float4 qn[NV], kn[NV], zn[GATED ? NV : 1];
     float vn[NJ];
     auto fetch = [&](int t) {
         const size_t at = (size_t)t * a.stride;
@@ -92,18 +98,24 @@ __global__ void __launch_bounds__(LA_THREADS) linear_attention_kernel(LinearAtte
         for (int u = 0; u < NV; ++u) {
             qn[u] = la_four(qp + at, (u * LI + li) * 4, d, vectors);
             kn[u] = la_four(kp + at, (u * LI + li) * 4, d, vectors);
+            if constexpr (GATED) zn[u] = la_four(a.pre + (size_t)t * a.H * d + (size_t)head * d, (u * LI + li) * 4, d, vectors);
         }
 #pragma unroll
         for (int m = 0; m < NJ; ++m) vn[m] = ka_to_float(vp[at + jc[m]]);
     };
     fetch(t0);
     for (int t = t0; t < t1; ++t) {
-        float4 q[NV], k[NV];
+        float4 q[NV], k[NV], w[GATED ? NV : 1];
         float v[NJ];
 #pragma unroll
         for (int u = 0; u < NV; ++u) {
             q[u] = la_act4<T>(a.act, qn[u]);
             k[u] = la_act4<T>(a.act, kn[u]);
+            if constexpr (GATED) {
+                q[u] = make_float4(q[u].x * a.q_scale, q[u].y * a.q_scale, q[u].z * a.q_scale, q[u].w * a.q_scale);
+                w[u] = make_float4(ka_decay<sizeof(T) == 2>(zn[u].x, a.per_tau), ka_decay<sizeof(T) == 2>(zn[u].y, a.per_tau),
+                                   ka_decay<sizeof(T) == 2>(zn[u].z, a.per_tau), ka_decay<sizeof(T) == 2>(zn[u].w, a.per_tau));
+            }
         }
 #pragma unroll
         for (int m = 0; m < NJ; ++m) v[m] = la_act<T>(a.act, vn[m]);
@@ -114,10 +126,11 @@ __global__ void __launch_bounds__(LA_THREADS) linear_attention_kernel(LinearAtte
 #pragma unroll
             for (int u = 0; u < NV; ++u) {
                 float4& s = S[m][u];
-                s.x = fmaf(keep, s.x, k[u].x * v[m]);
-                s.y = fmaf(keep, s.y, k[u].y * v[m]);
-                s.z = fmaf(keep, s.z, k[u].z * v[m]);
-                s.w = fmaf(keep, s.w, k[u].w * v[m]);
+                const float4 f = GATED ? w[GATED ? u : 0] : make_float4(keep, keep, keep, keep);
+                s.x = fmaf(f.x, s.x, k[u].x * v[m]);
+                s.y = fmaf(f.y, s.y, k[u].y * v[m]);
+                s.z = fmaf(f.z, s.z, k[u].z * v[m]);
+                s.w = fmaf(f.w, s.w, k[u].w * v[m]);
                 acc = fmaf(q[u].x, s.x, acc);
                 acc = fmaf(q[u].y, s.y, acc);
                 acc = fmaf(q[u].z, s.z, acc);
@@ -152,10 +165,31 @@ constexpr int LA_MAX_D = 512;
 
 KA_API int ka_linear_attention_supported(int d, int dv) { return d > 0 && d <= LA_MAX_D && dv > 0 ? 1 : 0; }
 
+template <bool GATED>
+static int la_run(const char* who, const LinearAttentionArgs& given, int dtype, int n, int n_rows, hipStream_t stream);
+
 KA_API int ka_linear_attention(const void* q, const void* k, const void* v, long stride, int dtype, const float* decay, float* state,
                                long state_stride, const int* cu_q, const int* row_slot, float* raw, int n, int n_rows, int H, int d,
                                int dv, int act, hipStream_t stream) {
-    const char* who = "ka_linear_attention";
+    return la_run<false>("ka_linear_attention", {q, k, v, stride, decay, state, state_stride, cu_q, row_slot, raw, H, d, dv, act, 0, nullptr, 0.f, 1.f},
+                         dtype, n, n_rows, stream);
+}
+
+// pre: fp32 [n, H d]; a key channel's decay is sigmoid(pre)^(1 / tau).
+KA_API int ka_gated_linear_attention(const void* q, const void* k, const void* v, long stride, int dtype, const float* pre, float tau,
+                                     float q_scale, float* state, long state_stride, const int* cu_q, const int* row_slot, float* raw,
+                                     int n, int n_rows, int H, int d, int dv, hipStream_t stream) {
+    const char* who = "ka_gated_linear_attention";
+    KA_CHECK(tau > 0.f && pre != nullptr, "%s: a decay needs its pre-activations and a positive tau", who);
+    return la_run<true>(who, {q, k, v, stride, nullptr, state, state_stride, cu_q, row_slot, raw, H, d, dv, KA_ACT_NONE, 0, pre, 1.f / tau, q_scale},
+                        dtype, n, n_rows, stream);
+}
+
+template <bool GATED>
+static int la_run(const char* who, const LinearAttentionArgs& given, int dtype, int n, int n_rows, hipStream_t stream) {
+    const int H = given.H, d = given.d, dv = given.dv, act = given.act;
+    const long stride = given.stride, state_stride = given.state_stride;
+    const void *q = given.q, *k = given.k, *state = given.state;
     KA_CHECK(n >= 0 && n_rows >= 0 && H > 0 && ka_linear_attention_supported(d, dv), "%s: heads of %d x %d channels are not covered (keys up to %d)", who, d, dv, LA_MAX_D);
     KA_CHECK(dtype == KA_F32 || dtype == KA_BF16, "%s: unsupported dtype %d", who, dtype);
     KA_CHECK(ka_act_known(act) && !ka_act_gated(act), "%s: unknown activation %d", who, act);
@@ -165,13 +199,14 @@ KA_API int ka_linear_attention(const void* q, const void* k, const void* v, long
     if (n == 0 || n_rows == 0) return 0;
     const size_t align = dtype == KA_F32 ? 16 : 8;
     const int vectors = d % 4 == 0 && stride % 4 == 0 && (uintptr_t)q % align == 0 && (uintptr_t)k % align == 0;
-    LinearAttentionArgs a{q, k, v, stride, decay, state, state_stride, cu_q, row_slot, raw, H, d, dv, act, vectors};
+    LinearAttentionArgs a = given;
+    a.vectors = vectors && (!GATED || (uintptr_t)given.pre % 16 == 0);
     const int lanes = d <= 32 ? 8 : d <= 64 ? 16 : d <= 128 ? 32 : 64;
     // (few workgroups: a value channel a group of lanes; many: four, so that a token's keys and queries serve four)
     const int jw = LA_THREADS / lanes;
     const int nj = (long)H * n_rows * ka_cdiv(dv, jw) >= 8L * ka_compute_units() ? 4 : 1;
     const dim3 grid(H, n_rows, ka_cdiv(dv, jw * nj));
-#define LA_LAUNCH(T, LI, NV, NJ) hipLaunchKernelGGL((linear_attention_kernel<T, LI, NV, NJ>), grid, dim3(LA_THREADS), 0, stream, a)
+#define LA_LAUNCH(T, LI, NV, NJ) hipLaunchKernelGGL((linear_attention_kernel<T, LI, NV, NJ, GATED>), grid, dim3(LA_THREADS), 0, stream, a)
 #define LA_LAUNCH_NJ(T, LI, NV)          \
     if (nj == 4) LA_LAUNCH(T, LI, NV, 4); \
     else LA_LAUNCH(T, LI, NV, 1)
@@ -283,6 +318,73 @@ KA_API int ka_gated_rmsnorm(const float* x, const float* gain, const void* gate,
     if (dtype == KA_F32) { LA_NORM_ALL(float) } else { LA_NORM_ALL(bf16_t) }
 #undef LA_NORM_ALL
 #undef LA_NORM
+    KA_LAUNCH_CHECK();
+    return 0;
+}
+
+// ----------------------------------------------------------------------------
+// Every head of fp32 read-outs raw [n, H, dv] normalised by itself: out = o / sqrt(mean(o^2) + eps) * gain [dv] (shared by the
+// heads) * silu(gate): a group of 16 lanes per (token, head).
+// ----------------------------------------------------------------------------
+template <typename T, bool VECTORS>
+__global__ void __launch_bounds__(LA_THREADS)
+heads_rmsnorm_kernel(const float* __restrict__ raw, const float* __restrict__ gain, const T* __restrict__ gate, long gate_stride,
+                     T* __restrict__ out, long out_stride, long pairs, int H, int dv, float eps) {
+    constexpr int LANES = 16;
+    const long pair = (long)blockIdx.x * (LA_THREADS / LANES) + threadIdx.x / LANES;
+    const int lane = threadIdx.x % LANES;
+    const bool live = pair < pairs;
+    const long t = live ? pair / H : 0;
+    const int head = live ? (int)(pair % H) : 0;
+    const float* o = raw + (t * H + head) * dv;
+    const T* g = gate + t * gate_stride + (size_t)head * dv;
+    T* dst = out + t * out_stride + (size_t)head * dv;
+    float ss = 0.f;
+    if constexpr (VECTORS) {
+        for (int c = lane * 4; c < dv; c += LANES * 4) {
+            const float4 v = *reinterpret_cast<const float4*>(o + c);
+            ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+        }
+    } else {
+        for (int c = lane; c < dv; c += LANES) ss = fmaf(o[c], o[c], ss);
+    }
+    ss = ka_lanes_reduce<1, LANES>(ss, KaSum{});
+    if (!live) return;
+    const float r = 1.0f / sqrtf(ss / (float)dv + eps);
+    if constexpr (VECTORS) {
+        typedef __attribute__((ext_vector_type(4))) T vec;
+        for (int c = lane * 4; c < dv; c += LANES * 4) {
+            const float4 v = *reinterpret_cast<const float4*>(o + c), w = *reinterpret_cast<const float4*>(gain + c);
+            const vec x = *reinterpret_cast<const vec*>(g + c);
+            const float y[4] = {v.x * w.x, v.y * w.y, v.z * w.z, v.w * w.w};
+            vec b;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) b[e] = ka_from_float<T>(y[e] * r * la_act<T>(KA_ACT_SILU, ka_to_float(x[e])));
+            *reinterpret_cast<vec*>(dst + c) = b;
+        }
+    } else {
+        for (int c = lane; c < dv; c += LANES)
+            dst[c] = ka_from_float<T>(o[c] * r * gain[c] * la_act<T>(KA_ACT_SILU, ka_to_float(g[c])));
+    }
+}
+
+KA_API int ka_heads_rmsnorm(const float* raw, const float* gain, const void* gate, long gate_stride, void* out, long out_stride, int dtype,
+                            int n, int H, int dv, float eps, hipStream_t stream) {
+    const char* who = "ka_heads_rmsnorm";
+    KA_CHECK(n >= 0 && H > 0 && dv > 0 && eps >= 0.f && gate_stride >= (long)H * dv && out_stride >= (long)H * dv, "%s: bad sizes", who);
+    KA_CHECK(dtype == KA_F32 || dtype == KA_BF16, "%s: unsupported dtype %d", who, dtype);
+    KA_CHECK(gain != nullptr && gate != nullptr, "%s: gains and gate missing", who);
+    if (n == 0) return 0;
+    const size_t align = dtype == KA_F32 ? 16 : 8;
+    const bool vectors = dv % 4 == 0 && gate_stride % 4 == 0 && out_stride % 4 == 0 && (uintptr_t)raw % 16 == 0 && (uintptr_t)gain % 16 == 0 &&
+                         (uintptr_t)gate % align == 0 && (uintptr_t)out % align == 0;
+    const long pairs = (long)n * H;
+    const dim3 grid(ka_cdiv(pairs, LA_THREADS / 16));
+#define LA_HEADS(T, V) \
+    hipLaunchKernelGGL((heads_rmsnorm_kernel<T, V>), grid, dim3(LA_THREADS), 0, stream, raw, gain, (const T*)gate, gate_stride, (T*)out, out_stride, pairs, H, dv, eps)
+    if (dtype == KA_F32) { if (vectors) LA_HEADS(float, true); else LA_HEADS(float, false); }
+    else { if (vectors) LA_HEADS(bf16_t, true); else LA_HEADS(bf16_t, false); }
+#undef LA_HEADS
     KA_LAUNCH_CHECK();
     return 0;
 }

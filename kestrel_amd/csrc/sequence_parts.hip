@@ -91,8 +91,9 @@ KA_API int ka_pair_embed(const void* table, int table_dtype, const int* ids, con
 //   y_t[c] = sum_j taps[c, j] * u_(t - K + 1 + j)[c]
 // where inputs before the first token of this step come from `state` [slots + 1, K - 1, C] fp32 (the last K - 1 projected
 // rows of the sequence, zero for a new one) and K = 0 means no convolution. Rotation of the first `rot` channels of every
-// query and key head by place * freqs[i] (interleaved 1: channels 2i, 2i + 1; 0: i, i + rot / 2). Queries go to `q_out`,
-// keys into [pages, Hk, page_size, hd], values into [pages, Hv, hdv, page_size]; a negative slot caches nothing.
+// query and key head by place * freqs[i] (interleaved 1: channels 2i, 2i + 1; 0: i, i + rot / 2). normed: every query and
+// key head is divided by its root mean square sqrt(mean(y^2) + eps) (before or behind the rotation, which turns pairs of
+// its own channels, is the same). Queries go to `q_out`, keys into [pages, Hk, page_size, hd], values into [pages, Hv, hdv, page_size]; a negative slot caches nothing.
 // The second kernel then moves the state on (it reads `u`, which the first leaves as it was).
 // ----------------------------------------------------------------------------
 struct ConvArgs {
@@ -100,6 +101,7 @@ struct ConvArgs {
     long u_stride;
     const float* taps;
     float* state;
+    long state_stride;      // from one slot's rows to the next slot's
     int K, C;
     const int* cu_q;
     const int* row_slot;
@@ -113,6 +115,13 @@ struct ConvArgs {
     int Hq, Hk, hd, Hv, hdv, page_size;
     const float* freqs;
     int rot, interleaved;
+    int normed;
+    float eps;
+    // the form of eight channels a thread: the tokens cut into runs of at most page_size (null: every token by itself), and
+    // whether every row brings one token (its thread then moves the state on as well)
+    const int* run_first;
+    const int* run_count;
+    int moves_state;
 };
 
 template <typename T>
@@ -124,7 +133,7 @@ __device__ __forceinline__ float sp_conv_at(const ConvArgs& a, int t, int local,
         const int back = a.K - 1 - j;           // how many places before t
         float v = 0.f;
         if (back <= local) v = ka_to_float(u[(size_t)(t - back) * a.u_stride + c]);
-        else if (slot >= 0) v = a.state[((size_t)slot * (a.K - 1) + (local - back + a.K - 1)) * a.C + c];
+        else if (slot >= 0) v = a.state[(size_t)slot * a.state_stride + (size_t)(local - back + a.K - 1) * a.C + c];
         acc += a.taps[(size_t)c * a.K + j] * v;
     }
     return acc;
@@ -182,6 +191,263 @@ __global__ void __launch_bounds__(SP_THREADS) conv_prepare_kernel(ConvArgs a) {
     }
 }
 
+// Queries and keys normalised head by head: a wave per head in turns, a workgroup per token. The convolution of a channel is
+// computed twice, for the head's sum of squares and for its result.
+template <typename T>
+__global__ void __launch_bounds__(SP_THREADS) conv_prepare_normed_kernel(ConvArgs a) {
+    __shared__ float cs[SP_MAX_ROT / 2], sn[SP_MAX_ROT / 2];
+    const int t = blockIdx.x, wave = threadIdx.x / KA_WAVE, lane = threadIdx.x % KA_WAVE;
+    const int r = a.token_row[t];
+    const int local = t - a.cu_q[r];
+    const int slot = a.row_slot[r];
+    const int Cq = a.Hq * a.hd, Ck = a.Hk * a.hd, heads = a.Hq + a.Hk;
+    const float place = (float)a.positions[t];
+    const int at = a.slots ? a.slots[t] : -1;
+    const int page = at >= 0 ? at / a.page_size : 0, off = at >= 0 ? at % a.page_size : 0;
+    const int half = a.rot / 2;
+    if (a.freqs) {
+        for (int i = threadIdx.x; i < half; i += SP_THREADS) sincosf(place * a.freqs[i], &sn[i], &cs[i]);
+        __syncthreads();
+    }
+    for (int h = blockIdx.y * (SP_THREADS / KA_WAVE) + wave; h < heads; h += gridDim.y * (SP_THREADS / KA_WAVE)) {
+        float ss = 0.f;
+        for (int d = lane; d < a.hd; d += KA_WAVE) {
+            const float y = sp_conv_at<T>(a, t, local, slot, h * a.hd + d);
+            ss = fmaf(y, y, ss);
+        }
+        const float scale = 1.0f / sqrtf(ka_wave_sum(ss) / (float)a.hd + a.eps);
+        T* dst;
+        if (h < a.Hq) dst = reinterpret_cast<T*>(a.q_out) + (size_t)t * a.q_stride + (size_t)h * a.hd;
+        else if (at < 0) continue;
+        else dst = reinterpret_cast<T*>(a.k_cache) + (((size_t)page * a.Hk + (h - a.Hq)) * a.page_size + off) * a.hd;
+        for (int d = lane; d < a.hd; d += KA_WAVE) {
+            const int c = h * a.hd + d;
+            const float y = sp_conv_at<T>(a, t, local, slot, c) * scale;
+            if (a.freqs && d < a.rot) {
+                const bool first = a.interleaved ? (d & 1) == 0 : d < half;
+                if (!first) continue;                   // (written by the thread of its partner)
+                const int step = a.interleaved ? 1 : half;
+                const int i = a.interleaved ? d / 2 : d;
+                const float other = sp_conv_at<T>(a, t, local, slot, c + step) * scale;
+                dst[d] = ka_from_float<T>(y * cs[i] - other * sn[i]);
+                dst[d + step] = ka_from_float<T>(other * cs[i] + y * sn[i]);
+            } else {
+                dst[d] = ka_from_float<T>(y);
+            }
+        }
+    }
+    if (at < 0) return;
+    for (int e = blockIdx.y * SP_THREADS + threadIdx.x; e < a.Hv * a.hdv; e += gridDim.y * SP_THREADS) {
+        const int head = e / a.hdv, d = e % a.hdv;
+        reinterpret_cast<T*>(a.v_cache)[(((size_t)page * a.Hv + head) * a.hdv + d) * a.page_size + off] =
+            ka_from_float<T>(sp_conv_at<T>(a, t, local, slot, Cq + Ck + e));
+    }
+}
+
+// The same for bf16 rows, up to SP_WIDE_TAPS taps, and query and key heads of 8 LPH channels, LPH a power of two: a thread
+// keeps eight neighbouring channels, their taps and the rows the taps still reach in registers and walks over the tokens of a
+// run, one 16-byte load a token; a head's sum of squares meets inside its LPH lanes, and the lanes of a rotated pair of
+// halves exchange their numbers. Grid (blocks of 2,048 channels: queries and keys, then values; runs). Values of a run that
+// fills a page leave as 32 bytes a channel. rot is a multiple of 16 for pairs of halves.
+typedef __attribute__((ext_vector_type(8))) __bf16 sp_bf16x8;
+typedef __attribute__((ext_vector_type(4))) float sp_floatx4;
+constexpr int SP_WIDE_TAPS = 4;
+constexpr int SP_WIDE_RUN = 16;                     // tokens of a run at most
+constexpr int SP_WIDE_MAX_ROT = 256;
+
+// Whatever `back` = 1 .. SP_WIDE_TAPS - 1 rows before token t hold of channels c .. c + 7, into hist[back - 1].
+__device__ __forceinline__ void sp_wide_history(const ConvArgs& a, int t, int local, int slot, int c, float (&hist)[SP_WIDE_TAPS - 1][8]) {
+    const bf16_t* u = reinterpret_cast<const bf16_t*>(a.u);
+#pragma unroll
+    for (int back = 1; back < SP_WIDE_TAPS; ++back) {
+        if (back < a.K && back <= local) {
+            const sp_bf16x8 x = *reinterpret_cast<const sp_bf16x8*>(u + (size_t)(t - back) * a.u_stride + c);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) hist[back - 1][e] = (float)x[e];
+        } else if (back < a.K && slot >= 0) {
+            const float* st = a.state + (size_t)slot * a.state_stride + (size_t)(local - back + a.K - 1) * a.C + c;
+            const sp_floatx4 x0 = *reinterpret_cast<const sp_floatx4*>(st), x1 = *reinterpret_cast<const sp_floatx4*>(st + 4);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) { hist[back - 1][e] = x0[e]; hist[back - 1][4 + e] = x1[e]; }
+        } else {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) hist[back - 1][e] = 0.f;
+        }
+    }
+}
+
+template <int LPH>
+__global__ void __launch_bounds__(SP_THREADS) conv_prepare_wide_kernel(ConvArgs a) {
+    __shared__ float cs[SP_WIDE_RUN][SP_WIDE_MAX_ROT / 2], sn[SP_WIDE_RUN][SP_WIDE_MAX_ROT / 2];
+    constexpr int HD = 8 * LPH;
+    const int tid = threadIdx.x;
+    const int Cqk = (a.Hq + a.Hk) * HD, Cv = a.Hv * a.hdv;
+    const int qk_blocks = (Cqk + 8 * SP_THREADS - 1) / (8 * SP_THREADS);
+    const bool values = (int)blockIdx.x >= qk_blocks;
+    const int first = a.run_first ? a.run_first[blockIdx.y] : (int)blockIdx.y;
+    const int count = a.run_first ? min(a.run_count[blockIdx.y], SP_WIDE_RUN) : 1;
+    if (count <= 0) return;
+    const int half = a.rot / 2;
+    if (a.freqs && !values) {
+        for (int e = tid; e < count * half; e += SP_THREADS)
+            sincosf((float)a.positions[first + e / half] * a.freqs[e % half], &sn[e / half][e % half], &cs[e / half][e % half]);
+        __syncthreads();
+    }
+    // (threads behind the last channel do the work of the first ones and store nothing: all lanes of a wave stay together)
+    const int mine = ((int)blockIdx.x - (values ? qk_blocks : 0)) * SP_THREADS + tid;
+    const bool live = 8 * mine < (values ? Cv : Cqk);
+    const int within = live ? 8 * mine : 8 * (tid % LPH);
+    const int c = values ? Cqk + (live ? 8 * mine : 0) : within;
+    float w[SP_WIDE_TAPS][8];               // w[back]: the tap that reads `back` rows before
+#pragma unroll
+    for (int back = 0; back < SP_WIDE_TAPS; ++back)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) w[back][e] = back < a.K ? a.taps[(size_t)(c + e) * a.K + (a.K - 1 - back)] : 0.f;
+    const bf16_t* u = reinterpret_cast<const bf16_t*>(a.u);
+    float hist[SP_WIDE_TAPS - 1][8];
+    int row = -1, slot = -1;
+    // the rows before token t, where it is not the one behind the last token of its row
+    auto enter = [&](int t) {
+        const int r = a.token_row[t];
+        if (r == row) return;
+        row = r;
+        slot = a.row_slot[r];
+        sp_wide_history(a, t, t - a.cu_q[r], slot, c, hist);
+    };
+    auto convolve = [&](int t, float (&y)[8]) {
+        const sp_bf16x8 x = *reinterpret_cast<const sp_bf16x8*>(u + (size_t)t * a.u_stride + c);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            float s = 0.f;
+#pragma unroll
+            for (int back = SP_WIDE_TAPS - 1; back >= 1; --back) s = fmaf(w[back][e], hist[back - 1][e], s);
+            y[e] = fmaf(w[0][e], (float)x[e], s);
+        }
+#pragma unroll
+        for (int back = SP_WIDE_TAPS - 2; back >= 1; --back)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) hist[back][e] = hist[back - 1][e];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) hist[0][e] = (float)x[e];
+    };
+    // (the row's only token: entry s of the state is now what stands K - 2 - s rows before the next token's predecessor)
+    auto move_state = [&]() {
+        if (!a.moves_state || slot < 0 || !live) return;
+        float* st = a.state + (size_t)slot * a.state_stride + c;
+#pragma unroll
+        for (int back = 0; back < SP_WIDE_TAPS - 1; ++back) {
+            if (back >= a.K - 1) continue;
+            sp_floatx4 v0, v1;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) { v0[e] = hist[back][e]; v1[e] = hist[back][4 + e]; }
+            *reinterpret_cast<sp_floatx4*>(st + (size_t)(a.K - 2 - back) * a.C) = v0;
+            *reinterpret_cast<sp_floatx4*>(st + (size_t)(a.K - 2 - back) * a.C + 4) = v1;
+        }
+    };
+    if (!values) {
+        const int head = within / HD, sub = within % HD / 8;
+        const bool is_q = head < a.Hq;
+        for (int i = 0; i < count; ++i) {
+            const int t = first + i;
+            float y[8];
+            enter(t);
+            convolve(t, y);
+            if (a.normed) {
+                float ss = 0.f;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) ss = fmaf(y[e], y[e], ss);
+                const float scale = 1.0f / sqrtf(ka_lanes_reduce<1, LPH>(ss, KaSum{}) / (float)HD + a.eps);
+#pragma unroll
+                for (int e = 0; e < 8; ++e) y[e] *= scale;
+            }
+            if (a.freqs && a.interleaved) {
+#pragma unroll
+                for (int p = 0; p < 4; ++p) {
+                    const int j = sub * 4 + p;
+                    if (2 * j < a.rot) {
+                        const float v0 = y[2 * p], v1 = y[2 * p + 1];
+                        y[2 * p] = v0 * cs[i][j] - v1 * sn[i][j];
+                        y[2 * p + 1] = v1 * cs[i][j] + v0 * sn[i][j];
+                    }
+                }
+            } else if (a.freqs) {
+                const int apart = a.rot / 16;
+                const bool low = sub < apart, turned = sub < 2 * apart;
+                const int partner = (tid % KA_WAVE) + (low ? apart : -apart);
+                float other[8];
+#pragma unroll
+                for (int e = 0; e < 8; ++e) other[e] = __shfl(y[e], turned ? partner : tid % KA_WAVE);
+                if (turned) {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) {
+                        const int j = (low ? sub : sub - apart) * 8 + e;
+                        y[e] = low ? y[e] * cs[i][j] - other[e] * sn[i][j] : y[e] * cs[i][j] + other[e] * sn[i][j];
+                    }
+                }
+            }
+            sp_bf16x8 o;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) o[e] = (bf16_t)y[e];
+            if (!live) continue;
+            if (is_q) {
+                *reinterpret_cast<sp_bf16x8*>(reinterpret_cast<bf16_t*>(a.q_out) + (size_t)t * a.q_stride + within) = o;
+            } else {
+                const int at = a.slots ? a.slots[t] : -1;
+                if (at >= 0)
+                    *reinterpret_cast<sp_bf16x8*>(reinterpret_cast<bf16_t*>(a.k_cache) + (((size_t)(at / a.page_size) * a.Hk + (head - a.Hq)) * a.page_size +
+                                                  at % a.page_size) * HD + sub * 8) = o;
+            }
+        }
+        move_state();
+        return;
+    }
+    if (!live) return;                              // (nothing below meets other lanes)
+    const int vc = 8 * mine, vhead = vc / a.hdv, vd = vc % a.hdv;
+    bf16_t* vbase = reinterpret_cast<bf16_t*>(a.v_cache);
+    const int at0 = a.slots ? a.slots[first] : -1;
+    if (count == SP_WIDE_RUN && a.page_size == SP_WIDE_RUN && at0 >= 0 && at0 % SP_WIDE_RUN == 0 && a.slots[first + SP_WIDE_RUN - 1] == at0 + SP_WIDE_RUN - 1) {
+        sp_bf16x8 page[8][2];
+        enter(first);
+#pragma unroll
+        for (int i = 0; i < SP_WIDE_RUN; ++i) {
+            float y[8];
+            convolve(first + i, y);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) page[e][i / 8][i % 8] = (bf16_t)y[e];
+        }
+        bf16_t* dst = vbase + (((size_t)(at0 / SP_WIDE_RUN) * a.Hv + vhead) * a.hdv + vd) * SP_WIDE_RUN;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            *reinterpret_cast<sp_bf16x8*>(dst + (size_t)e * SP_WIDE_RUN) = page[e][0];
+            *reinterpret_cast<sp_bf16x8*>(dst + (size_t)e * SP_WIDE_RUN + 8) = page[e][1];
+        }
+        return;
+    }
+    for (int i = 0; i < count; ++i) {
+        float y[8];
+        enter(first + i);
+        convolve(first + i, y);
+        const int at = a.slots ? a.slots[first + i] : -1;
+        if (at < 0) continue;
+        bf16_t* dst = vbase + (((size_t)(at / a.page_size) * a.Hv + vhead) * a.hdv + vd) * a.page_size + at % a.page_size;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) dst[(size_t)e * a.page_size] = (bf16_t)y[e];
+    }
+    move_state();
+}
+
+// Whether the form of eight channels a thread covers the call; 0, or the lanes of a head.
+static int sp_wide_lanes(const ConvArgs& a, int dtype, int n_runs) {
+    const int lanes = a.hd / 8;
+    if (dtype != KA_BF16 || a.K < 1 || a.K > SP_WIDE_TAPS || a.hd % 8 != 0 || a.hdv % 8 != 0 || n_runs > 65535) return 0;
+    if (lanes != 2 && lanes != 4 && lanes != 8 && lanes != 16 && lanes != 32) return 0;
+    if (a.freqs && (a.rot > SP_WIDE_MAX_ROT || (!a.interleaved && a.rot % 16 != 0))) return 0;
+    if ((uintptr_t)a.u % 16 != 0 || a.u_stride % 8 != 0 || (uintptr_t)a.q_out % 16 != 0 || a.q_stride % 8 != 0) return 0;
+    if ((uintptr_t)a.k_cache % 16 != 0 || (uintptr_t)a.v_cache % 16 != 0) return 0;
+    if (a.K > 1 && ((uintptr_t)a.state % 16 != 0 || a.state_stride % 4 != 0)) return 0;
+    return lanes;
+}
+
 template <typename T>
 __global__ void __launch_bounds__(SP_THREADS) conv_state_kernel(ConvArgs a) {
     const int r = blockIdx.x;
@@ -190,7 +456,7 @@ __global__ void __launch_bounds__(SP_THREADS) conv_state_kernel(ConvArgs a) {
     if (slot < 0 || q <= 0) return;
     const T* u = reinterpret_cast<const T*>(a.u);
     const int keep = a.K - 1;
-    float* st = a.state + (size_t)slot * keep * a.C;
+    float* st = a.state + (size_t)slot * a.state_stride;
     {
         const int c = blockIdx.y * SP_THREADS + threadIdx.x;
         if (c >= a.C) return;
@@ -206,8 +472,10 @@ __global__ void __launch_bounds__(SP_THREADS) conv_state_kernel(ConvArgs a) {
 KA_API int ka_conv_prepare(const void* u, int dtype, long u_stride, const float* taps, float* state, int K, const int* cu_q,
                            const int* row_slot, const int* token_row, const int* positions, const int* slots, void* q_out,
                            long q_stride, void* k_cache, void* v_cache, int n, int n_rows, int Hq, int Hk, int hd, int Hv, int hdv,
-                           int page_size, const float* freqs, int rot, int interleaved, hipStream_t stream) {
-    KA_CHECK(n >= 0 && n_rows >= 0 && Hq > 0 && Hk > 0 && hd > 0 && Hv > 0 && hdv > 0 && page_size > 0 && K >= 0, "ka_conv_prepare: bad sizes");
+                           int page_size, const float* freqs, int rot, int interleaved, long state_stride, int normed, float eps,
+                           const int* run_first, const int* run_count, int n_runs, int single_tokens, hipStream_t stream) {
+    KA_CHECK(n >= 0 && n_rows >= 0 && Hq > 0 && Hk > 0 && hd > 0 && Hv > 0 && hdv > 0 && page_size > 0 && K >= 0 && eps >= 0.f, "ka_conv_prepare: bad sizes");
+    KA_CHECK((run_first == nullptr) == (run_count == nullptr) && n_runs >= 0, "ka_conv_prepare: runs are two lists");
     KA_CHECK(dtype == KA_F32 || dtype == KA_BF16, "ka_conv_prepare: unsupported dtype %d", dtype);
     KA_CHECK(K == 0 || taps != nullptr, "ka_conv_prepare: taps missing");
     KA_CHECK(K <= 1 || state != nullptr, "ka_conv_prepare: a convolution of %d taps needs its state", K);
@@ -221,13 +489,37 @@ KA_API int ka_conv_prepare(const void* u, int dtype, long u_stride, const float*
     a.q_out = q_out; a.q_stride = q_stride; a.k_cache = k_cache; a.v_cache = v_cache;
     a.Hq = Hq; a.Hk = Hk; a.hd = hd; a.Hv = Hv; a.hdv = hdv; a.page_size = page_size;
     a.freqs = freqs; a.rot = freqs ? rot : 0; a.interleaved = interleaved;
+    a.state_stride = state_stride; a.normed = normed; a.eps = eps;
+    KA_CHECK(K <= 1 || state_stride >= (long)(K - 1) * a.C, "ka_conv_prepare: the state's rows are too short");
+    a.run_first = nullptr; a.run_count = nullptr; a.moves_state = 0;
     if (n == 0) return 0;
     const int blocks = (a.C + SP_THREADS - 1) / SP_THREADS;
     KA_CHECK(blocks <= 65535, "ka_conv_prepare: too many channels %d", a.C);
-    if (dtype == KA_F32) hipLaunchKernelGGL(conv_prepare_kernel<float>, dim3(n, n > SP_SPREAD_TOKENS ? 1 : blocks), dim3(SP_THREADS), 0, stream, a);
+    // (a step of one token a row, or without lists of runs: every token is a run of its own)
+    const bool by_runs = run_first != nullptr && !single_tokens && page_size <= SP_WIDE_RUN;
+    const int grid_runs = by_runs ? n_runs : n;
+    const int wide = sp_wide_lanes(a, dtype, grid_runs);
+    if (wide) {
+        if (by_runs) { a.run_first = run_first; a.run_count = run_count; }
+        a.moves_state = K > 1 && single_tokens;
+        const int per = 8 * SP_THREADS;
+        const dim3 grid(ka_cdiv((long)(Hq + Hk) * hd, per) + ka_cdiv((long)Hv * hdv, per), grid_runs);
+        switch (wide) {
+            case 2: hipLaunchKernelGGL(conv_prepare_wide_kernel<2>, grid, dim3(SP_THREADS), 0, stream, a); break;
+            case 4: hipLaunchKernelGGL(conv_prepare_wide_kernel<4>, grid, dim3(SP_THREADS), 0, stream, a); break;
+            case 8: hipLaunchKernelGGL(conv_prepare_wide_kernel<8>, grid, dim3(SP_THREADS), 0, stream, a); break;
+            case 16: hipLaunchKernelGGL(conv_prepare_wide_kernel<16>, grid, dim3(SP_THREADS), 0, stream, a); break;
+            default: hipLaunchKernelGGL(conv_prepare_wide_kernel<32>, grid, dim3(SP_THREADS), 0, stream, a); break;
+        }
+    } else if (normed) {
+        const dim3 grid(n, n > SP_SPREAD_TOKENS ? 1 : ka_cdiv(Hq + Hk, SP_THREADS / KA_WAVE));
+        KA_CHECK(grid.y <= 65535, "ka_conv_prepare: too many heads");
+        if (dtype == KA_F32) hipLaunchKernelGGL(conv_prepare_normed_kernel<float>, grid, dim3(SP_THREADS), 0, stream, a);
+        else hipLaunchKernelGGL(conv_prepare_normed_kernel<bf16_t>, grid, dim3(SP_THREADS), 0, stream, a);
+    } else if (dtype == KA_F32) hipLaunchKernelGGL(conv_prepare_kernel<float>, dim3(n, n > SP_SPREAD_TOKENS ? 1 : blocks), dim3(SP_THREADS), 0, stream, a);
     else hipLaunchKernelGGL(conv_prepare_kernel<bf16_t>, dim3(n, n > SP_SPREAD_TOKENS ? 1 : blocks), dim3(SP_THREADS), 0, stream, a);
     KA_LAUNCH_CHECK();
-    if (K > 1 && n_rows > 0) {
+    if (K > 1 && n_rows > 0 && !a.moves_state) {
         if (dtype == KA_F32) hipLaunchKernelGGL(conv_state_kernel<float>, dim3(n_rows, blocks), dim3(SP_THREADS), 0, stream, a);
         else hipLaunchKernelGGL(conv_state_kernel<bf16_t>, dim3(n_rows, blocks), dim3(SP_THREADS), 0, stream, a);
         KA_LAUNCH_CHECK();

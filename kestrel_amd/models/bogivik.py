@@ -293,7 +293,7 @@ def build_plan(cfg: BogivikConfig) -> ModelPlan:
 
 def _claims(config: Dict[str, Any]) -> bool:
     layers = config.get("layers")
-    return isinstance(layers, list) and bool(layers) and "residual_mult" not in config and "width" in config and \
+    return isinstance(layers, list) and bool(layers) and "residual_mult" not in config and "streams" not in config and "width" in config and \
         all(isinstance(e, dict) and e.get("type") in ("attention", "parallel") and "mixer" in e for e in layers) and \
         any(e.get("type") == "parallel" or "bias_max" in (e.get("mixer") or {}) for e in layers)
 

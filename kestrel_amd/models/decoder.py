@@ -17,6 +17,7 @@ from ..ops.linear import linear
 from ..parts.base import LayerCache, build_part
 from ..parts.block import Block, settle
 from ..parts.specs import ModelPlan, ParamSpec
+from ..parts.streams import StreamReading
 
 
 class DecoderModel:
@@ -40,6 +41,13 @@ class DecoderModel:
                     raise ValueError(f"schedule entry {index} must read the cache of an earlier entry")
                 if plan.schedule[entry.reads_cache_of].reads_cache_of is not None:
                     raise ValueError(f"schedule entry {index} reads the cache of an entry that keeps none")
+        self.streams: Optional[int] = getattr(plan, "streams", None)
+        mixes = [m.spec.streams for b in self.blocks for m in (b.streams, b.streams2) if m is not None]
+        if self.streams is not None:
+            if self.junctions or any(b.spec.arrangement != "streams" for b in self.blocks) or any(s != self.streams for s in mixes):
+                raise ValueError(f"a stream of {self.streams} copies passes through blocks of the arrangement 'streams' for as many, and through no junction")
+        elif mixes:
+            raise ValueError("blocks that read several streams need a plan that names how many there are")
         self.embedding: Optional[torch.Tensor] = None
         self.head_weight: Optional[torch.Tensor] = None
         self.head_bias: Optional[torch.Tensor] = None
@@ -156,10 +164,20 @@ class DecoderModel:
         for junction in self.junctions.values():
             junction.begin(x, batch)
         handed = None      # the next block's first norm of x, where a block's last launch has computed it
+        final = None
+        if self.streams is not None:
+            # every stream starts as the embedding output; the launch that says so leaves what the first block reads
+            embedded, x = x, ws.get("model.streams", (batch.n_tokens, self.streams, plan.dim), torch.float32)
+            final = StreamReading(None, self.final_norm)
+            first = self.blocks[plan.schedule[0].layer].reader if plan.schedule else None
+            handed = ws.get("block.h", (batch.n_tokens, plan.dim), self.dtype) if first is not None else None
+            core.streams_step(x, embedded=embedded, reading=first.operands() if first is not None else None, h=handed)
         for index, entry in enumerate(plan.schedule):
             after = plan.schedule[index + 1] if index + 1 < len(plan.schedule) else None
             # (a junction between two runs changes the stream: no norm is handed across it)
-            then = self.blocks[after.layer].norm if after is not None and getattr(after, "before", None) is None else None
+            then = self.blocks[after.layer].reader if after is not None and getattr(after, "before", None) is None else None
+            if after is None and final is not None and batch.decode_only and getattr(batch, "wants_every_token", False):
+                then = final       # (every row goes to the head, in order: the last launch leaves what the head reads)
             before = getattr(entry, "before", None)
             if before is not None:
                 settle(x, batch)
@@ -169,11 +187,18 @@ class DecoderModel:
         settle(x, batch)       # (what the last block has left to be added into the stream)
         wanted = int(batch.logit_rows.numel())
         logits = ws.get("model.logits", (wanted, plan.vocab_size), torch.float32)
-        if wanted:
+        if wanted and self.streams is not None:
+            normed = handed if batch.decode_only and getattr(batch, "wants_every_token", False) else None
+            if normed is None:
+                normed = ws.get("model.head_in", (wanted, plan.dim), self.dtype)
+                core.streams_step(x, reading=final.operands(), h=normed, rows=batch.logit_rows)
+            linear(normed, self.head_weight, self.head_bias, logits)
+        elif wanted:
             if not self._head_with_norm(x, batch, logits):
                 normed = ws.get("model.head_in", (wanted, plan.dim), self.dtype)
                 self.final_norm.forward(x, normed, rows=batch.logit_rows)
                 linear(normed, self.head_weight, self.head_bias, logits)
+        if wanted:
             if plan.logit_scale != 1.0 or plan.logit_softcap is not None:
                 core.adjust_logits(logits, plan.logit_scale, plan.logit_softcap)
         return logits

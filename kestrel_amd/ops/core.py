@@ -42,7 +42,7 @@ _SIGNATURES = {
                       _c_int, _c_long, _c_long, _c_void_p, _c_int, _c_int, _c_int, _c_void_p],
     "ka_conv_prepare": [_c_void_p, _c_int, _c_long, _c_void_p, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                         _c_void_p, _c_long, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                        _c_void_p, _c_int, _c_int, _c_void_p],
+                        _c_void_p, _c_int, _c_int, _c_long, _c_int, _c_float, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p],
     "ka_maps_combine": [_c_void_p, _c_void_p, _c_int, _c_long, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float, _c_void_p],
     "ka_latent_prepare": [_c_void_p, _c_int, _c_long, _c_int, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_int,
                           _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_float, _c_int, _c_void_p],
@@ -68,9 +68,18 @@ _SIGNATURES = {
     "ka_decayed_memory": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                           _c_long, _c_void_p, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_float,
                           _c_void_p, _c_void_p],
-    "ka_route": [_c_void_p, _c_long, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_void_p, _c_void_p, _c_void_p],
-    "ka_experts_linear": [_c_void_p, _c_long, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p,
-                          _c_long, _c_int, _c_void_p],
+    "ka_route": [_c_void_p, _c_long, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_void_p, _c_void_p,
+                 _c_void_p],
+    "ka_experts_linear": [_c_void_p, _c_long, _c_int, _c_void_p, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
+                          _c_float, _c_float, _c_void_p, _c_long, _c_int, _c_void_p],
+    "ka_streams_step": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_float, _c_int,
+                        _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+    "ka_streams_experts": [_c_void_p, _c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_void_p, _c_void_p, _c_long,
+                           _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_float, _c_int, _c_void_p, _c_int, _c_int, _c_int, _c_int,
+                           _c_void_p],
+    "ka_gated_linear_attention": [_c_void_p, _c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_float, _c_float, _c_void_p, _c_long,
+                                  _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+    "ka_heads_rmsnorm": [_c_void_p, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void_p],
     "ka_experts_combine": [_c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p,
                            _c_long, _c_void_p, _c_int, _c_int, _c_void_p],
     "ka_experts_sort": [_c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p],
@@ -497,6 +506,21 @@ def linear_attention_supported(head_dim: int, value_dim: int) -> bool:
     return 0 < head_dim <= 512 and value_dim > 0
 
 
+def _check_recurrence(who, projected, offsets, state, cu_q, row_slot, raw, n_heads: int, head_dim: int, value_dim: int):
+    """Operands that the kernels of linear attention share; ``(q, k, v offsets, rows)``."""
+    n = projected.shape[0]
+    _need(linear_attention_supported(head_dim, value_dim), f"{who}: head sizes not covered")
+    oq, ok, ov = (int(o) for o in offsets)
+    _need(projected.dim() == 2 and projected.stride(1) == 1 and max(oq + n_heads * head_dim, ok + n_heads * head_dim, ov + n_heads * value_dim)
+          <= projected.shape[1], f"{who}: the projected rows are too short")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] == n_heads * head_dim * value_dim,
+          f"{who}: state fp32 [slots, H dv d]")
+    n_rows = row_slot.numel()
+    _need(cu_q.dtype == torch.int32 and cu_q.numel() == n_rows + 1 and row_slot.dtype == torch.int32, f"{who}: cu_q int32 [rows + 1]")
+    _need(raw.dtype == torch.float32 and raw.is_contiguous() and tuple(raw.shape) == (n, n_heads * value_dim), f"{who}: raw fp32 [n, H dv]")
+    return oq, ok, ov, n_rows
+
+
 def linear_attention(projected: torch.Tensor, offsets, decay: torch.Tensor, state: torch.Tensor, cu_q: torch.Tensor,
                      row_slot: torch.Tensor, raw: torch.Tensor, n_heads: int, head_dim: int, value_dim: int, act: int) -> None:
     """``S <- decay_h S + v k^T, o = S q`` over every row's tokens in order, with ``q, k, v = act(.)`` of the columns of ``projected``
@@ -505,16 +529,8 @@ def linear_attention(projected: torch.Tensor, offsets, decay: torch.Tensor, stat
     get zeros."""
     _dev(projected, decay, state, cu_q, row_slot, raw)
     n = projected.shape[0]
-    _need(linear_attention_supported(head_dim, value_dim), "linear_attention: head sizes not covered")
-    oq, ok, ov = (int(o) for o in offsets)
-    _need(projected.dim() == 2 and projected.stride(1) == 1 and max(oq + n_heads * head_dim, ok + n_heads * head_dim, ov + n_heads * value_dim)
-          <= projected.shape[1], "linear_attention: the projected rows are too short")
+    oq, ok, ov, n_rows = _check_recurrence("linear_attention", projected, offsets, state, cu_q, row_slot, raw, n_heads, head_dim, value_dim)
     _need(decay.dtype == torch.float32 and decay.numel() == n_heads and decay.is_contiguous(), "linear_attention: decay fp32 [H]")
-    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] == n_heads * head_dim * value_dim,
-          "linear_attention: state fp32 [slots, H dv d]")
-    n_rows = row_slot.numel()
-    _need(cu_q.dtype == torch.int32 and cu_q.numel() == n_rows + 1 and row_slot.dtype == torch.int32, "linear_attention: cu_q int32 [rows + 1]")
-    _need(raw.dtype == torch.float32 and raw.is_contiguous() and tuple(raw.shape) == (n, n_heads * value_dim), "linear_attention: raw fp32 [n, H dv]")
     size, base = projected.element_size(), projected.data_ptr()
     _check(lib().ka_linear_attention(base + oq * size, base + ok * size, base + ov * size, projected.stride(0) if n > 1 else projected.shape[1],
                                      code_of(projected.dtype), decay.data_ptr(), state.data_ptr(), state.stride(0), cu_q.data_ptr(),
@@ -532,6 +548,99 @@ def gated_rmsnorm(x: torch.Tensor, gain: Optional[torch.Tensor], eps: float, gat
           "gated_rmsnorm: the gate must be [n, dim] of the output's type")
     _check(lib().ka_gated_rmsnorm(x.data_ptr(), _ptr(gain), _ptr(gate), (gate.stride(0) if n > 1 else dim) if gate is not None else 0,
                                   out.data_ptr(), code_of(out.dtype), n, dim, float(eps), stream_ptr()))
+
+
+def gated_linear_attention(projected: torch.Tensor, offsets, pre: torch.Tensor, tau: float, q_scale: float, state: torch.Tensor,
+                           cu_q: torch.Tensor, row_slot: torch.Tensor, raw: torch.Tensor, n_heads: int, head_dim: int, value_dim: int) -> None:
+    """``S <- S diag(a) + v k^T, o = S (q_scale q)`` over every row's tokens in order, with ``a = sigmoid(pre) ** (1 / tau)`` per token and
+    key channel (``pre`` fp32 ``[n, H head_dim]``), ``state`` and the other operands as ``linear_attention`` takes them."""
+    _dev(projected, pre, state, cu_q, row_slot, raw)
+    n = projected.shape[0]
+    who = "gated_linear_attention"
+    oq, ok, ov, n_rows = _check_recurrence(who, projected, offsets, state, cu_q, row_slot, raw, n_heads, head_dim, value_dim)
+    _need(pre.dtype == torch.float32 and pre.is_contiguous() and tuple(pre.shape) == (n, n_heads * head_dim) and tau > 0, f"{who}: pre fp32 [n, H d]")
+    size, base = projected.element_size(), projected.data_ptr()
+    _check(lib().ka_gated_linear_attention(base + oq * size, base + ok * size, base + ov * size,
+                                           projected.stride(0) if n > 1 else projected.shape[1], code_of(projected.dtype), pre.data_ptr(),
+                                           float(tau), float(q_scale), state.data_ptr(), state.stride(0), cu_q.data_ptr(), row_slot.data_ptr(),
+                                           raw.data_ptr(), n, n_rows, n_heads, head_dim, value_dim, stream_ptr()))
+
+
+def heads_rmsnorm(raw: torch.Tensor, gain: torch.Tensor, gate: torch.Tensor, out: torch.Tensor, n_heads: int, value_dim: int, eps: float) -> None:
+    """``out = raw / sqrt(mean(raw^2) + eps) * gain * silu(gate)`` with every head of fp32 ``raw`` ``[n, H dv]`` normalised by itself, one
+    ``gain`` ``[dv]`` for all heads, and ``gate`` and ``out`` ``[n, H dv]`` of one type (rows may lie in wider ones)."""
+    _dev(raw, gain, gate, out)
+    n = out.shape[0]
+    for t in (gate, out):
+        _need(t.dim() == 2 and tuple(t.shape) == (n, n_heads * value_dim) and t.stride(1) == 1 and t.dtype == out.dtype, "heads_rmsnorm: gate and out [n, H dv]")
+    _need(raw.dtype == torch.float32 and raw.is_contiguous() and tuple(raw.shape) == (n, n_heads * value_dim), "heads_rmsnorm: raw fp32 [n, H dv]")
+    _need(gain.dtype == torch.float32 and gain.is_contiguous() and gain.numel() == value_dim, "heads_rmsnorm: gain fp32 [dv]")
+    width = n_heads * value_dim
+    _check(lib().ka_heads_rmsnorm(raw.data_ptr(), gain.data_ptr(), gate.data_ptr(), gate.stride(0) if n > 1 else max(gate.stride(0), width),
+                                  out.data_ptr(), out.stride(0) if n > 1 else max(out.stride(0), width), code_of(out.dtype), n, n_heads, value_dim,
+                                  float(eps), stream_ptr()))
+
+
+def _stream_args(who: str, x, mix, out, reading, h, rows=None):
+    """The streams and what is written and read of them: ``mix`` fp32 ``[S, S]`` and ``out`` fp32 ``[S]`` (or neither); ``reading =
+    (into fp32 [S] or None, (kind, gain, bias, eps))`` with ``kind`` ``"layernorm"`` or ``"rms"`` and ``h`` for its rows (or neither)."""
+    n, S, dim = x.shape
+    _dev(x, mix, out, h, rows)
+    _need(x.dtype == torch.float32 and x.is_contiguous(), f"{who}: the streams must be contiguous fp32 [n, S, dim]")
+    for t, shape in ((mix, (S, S)), (out, (S,))):
+        _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == shape), f"{who}: mix fp32 [S, S] and out fp32 [S]")
+    _need((reading is None) == (h is None), f"{who}: what is read needs rows to go to")
+    into = gain = bias = None
+    eps, rms = 0.0, 0
+    if reading is not None:
+        into, (kind, gain, bias, eps) = reading
+        rms = {"layernorm": 0, "rms": 1}[kind]
+        _dev(into, gain, bias)
+        _need(into is None or (into.dtype == torch.float32 and into.is_contiguous() and into.numel() == S), f"{who}: into fp32 [S]")
+        for t in (gain, bias):
+            _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == dim), f"{who}: gains fp32 [dim]")
+        wanted = n if rows is None else rows.numel()
+        _need(h.is_contiguous() and tuple(h.shape) == (wanted, dim), f"{who}: h must be [rows, dim]")
+    return into, gain, bias, float(eps), rms
+
+
+def streams_step(x: torch.Tensor, y: Optional[torch.Tensor] = None, mix: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None,
+                 reading=None, h: Optional[torch.Tensor] = None, embedded: Optional[torch.Tensor] = None,
+                 rows: Optional[torch.Tensor] = None) -> None:
+    """The streams ``x`` fp32 ``[n, S, dim]`` between two sublayers, in one launch: every stream becomes ``embedded`` ``[n, dim]`` first, if
+    that is given; then ``x_t <- sum_s mix[s, t] x_s + out[t] y`` for the output ``y`` ``[n, dim]`` of the sublayer before, if there is one;
+    then ``h = norm(sum_t into[t] x_t)`` for the next one (``_stream_args`` says what ``reading`` holds; ``into`` ``None``: the sum). ``rows``
+    (int32): only these rows are read (nothing is written)."""
+    n, S, dim = x.shape
+    into, gain, bias, eps, rms = _stream_args("streams_step", x, mix, out, reading, h, rows)
+    _dev(y, embedded)
+    for t in (y, embedded):
+        _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (n, dim)), "streams_step: fp32 rows [n, dim]")
+    _need(rows is None or (rows.dtype == torch.int32 and rows.is_contiguous()), "streams_step: rows int32")
+    _check(lib().ka_streams_step(x.data_ptr(), _ptr(embedded), _ptr(y), _ptr(mix), _ptr(out), _ptr(into), _ptr(rows), _ptr(gain), _ptr(bias), eps,
+                                 rms, _ptr(h), code_of(h.dtype) if h is not None else KA_F32, n if rows is None else rows.numel(), S, dim,
+                                 stream_ptr()))
+
+
+def streams_experts(x: torch.Tensor, pairs: torch.Tensor, h_in: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor, n_experts: int,
+                    shared: Optional[torch.Tensor], shared_gate: Optional[torch.Tensor], mix: torch.Tensor, out: torch.Tensor,
+                    reading=None, h: Optional[torch.Tensor] = None) -> None:
+    """``streams_step`` whose ``y`` is the weighted sum of ``experts_combine`` (operands as there)."""
+    n, S, dim = x.shape
+    top = chosen.shape[1]
+    who = "streams_experts"
+    into, gain, bias, eps, rms = _stream_args(who, x, mix, out, reading, h)
+    _dev(pairs, h_in, chosen, weights, shared, shared_gate)
+    _need(pairs.dtype == torch.float32 and pairs.is_contiguous() and tuple(pairs.shape) == (n * top, dim), f"{who}: pairs fp32 [n top, dim]")
+    _need(h_in.dim() == 2 and tuple(h_in.shape) == (n, dim) and h_in.stride(1) == 1, f"{who}: h_in [n, dim]")
+    _need(chosen.dtype == torch.int32 and chosen.is_contiguous() and weights.dtype == torch.float32 and weights.is_contiguous()
+          and tuple(chosen.shape) == tuple(weights.shape) == (n, top), f"{who}: chosen int32 and weights fp32 [n, top]")
+    _need(shared is None or (shared.dtype == torch.float32 and shared.is_contiguous() and tuple(shared.shape) == (n, dim)), f"{who}: shared fp32 [n, dim]")
+    _need(shared_gate is None or (shared_gate.dtype == torch.float32 and shared_gate.dim() == 1 and shared_gate.numel() == n), f"{who}: the gate is an fp32 column")
+    _check(lib().ka_streams_experts(x.data_ptr(), pairs.data_ptr(), h_in.data_ptr(), h_in.stride(0) if n > 1 else dim, code_of(h_in.dtype),
+                                    chosen.data_ptr(), weights.data_ptr(), top, int(n_experts), _ptr(shared), _ptr(shared_gate),
+                                    (shared_gate.stride(0) if n > 1 else 1) if shared_gate is not None else 0, _ptr(mix), _ptr(out), _ptr(into),
+                                    _ptr(gain), _ptr(bias), eps, rms, _ptr(h), code_of(h.dtype) if h is not None else KA_F32, n, S, dim, stream_ptr()))
 
 
 def pair_embed(table: torch.Tensor, ids: torch.Tensor, positions: torch.Tensor, token_row: torch.Tensor, cu_q: torch.Tensor,
@@ -562,13 +671,15 @@ def conv_prepare(u: torch.Tensor, taps: Optional[torch.Tensor], state: Optional[
                  row_slot: torch.Tensor, token_row: torch.Tensor, positions: torch.Tensor, slots: Optional[torch.Tensor],
                  q_out: torch.Tensor, k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], q_heads: int, k_heads: int,
                  head_dim: int, v_heads: int, value_dim: int, page_size: int, freqs: Optional[torch.Tensor] = None,
-                 pairing: str = "halves") -> None:
+                 pairing: str = "halves", unit_norm_eps: Optional[float] = None, runs=None, single_tokens: bool = False) -> None:
     """A short causal convolution over time on every channel of the projected rows ``u`` ``[n, q | k | v]``
     (``taps`` fp32 ``[channels, K]``: ``y_t = sum_j taps[:, j] u_(t - K + 1 + j)``; ``None``: none), then the rotation of the
     first ``2 len(freqs)`` channels of every query and key head by ``place * freqs``, then queries into ``q_out`` ``[n, q]``,
     keys into the paged ``k_cache`` ``[pages, k_heads, page, hd]`` and values into ``v_cache`` ``[pages, v_heads, hdv, page]`` at
-    ``slots``. Inputs from before this step come from ``state`` fp32 ``[slots + 1, K - 1, channels]`` (by ``row_slot``), which is
-    then moved on to the last ``K - 1`` rows of ``u`` of every row."""
+    ``slots``. Inputs from before this step come from ``state`` fp32 ``[slots + 1, K - 1, channels]`` (by ``row_slot``; a slot's rows
+    may lie in a wider one), which is then moved on to the last ``K - 1`` rows of ``u`` of every row. ``unit_norm_eps``: every query
+    and key head is divided by its root mean square ``sqrt(mean(square) + eps)`` as well. ``runs``: (int32 first token, int32 count) of
+    the runs the tokens are cut into (``StepBatch.page_runs``); ``single_tokens``: every row brings one token."""
     _need(pairing in ROTARY_PAIRINGS, f"conv_prepare: pairing {pairing!r} is not one of {sorted(ROTARY_PAIRINGS)}")
     _dev(u, taps, state, cu_q, row_slot, token_row, positions, slots, q_out, k_cache, v_cache, freqs)
     n = u.shape[0]
@@ -584,8 +695,8 @@ def conv_prepare(u: torch.Tensor, taps: Optional[torch.Tensor], state: Optional[
         _need(K >= 1, "conv_prepare: at least one tap")
     n_rows = row_slot.numel()
     if K > 1:
-        _need(state is not None and state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (K - 1, channels),
-              "conv_prepare: state must be fp32 [slots + 1, K - 1, channels]")
+        _need(state is not None and state.dtype == torch.float32 and tuple(state.shape[1:]) == (K - 1, channels)
+              and state.stride(2) == 1 and (K == 2 or state.stride(1) == channels), "conv_prepare: state must be fp32 [slots + 1, K - 1, channels]")
     for t in (token_row, positions) + ((slots,) if slots is not None else ()):
         _need(t.dtype == torch.int32 and t.numel() == n and t.is_contiguous(), "conv_prepare: per-token int32 [n] expected")
     _need(cu_q.dtype == torch.int32 and cu_q.numel() == n_rows + 1 and cu_q.is_contiguous() and row_slot.dtype == torch.int32
@@ -595,6 +706,11 @@ def conv_prepare(u: torch.Tensor, taps: Optional[torch.Tensor], state: Optional[
               and k_cache.is_contiguous() and v_cache.is_contiguous()
               and tuple(k_cache.shape[1:]) == (k_heads, page_size, head_dim)
               and tuple(v_cache.shape[1:]) == (v_heads, value_dim, page_size), "conv_prepare: caches [pages, Hk, page, hd] and [pages, Hv, hdv, page]")
+    first, count = runs if runs is not None else (None, None)
+    _need(first is None or (first.is_cuda and count.is_cuda and first.dtype == torch.int32 and count.dtype == torch.int32
+                            and first.numel() == count.numel() and first.is_contiguous() and count.is_contiguous()),
+          "conv_prepare: runs are two int32 lists of one length")
+    _need(not single_tokens or n == n_rows, "conv_prepare: a step of single tokens has as many rows as tokens")
     rot = 0
     if freqs is not None:
         _need(freqs.dtype == torch.float32 and freqs.dim() == 1 and freqs.is_contiguous(), "conv_prepare: freqs fp32 [R / 2]")
@@ -603,7 +719,8 @@ def conv_prepare(u: torch.Tensor, taps: Optional[torch.Tensor], state: Optional[
                                  cu_q.data_ptr(), row_slot.data_ptr(), token_row.data_ptr(), positions.data_ptr(), _ptr(slots),
                                  q_out.data_ptr(), q_out.stride(0) if n > 1 else q_heads * head_dim, _ptr(k_cache), _ptr(v_cache), n, n_rows,
                                  q_heads, k_heads, head_dim, v_heads, value_dim, page_size, _ptr(freqs), rot, ROTARY_PAIRINGS[pairing],
-                                 stream_ptr()))
+                                 state.stride(0) if K > 1 else 0, int(unit_norm_eps is not None), float(unit_norm_eps or 0.0), _ptr(first),
+                                 _ptr(count), int(first.numel()) if first is not None else 0, int(bool(single_tokens)), stream_ptr()))
 
 
 def maps_combine(maps: torch.Tensor, out: torch.Tensor, n_heads: int, value_dim: int, weight: float, eps: float, out_scale: float) -> None:
@@ -795,29 +912,45 @@ def decayed_memory(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torc
                                    out.stride(0) if n > 1 else width, n, n_rows, n_heads, head_dim, float(eps), raw.data_ptr(), stream_ptr()))
 
 
+ROUTER_SCORES = {"softmax": 0, "sigmoid": 2}
+
+
+def _clamp_args(clamp, act: int):
+    """A ``parts.specs.GateClamp`` (or ``None``) as the experts' kernels take it."""
+    _need(clamp is None or (act & 0x100 and clamp.limit > 0), "experts: clamps are a gated linear's, with a positive limit")
+    return (0, 0.0, 0.0, 0.0) if clamp is None else (1, float(clamp.limit), float(clamp.slope), float(clamp.shift))
+
+
 def route(logits: torch.Tensor, n_outputs: int, correction: Optional[torch.Tensor], top: int, n_groups: int, keep_groups: int,
-          scale: float, chosen: torch.Tensor, weights: torch.Tensor, weigh_chosen: bool = False) -> None:
+          scale: float, chosen: torch.Tensor, weights: torch.Tensor, weigh_chosen: bool = False, scores: str = "softmax",
+          group_best: int = 1, always: Optional[int] = None) -> None:
     """A router's choice per token from fp32 ``logits`` ``[n, >= n_outputs]``: scores = softmax over the first ``n_outputs``
     columns; the choice goes by scores + ``correction`` among the outputs of the ``keep_groups`` best of ``n_groups`` equal
     groups of neighbours (0 groups: among all); ``chosen`` int32 ``[n, top]``, ``weights`` fp32 ``[n, top]`` = the chosen scores
     over their sum (+ 1e-20), times ``scale``. ``weigh_chosen``: the choice goes by the logits alone and the weights are the softmax
-    over the chosen logits, times ``scale`` (no groups, no correction)."""
+    over the chosen logits, times ``scale`` (no groups, no correction). ``scores`` ``"sigmoid"``: the scores are the logits' sigmoids.
+    ``group_best`` 2: a group counts by the sum of its two largest choice scores. ``always``: ``chosen`` and ``weights`` are
+    ``[n, top + 1]`` and end in that number with weight 1."""
     _dev(logits, correction, chosen, weights)
+    _need(scores in ROUTER_SCORES and not (weigh_chosen and scores != "softmax"), f"route: unknown scores {scores!r}")
+    columns = top + (always is not None)
     _need(not weigh_chosen or (n_groups == 0 and correction is None), "route: a choice by the logits alone has no groups and no correction")
     n = logits.shape[0]
     _need(logits.dtype == torch.float32 and logits.dim() == 2 and logits.stride(1) == 1 and logits.shape[1] >= n_outputs, "route: logits fp32 [n, >= outputs]")
     _need(correction is None or (correction.dtype == torch.float32 and correction.is_contiguous() and correction.numel() == n_outputs),
           "route: correction fp32 [outputs]")
-    _need(chosen.dtype == torch.int32 and chosen.is_contiguous() and tuple(chosen.shape) == (n, top) and weights.dtype == torch.float32
-          and weights.is_contiguous() and tuple(weights.shape) == (n, top), "route: chosen int32 and weights fp32 [n, top]")
+    _need(chosen.dtype == torch.int32 and chosen.is_contiguous() and tuple(chosen.shape) == (n, columns) and weights.dtype == torch.float32
+          and weights.is_contiguous() and tuple(weights.shape) == (n, columns), "route: chosen int32 and weights fp32 [n, top]")
     _check(lib().ka_route(logits.data_ptr(), logits.stride(0) if n > 1 else logits.shape[1], _ptr(correction), n, int(n_outputs), int(top),
-                          int(n_groups), int(keep_groups), float(scale), int(bool(weigh_chosen)), chosen.data_ptr(), weights.data_ptr(), stream_ptr()))
+                          int(n_groups), int(keep_groups), int(group_best), float(scale), 1 if weigh_chosen else ROUTER_SCORES[scores],
+                          -1 if always is None else int(always), chosen.data_ptr(), weights.data_ptr(), stream_ptr()))
 
 
-def experts_linear(a: torch.Tensor, per_token: int, weights: torch.Tensor, chosen: torch.Tensor, out: torch.Tensor, act: int = 0) -> None:
+def experts_linear(a: torch.Tensor, per_token: int, weights: torch.Tensor, chosen: torch.Tensor, out: torch.Tensor, act: int = 0,
+                   clamp=None) -> None:
     """``out[p] = act(a[p // per_token] @ weights[chosen[p]].T)`` for every pair ``p`` whose choice is an expert with weights
     (``chosen[p] < E``; other rows of ``out`` are left alone). ``weights`` ``[E, N, K]``; ``act`` may carry the gated flag (rows of an
-    expert in pairs). ``out`` of the operands' type or fp32."""
+    expert in pairs); ``clamp`` (a ``GateClamp``): the pair's product is the clamped one. ``out`` of the operands' type or fp32."""
     _dev(a, weights, chosen, out)
     n_pairs = chosen.numel()
     E, N, K = weights.shape
@@ -828,7 +961,7 @@ def experts_linear(a: torch.Tensor, per_token: int, weights: torch.Tensor, chose
     _need(out.dim() == 2 and out.stride(1) == 1 and tuple(out.shape) == (n_pairs, n_out) and out.dtype in (a.dtype, torch.float32),
           "experts_linear: out must be [pairs, outputs]")
     _check(lib().ka_experts_linear(a.data_ptr(), a.stride(0) if a.shape[0] > 1 else K, int(per_token), weights.data_ptr(), code_of(a.dtype),
-                                   chosen.data_ptr(), n_pairs, E, N, K, int(act), out.data_ptr(), out.stride(0) if n_pairs > 1 else n_out,
+                                   chosen.data_ptr(), n_pairs, E, N, K, int(act), *_clamp_args(clamp, int(act)), out.data_ptr(), out.stride(0) if n_pairs > 1 else n_out,
                                    int(out.dtype == torch.float32 and a.dtype != torch.float32), stream_ptr()))
 
 

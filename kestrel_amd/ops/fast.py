@@ -69,8 +69,8 @@ _SIGNATURES = {
                              _c_long, _c_void_p, _c_void_p],
     "ka_heads_linear_supported": [_c_long, _c_int, _c_long, _c_int, _c_int, _c_int],
     "ka_experts_gemm_supported": [_c_long, _c_int, _c_int, _c_long, _c_int, _c_int],
-    "ka_experts_gemm_bf16": [_c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_void_p,
-                             _c_long, _c_int, _c_int, _c_void_p],
+    "ka_experts_gemm_bf16": [_c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
+                             _c_float, _c_float, _c_void_p, _c_long, _c_int, _c_int, _c_void_p],
     "ka_matrix_memory_chunks_bf16": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                                      _c_void_p, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float,
                                      _c_void_p, _c_int, _c_void_p],
@@ -906,12 +906,12 @@ def linear_attention_chunks_bf16(projected, offsets, log2_decay, state, cu_q, ro
     return True
 
 
-def experts_feed_forward_bf16(h, pairs, down, chosen, hidden, y, act, workspace) -> bool:
+def experts_feed_forward_bf16(h, pairs, down, chosen, hidden, y, act, workspace, clamp=None) -> bool:
     """Both linears of the chosen experts for all pairs of a step on the matrix cores, an expert's pairs together: the pairs
     are listed by expert (``ops.core.experts_sort``), the first linear (gated or not, as ``act`` says) gathers every pair's token from ``h`` ``[n, dim]`` and
     leaves the hidden rows in list order, the second writes fp32 ``y`` ``[n top, dim]`` at the pairs' own rows. ``pairs``
     ``[E, 2 hidden, dim]`` (not gated: ``[E, hidden, dim]``), ``down`` ``[E, dim, hidden]``, ``chosen`` int32 ``[n, top]``; ``hidden`` is not used (the list's hidden rows
-    live in the workspace). False: not covered (sizes that are no multiple of 16, alignment), nothing was run."""
+    live in the workspace). ``clamp`` (a ``GateClamp``): the pair's product is the clamped one. False: not covered (sizes that are no multiple of 16, alignment), nothing was run."""
     n, top = chosen.shape
     n_experts, n_pair_rows, dim = pairs.shape
     ff = down.shape[2]
@@ -936,7 +936,7 @@ def experts_feed_forward_bf16(h, pairs, down, chosen, hidden, y, act, workspace)
     rows = workspace.get("experts.hidden_listed", (capacity, ff), torch.bfloat16)
     core.experts_sort(chosen.view(-1), n_experts, tile, listed, tile_expert)
     _check(handle.ka_experts_gemm_bf16(h.data_ptr(), lda, top, pairs.data_ptr(), listed.data_ptr(), tile_expert.data_ptr(), capacity // tile,
-                                       n_pair_rows, dim, act, rows.data_ptr(), ff, 0, 0, stream_ptr()))
+                                       n_pair_rows, dim, act, *core._clamp_args(clamp, act), rows.data_ptr(), ff, 0, 0, stream_ptr()))
     _check(handle.ka_experts_gemm_bf16(rows.data_ptr(), ff, 0, down.data_ptr(), listed.data_ptr(), tile_expert.data_ptr(), capacity // tile,
-                                       dim, ff, 0, y.data_ptr(), dim, 1, 1, stream_ptr()))
+                                       dim, ff, 0, *core._clamp_args(None, 0), y.data_ptr(), dim, 1, 1, stream_ptr()))
     return True

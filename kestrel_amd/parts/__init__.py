@@ -1,7 +1,7 @@
 """Parts a model is put together from; importing the package registers the built-in kinds."""
 
-from . import (attention, branches, decayed_memory, differential_attention, experts, junction, latent_attention, learned_position,
-               linear_attention, matrix_memory, mlp, norm, pair_embedding, rotary)  # noqa: F401  (registration)
+from . import (attention, branches, decayed_memory, differential_attention, experts, gated_linear_attention, junction, latent_attention,
+               learned_position, linear_attention, matrix_memory, mlp, norm, pair_embedding, rotary, streams)  # noqa: F401  (registration)
 from .base import (FeedForward, Junction, LayerCache, Mixer, Norm, Part, PositionEncoding, Rotation, SideLinear, build_part, known_kinds,
                    register_feed_forward, register_junction, register_mixer, register_norm, register_position)
 from .block import ARRANGEMENTS, Block, register_arrangement

@@ -10,7 +10,7 @@ from ..ops import core
 from ..ops.attention import paged_attention
 from ..ops.linear import linear
 from .base import LayerCache, Mixer, build_part, register_mixer
-from .specs import AttentionSpec, CacheSpec, ParamSpec
+from .specs import AttentionSpec, CacheSpec, ParamSpec, StateSpec
 
 
 class PagedAttention(Mixer):
@@ -54,6 +54,11 @@ class PagedAttention(Mixer):
     ``softcap * tanh(score / softcap)``; a learned sink score per head (``head_sinks``, tensor ``sinks``); a gate of one
     number per head (``gate_per_head``); and a layer without keys and values of its own (``shares_kv``: it projects
     queries, and the gate, alone, and its schedule entry reads another entry's cache).
+
+    ``conv_taps``: a short causal convolution over time on every channel of q, k and v right after the projections (tensors
+    ``q.conv``, ``k.conv``, ``v.conv``), fused with the norm, the rotation and the cache write (``ops.core.conv_prepare``); the last
+    ``taps - 1`` projected rows of a sequence are per-request state. With it go a norm per head without gains and a rotation
+    by frequencies, and none of the other forms that change queries, keys or values.
     """
 
     replays_every_step = True
@@ -102,6 +107,15 @@ class PagedAttention(Mixer):
             raise ValueError("a layer without values of its own takes neither unit-norm keys nor blended values")
         if self.head_sinks and self.sink is not None:
             raise ValueError("a sink is one number (sink) or one per head (head_sinks), not both")
+        self.taps = int(getattr(spec, "conv_taps", None) or 0)
+        if self.taps:
+            self.prepared = True
+            if self.shares_kv or self.values_from_keys or self.blend is not None or self.growth is not None or self.unit_norm_eps is not None \
+                    or self.distance is not None or self.sink is not None or spec.bias \
+                    or (self.qk_norm is not None and (self.qk_norm.scope != "head" or self.qk_norm.gain)) or not spec.split_projections:
+                raise ValueError("attention behind convolutions takes split projections without biases, a norm per head without gains, and "
+                                 "no form that changes queries, keys or values otherwise")
+        self._taps: Optional[torch.Tensor] = None
         self.gate_dim = (spec.n_heads if self.gate_per_head else self.out_dim) if self.gated else 0
         self.in_dim = self.qkv_dim + self.gate_dim
         self._slopes: Optional[torch.Tensor] = None
@@ -125,6 +139,8 @@ class PagedAttention(Mixer):
             out["q_norm.weight"] = ParamSpec((spec.head_dim if per_head else self.q_dim,), "vector", "gain")
             if not self.shares_kv:
                 out["k_norm.weight"] = ParamSpec((spec.head_dim if per_head else self.kv_dim,), "vector", "gain")
+        if self.taps:
+            out.update({f"{name}.conv": ParamSpec((rows, self.taps), "matrix", "last") for name, rows in pieces.items()})
         if self.head_sinks:
             out["sinks"] = ParamSpec((spec.n_heads,), "vector", "bias")
         if self.buckets is not None:
@@ -139,6 +155,9 @@ class PagedAttention(Mixer):
     def cache_spec(self) -> CacheSpec:
         return CacheSpec(self.spec.n_kv_heads, self.spec.head_dim, self.spec.window,
                          self.value_dim if self.value_dim != self.spec.head_dim else None, getattr(self.spec, "chunk", None))
+
+    def state_spec(self) -> Optional[StateSpec]:
+        return StateSpec((self.taps - 1, self.qkv_dim), "float32") if self.taps > 1 else None
 
     def bind(self, tensors, dtype, device) -> None:
         spec = self.spec
@@ -165,6 +184,8 @@ class PagedAttention(Mixer):
             self._q_gain = tensors["q_norm.weight"].to(device=device, dtype=torch.float32).contiguous()
             if not self.shares_kv:
                 self._k_gain = tensors["k_norm.weight"].to(device=device, dtype=torch.float32).contiguous()
+        if self.taps:
+            self._taps = fused("conv").to(dtype=torch.float32).contiguous()
         if self.head_sinks:
             self._sinks = tensors["sinks"].to(device=device, dtype=torch.float32).contiguous()
         if self.buckets is not None:
@@ -225,6 +246,18 @@ class PagedAttention(Mixer):
     def output_projection(self):
         return self.proj_weight, self.proj_bias
 
+    def share_projections(self, in_weight, proj_weight) -> None:
+        self.qkv_weight, self.proj_weight = in_weight, proj_weight
+
+    def fold_output_weight(self, weight: float) -> bool:
+        if weight == 1.0:
+            return True
+        if not self.taps:
+            return False
+        # the heads are weighted sums of values, and the values of what their taps weigh: fp32 numbers that take up any factor
+        self._taps[self.q_dim + self.kv_dim:] *= float(weight)
+        return True
+
     def _decodes_fused(self, batch, cache: LayerCache) -> bool:
         """One token per row in bf16 with a rotation by halves: the decode kernel then rotates q and
         k and stores k and v itself."""
@@ -239,12 +272,13 @@ class PagedAttention(Mixer):
         return fast.attention_decode_takes(job, job.a.shape[0], self.spec.n_heads, self.spec.head_dim, cache.k.shape[2],
                                            batch.max_kv)
 
-    def attend(self, qkv, batch, cache: LayerCache, beside=None):
-        """Position encoding, cache write and attention on the projected input ``[n, q|k|v]``."""
+    def attend(self, qkv, batch, cache: LayerCache, beside=None, out=None):
+        """Position encoding, cache write and attention on the projected input ``[n, q|k|v]``; ``out``: where the heads go."""
         spec = self.spec
         n = qkv.shape[0]
         group = batch.groups[cache.group]
-        out = batch.workspace.get("attn.out", (n, self.out_dim), self.dtype)
+        if out is None:
+            out = batch.workspace.get("attn.out", (n, self.out_dim), self.dtype)
         if self.prepared:
             if beside is not None:
                 self._alone(beside)
@@ -317,12 +351,15 @@ class PagedAttention(Mixer):
         norm = self.qk_norm
         if self.shares_kv and cache.writes:
             raise RuntimeError("a layer without keys and values of its own must read another layer's cache (ScheduleEntry.reads_cache_of)")
-        core.qkv_prepare(qkv, batch.positions, slots, cache.k, cache.v, spec.n_heads, 0 if self.shares_kv else spec.n_kv_heads,
-                         spec.head_dim, self.value_dim, group.page_size, norm.scope if norm is not None else None, self._q_gain,
-                         self._k_gain, float(norm.eps) if norm is not None else 0.0, self._freqs, self._pairing,
-                         (self.growth.coef, self.growth.every) if self.growth is not None else None,
-                         self.blend.role if self.blend is not None else None, other, self._blend_weight,
-                         values_from_keys=self.values_from_keys)
+        if self.taps:
+            qkv = self._convolve(qkv, batch, cache, group, slots)
+        else:
+            core.qkv_prepare(qkv, batch.positions, slots, cache.k, cache.v, spec.n_heads, 0 if self.shares_kv else spec.n_kv_heads,
+                             spec.head_dim, self.value_dim, group.page_size, norm.scope if norm is not None else None, self._q_gain,
+                             self._k_gain, float(norm.eps) if norm is not None else 0.0, self._freqs, self._pairing,
+                             (self.growth.coef, self.growth.every) if self.growth is not None else None,
+                             self.blend.role if self.blend is not None else None, other, self._blend_weight,
+                             values_from_keys=self.values_from_keys)
         gate = projected[:, self.qkv_dim:] if self.gated else None
         more = dict(sinks=self._sinks, softcap=self.softcap, gate_per_head=self.gate_per_head)
         done = gated = False          # (gated: the attention kernel has applied the output gate in its epilogue)
@@ -345,6 +382,18 @@ class PagedAttention(Mixer):
         if self.gated and not gated:
             core.gate_mul(out, gate)
         return out
+
+    def _convolve(self, qkv, batch, cache: LayerCache, group, slots):
+        """The convolutions with all that follows them before attention; returns the queries."""
+        spec = self.spec
+        if self.taps > 1 and cache.state is None:
+            raise RuntimeError("the convolution needs its per-request state from the cache manager")
+        q = batch.workspace.get("attn.q", (qkv.shape[0], self.q_dim), self.dtype)
+        core.conv_prepare(qkv, self._taps, cache.state, batch.cu_q, batch.row_slot, batch.token_row, batch.positions, slots, q, cache.k, cache.v,
+                          spec.n_heads, spec.n_kv_heads, spec.head_dim, spec.n_kv_heads, self.value_dim, group.page_size, self._freqs,
+                          self._pairing, unit_norm_eps=float(self.qk_norm.eps) if self.qk_norm is not None else None,
+                          runs=getattr(batch, "page_runs", None), single_tokens=bool(batch.decode_only))
+        return q
 
     @staticmethod
     def _alone(job) -> None:

@@ -5,7 +5,7 @@ A part is built from its specification alone, says which tensors it owns
 (``forward``). It never sees the model or the architecture it is used in.
 
 Adding a part of a new kind: subclass the interface, and call ``register_mixer`` /
-``register_feed_forward`` / ``register_norm`` / ``register_position`` / ``register_junction`` with the kind
+``register_feed_forward`` / ``register_norm`` / ``register_position`` / ``register_junction`` / ``register_stream_mix`` with the kind
 name that its specification carries.
 """
 
@@ -204,6 +204,18 @@ class Mixer(Part):
         """``(weight, bias or None)`` of the last linear, whose result is added to the residual."""
         return None
 
+    # Optional, for mixers that stand side by side on one input (``parts/branches.py``): their first linears then run as one, and
+    # their last ones too. Such a mixer offers the three stages above without biases, takes ``out=`` (rows that may lie in
+    # wider ones) in ``attend``, and
+    def share_projections(self, in_weight, proj_weight) -> None:
+        """Hold these views of joint tensors instead of the mixer's own two weights (same values)."""
+        raise NotImplementedError
+
+    def fold_output_weight(self, weight: float) -> bool:
+        """Whether what ``attend`` returns is ``weight`` times what it would be from now on, at no cost and no loss (a factor
+        that some fp32 constant of the mixer takes up)."""
+        return weight == 1.0
+
 
 class FeedForward(Part):
     def forward(self, h: torch.Tensor, batch, residual: torch.Tensor) -> None:
@@ -220,7 +232,7 @@ class FeedForward(Part):
         return None
 
 
-_REGISTRIES: Dict[str, Dict[str, Callable]] = {"mixer": {}, "feed_forward": {}, "norm": {}, "position": {}, "junction": {}}
+_REGISTRIES: Dict[str, Dict[str, Callable]] = {"mixer": {}, "feed_forward": {}, "norm": {}, "position": {}, "junction": {}, "stream_mix": {}}
 
 
 def _register(family: str, kind: str, cls: Callable) -> None:
@@ -245,6 +257,10 @@ def register_position(kind: str, cls: Callable) -> None:
 
 def register_junction(kind: str, cls: Callable) -> None:
     _register("junction", kind, cls)
+
+
+def register_stream_mix(kind: str, cls: Callable) -> None:
+    _register("stream_mix", kind, cls)
 
 
 def build_part(family: str, spec) -> Part:

@@ -8,6 +8,7 @@ import torch
 
 from .base import LayerCache, Part, SideLinear, build_part
 from .specs import LayerSpec, ParamSpec
+from .streams import StreamReading
 
 
 def _parallel_few_rows(block: "Block", x, batch, cache, normed, then, handed) -> bool:
@@ -348,9 +349,53 @@ def _norms_around(block: "Block", x, batch, cache, normed=None, then=None):
 _norms_around.hands_over = True
 
 
+def _streams(block: "Block", x, batch, cache, normed=None, then=None):
+    """The stream as several copies ``x`` ``[n, S, dim]`` (hyper-connections): ``u = sum_s in[s] x_s``, ``y = mixer(norm(u))``,
+    ``x_t <- sum_s mix[s, t] x_s + out[t] y``, then the same with the feed-forward and its own numbers and norm.
+
+    One launch stands between two sublayers: it writes the one's output into the streams and leaves the norm of what the
+    next one reads (``then``, a ``StreamReading``, behind the last: its rows are handed over). A feed-forward that offers
+    ``mix_streams`` takes that launch's work into its own last one."""
+    from ..ops import core
+
+    ws = batch.workspace
+    n, _count, dim = x.shape
+    ff = block.feed_forward
+    delta = ws.get("block.delta", (n, dim), torch.float32)
+    h = normed
+    if h is None:
+        h = ws.get("block.h", (n, dim), block.dtype)
+        core.streams_step(x, reading=block.reader.operands(), h=h)
+
+    def into_delta(part, *operands):
+        if callable(getattr(part, "mix", None)):
+            part.mix(*operands, delta, False)
+        else:
+            delta.zero_()
+            part.forward(*operands, delta)
+
+    into_delta(block.mixer, h, batch, cache)
+    last = then.operands() if then is not None else None
+    handed = ws.get("block.handed", (n, dim), block.dtype) if then is not None else None
+    if ff is None:
+        core.streams_step(x, delta, block.streams.matrix, block.streams.out, last, handed)
+        return handed
+    h2 = ws.get("block.h2", (n, dim), block.dtype)
+    core.streams_step(x, delta, block.streams.matrix, block.streams.out, block.reader2.operands(), h2)
+    if callable(getattr(ff, "mix_streams", None)):
+        ff.mix_streams(h2, batch, x, block.streams2, last, handed)
+        return handed
+    into_delta(ff, h2, batch)
+    core.streams_step(x, delta, block.streams2.matrix, block.streams2.out, last, handed)
+    return handed
+
+
+_streams.hands_over = True
+
+
 ARRANGEMENTS: Dict[str, Callable] = {"parallel": _parallel, "sequential": _sequential,
                                      "parallel_two_norms": _parallel_two_norms, "output_norms": _output_norms,
-                                     "norms_around": _norms_around}
+                                     "norms_around": _norms_around, "streams": _streams}
 
 
 def register_arrangement(name: str, fn: Callable) -> None:
@@ -378,11 +423,19 @@ class Block:
         if spec.arrangement == "norms_around" and (self.norm_after is None or (
                 spec.feed_forward is not None and (self.norm2 is None or self.norm2_after is None))):
             raise ValueError("the norms_around arrangement needs norm_after, and norm2 and norm2_after for its feed-forward")
+        self.streams = build_part("stream_mix", spec.streams) if getattr(spec, "streams", None) is not None else None
+        self.streams2 = build_part("stream_mix", spec.streams2) if getattr(spec, "streams2", None) is not None else None
+        if spec.arrangement == "streams" and (self.streams is None or (
+                spec.feed_forward is not None and (self.norm2 is None or self.streams2 is None))):
+            raise ValueError("the streams arrangement needs streams, and norm2 and streams2 for its feed-forward")
+        # who reads the stream first in this block, as the block before is told (``then``)
+        self.reader = StreamReading(self.streams, self.norm) if spec.arrangement == "streams" else self.norm
+        self.reader2 = StreamReading(self.streams2, self.norm2) if spec.arrangement == "streams" and spec.feed_forward is not None else None
         self.mixer = build_part("mixer", spec.mixer)
         if spec.arrangement == "output_norms" and self.norm2 is None and spec.feed_forward is not None:
             raise ValueError("the output_norms arrangement needs norm2 for its feed-forward")
         if spec.feed_forward is None and spec.arrangement not in ("parallel_two_norms", "parallel", "sequential", "output_norms",
-                                                                          "norms_around"):
+                                                                          "norms_around", "streams"):
             raise ValueError(f"the {spec.arrangement} arrangement needs a feed-forward")
         if spec.arrangement == "parallel_two_norms" and spec.feed_forward is not None and self.norm2 is None:
             raise ValueError("the parallel_two_norms arrangement needs norm2 for its feed-forward")
@@ -400,6 +453,10 @@ class Block:
             out["norm_after"] = self.norm_after
         if self.norm2_after is not None:
             out["norm2_after"] = self.norm2_after
+        if self.streams is not None:
+            out["streams"] = self.streams
+        if self.streams2 is not None:
+            out["streams2"] = self.streams2
         return out
 
     def params(self) -> Dict[str, ParamSpec]:
@@ -422,8 +479,9 @@ class Block:
     def forward(self, x: torch.Tensor, batch, cache: LayerCache, normed: Optional[torch.Tensor] = None,
                 then: Optional[Part] = None) -> Optional[torch.Tensor]:
         """Updates the fp32 residual ``x`` in place. ``normed``: this block's first norm of ``x``, if the
-        block before has computed it; ``then``: the first norm of the block that follows. Returns that
-        norm of the result where the block's last launch computed it, else ``None``."""
+        block before has computed it; ``then``: the first norm of the block that follows (its ``reader``). Returns that
+        norm of the result where the block's last launch computed it, else ``None``. In the ``streams`` arrangement ``x`` is
+        ``[n, S, dim]``, and norms are those of what is read of the streams."""
         if not getattr(self._run, "defers", False):
             settle(x, batch)          # (an arrangement that knows nothing of sums left to be added)
         if getattr(self._run, "hands_over", False):

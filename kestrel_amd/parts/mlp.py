@@ -48,10 +48,14 @@ class DenseFeedForward(FeedForward):
     def output_projection(self):
         return self.fc2_weight, self.fc2_bias
 
-    def forward(self, h, batch, residual) -> None:
+    def mix(self, h, batch, out, accumulate: bool) -> None:
+        """The feed-forward of ``h`` written into (or added to) fp32 ``out``."""
         hidden = batch.workspace.get("ff.hidden", (h.shape[0], self.spec.hidden_dim), self.dtype)
         linear(h, self.fc1_weight, self.fc1_bias, hidden, act=self.act)
-        linear(hidden, self.fc2_weight, self.fc2_bias, residual, accumulate=True)
+        linear(hidden, self.fc2_weight, self.fc2_bias, out, accumulate=accumulate)
+
+    def forward(self, h, batch, residual) -> None:
+        self.mix(h, batch, residual, True)
 
 
 class GatedFeedForward(FeedForward):

@@ -21,7 +21,8 @@ class ParamSpec:
     ``role`` fixes how the tensor is held and initialised: ``matrix`` (2-D weight,
     model precision), ``vector`` (bias or gain), ``table`` (integer table, int32).
     ``init`` names the random-weights recipe: ``normal``, ``bias``, ``gain`` (around 1),
-    ``shift`` (around 0) or ``fraction`` (around one half, inside 0 .. 1). An extent of -1 in ``shape`` leaves that
+    ``shift`` (around 0), ``fraction`` (around one half, inside 0 .. 1), ``share`` (around one over the number of entries), ``open``
+    (around 1, with a third of it as deviation), ``identity`` (around the identity) or ``last`` (around 1 in the last column, 0 in the others). An extent of -1 in ``shape`` leaves that
     size to the weights file (the part then reads it off the tensor it is bound to).
     """
 
@@ -110,7 +111,8 @@ class DistanceSlopes:
 class QKNorm:
     """Queries and keys divided by a root mean square ``sqrt(mean(square) + eps)`` before rotation and scores: over
     every head by itself (``scope`` ``"head"``, gains of one head's size shared by all heads) or over the whole
-    projection of a token (``"projection"``, gains of the projection's size). ``gain`` ``False``: no gains."""
+    projection of a token (``"projection"``, gains of the projection's size). ``gain`` ``False``: no gains; over every head
+    by itself, the norm is then the same before and behind a rotation, which turns pairs of a head's own channels."""
 
     scope: str
     eps: float
@@ -300,6 +302,9 @@ class AttentionSpec:
     # the layer has no keys and values of its own: its schedule entry reads the cache of another (``reads_cache_of``),
     # and it holds no tensors of key and value projections or of their norm
     shares_kv: bool = False
+    # a causal convolution of this many taps over time on every channel of q, k and v, right after their projections
+    # (tensors ``q.conv``, ``k.conv``, ``v.conv`` ``[channels, taps]``)
+    conv_taps: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -360,6 +365,16 @@ class LatentAttentionSpec:
     output_gate: bool = True
     gate_per_head: bool = False
     window: Optional[int] = None
+
+
+@dataclass(frozen=True)
+class GateClamp:
+    """The constants of a clamped gated pair, ``g sigmoid(slope g) (u + shift)`` with ``g = min(gate, limit)`` and
+    ``u = clamp(up, -limit, limit)``."""
+
+    limit: float
+    slope: float = 1.702
+    shift: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -434,7 +449,10 @@ class RoutedExpertsSpec:
     number per token) if ``shared_gate``. ``gated`` ``False``: the experts are plain, ``down(act(up h))``.
     ``weigh_chosen``: choice and weights go by the logits alone, ``router h`` plus a stored bias (tensor ``router.bias``): the
     ``top`` largest are chosen and their weights are the softmax over the chosen logits (times ``scale``); there is no
-    ``correction``."""
+    ``correction``. ``scores`` ``"sigmoid"``: the scores are the logits' sigmoids, each by itself. ``group_best``: how many of
+    its largest choice scores a group counts by (their sum). ``clamp``: the experts, the shared one among them, are
+    ``down(g sigmoid(slope g) (u + shift))`` with ``g = min(gate h, limit)`` and ``u = clamp(up h, -limit, limit)`` (``activation``
+    is not read); ``shared_clamp``: the shared expert's own constants."""
 
     kind: str
     dim: int
@@ -450,6 +468,10 @@ class RoutedExpertsSpec:
     shared_gate: bool = True
     gated: bool = True
     weigh_chosen: bool = False
+    scores: str = "softmax"
+    group_best: int = 1
+    clamp: Optional[GateClamp] = None
+    shared_clamp: Optional[GateClamp] = None
 
 
 @dataclass(frozen=True)
@@ -468,6 +490,23 @@ class LinearAttentionSpec:
     eps: float
     activation: str = "silu"
     output_gate: bool = True
+
+
+@dataclass(frozen=True)
+class GatedLinearAttentionSpec:
+    """Linear attention whose state forgets channel by channel, by factors computed from the input: per head a state ``S``
+    ``[head_dim, value_dim]``, ``S <- diag(a_t) S + k v^T`` with ``a_t = sigmoid(z_t) ** (1 / tau)``, read as ``S^T q``
+    (``parts/gated_linear_attention.py``). ``decay_rank``: the size of the low-rank bottleneck that ``z`` comes through (``None``: as
+    the weights file has it)."""
+
+    kind: str
+    dim: int
+    n_heads: int
+    head_dim: int
+    value_dim: int
+    tau: float
+    eps: float                      # of the norm of every head's read-out
+    decay_rank: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -502,13 +541,25 @@ class MatrixMemorySpec:
 @dataclass(frozen=True)
 class BranchesSpec:
     """Mixers side by side on the same input: the result is ``sum_i weights[i] * rms(branch_i(h)) * gain_i``, every
-    branch's output normalised over the model width (``eps``) with a gain of its own."""
+    branch's output normalised over the model width (``eps``) with a gain of its own, or, with ``norms`` off,
+    ``sum_i weights[i] * branch_i(h)``."""
 
     kind: str
     dim: int
     branches: Tuple[object, ...]
     weights: Tuple[float, ...]
     eps: float
+    norms: bool = True
+
+
+@dataclass(frozen=True)
+class StreamMixSpec:
+    """The numbers by which a sublayer reads and writes ``streams`` copies of the residual stream (hyper-connections): it reads
+    ``sum_s in[s] x_s`` and, all at once, ``x_t <- sum_s mix[s, t] x_s + out[t] y`` with its output ``y`` (tensors ``in``, ``out``
+    ``[streams]`` and ``mix`` ``[streams, streams]``, from and to)."""
+
+    kind: str
+    streams: int
 
 
 @dataclass(frozen=True)
@@ -523,8 +574,11 @@ class LayerSpec:
     behind them (``feed_forward`` and ``norm2`` may be ``None``).
     ``norms_around`` = ``x += norm_after(mixer(norm(x))); x += norm2_after(ff(norm2(x)))`` (``feed_forward``, ``norm2`` and
     ``norm2_after`` may be ``None``).
+    ``streams`` = the stream is several copies (``ModelPlan.streams``), which mixer and feed-forward read and write by the
+    numbers of ``streams`` and ``streams2`` (``StreamMixSpec``), with ``norm`` and ``norm2`` on what they read
+    (``feed_forward``, ``norm2`` and ``streams2`` may be ``None``).
     ``names`` maps ``"<part>.<local tensor name>"`` (parts: ``norm``, ``norm2``, ``norm_after``,
-    ``norm2_after``, ``mixer``, ``feed_forward``) to the tensor's name in the checkpoint.
+    ``norm2_after``, ``streams``, ``streams2``, ``mixer``, ``feed_forward``) to the tensor's name in the checkpoint.
     """
 
     arrangement: str
@@ -536,6 +590,8 @@ class LayerSpec:
     residual_scale: float = 1.0        # weight of the branches' sum in arrangements that have one
     norm_after: Optional[object] = None
     norm2_after: Optional[object] = None
+    streams: Optional[object] = None
+    streams2: Optional[object] = None
 
 
 @dataclass(frozen=True)
@@ -584,6 +640,9 @@ class ModelPlan:
     junctions: Mapping[str, object] = field(default_factory=dict)
     # tensors of a checkpoint with these prefixes are passed over (parts that a configuration leaves out)
     ignored_prefixes: Tuple[str, ...] = ()
+    # copies of the residual stream, all equal to the embedding output at first and summed before the final norm (every
+    # layer is then of the arrangement ``streams``); ``None``: the stream is what it always is
+    streams: Optional[int] = None
 
     def describe(self) -> Dict[str, object]:
         return {"architecture": self.architecture, "layers": len(self.layers), "schedule": len(self.schedule),

@@ -56,6 +56,16 @@ def random_tensor(name: str, spec: ParamSpec, seed: int, recipe: InitRecipe, dev
         return 1.0 + noise * recipe.gain_std
     if spec.init == "shift":
         return noise * recipe.shift_std
+    if spec.init == "share":
+        return (1.0 + 0.3 * noise) / max(1, spec.shape[-1])
+    if spec.init == "open":
+        return 1.0 + 0.3 * noise
+    if spec.init == "identity":
+        return 0.85 * torch.eye(*spec.shape, dtype=torch.float32, device=device) + 0.08 * noise
+    if spec.init == "last":
+        base = torch.zeros_like(noise)
+        base[..., -1] = 1.0
+        return base + 0.3 * noise
     if spec.init == "fraction":
         return (0.5 + 0.15 * noise).clamp(0.05, 0.95)
     raise ValueError(f"{name}: unknown init {spec.init!r}")
