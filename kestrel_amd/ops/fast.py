@@ -74,6 +74,10 @@ _SIGNATURES = {
     "ka_matrix_memory_chunks_bf16": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                                      _c_void_p, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float,
                                      _c_void_p, _c_int, _c_void_p],
+    "ka_gated_chunks_supported": [_c_int, _c_int],
+    "ka_gated_chunks_scratch": [_c_int, _c_int, _c_int, _c_int, _c_int],
+    "ka_gated_chunks_bf16": [_c_void_p, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_float, _c_float, _c_void_p, _c_long, _c_void_p, _c_void_p,
+                             _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
     "ka_linear_chunks_bf16": [_c_void_p, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_void_p, _c_void_p,
                               _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
     "ka_linear_skinny_norm_store": [_c_void_p, _c_void_p, _c_void_p, _c_float, _c_int, _c_void_p, _c_long, _c_void_p, _c_void_p,
@@ -903,6 +907,47 @@ def linear_attention_chunks_bf16(projected, offsets, log2_decay, state, cu_q, ro
     _check(handle.ka_linear_chunks_bf16(base + oq * size, base + ok * size, base + ov * size, stride, log2_decay.data_ptr(), state.data_ptr(),
                                         state.stride(0), cu_q.data_ptr(), row_slot.data_ptr(), raw.data_ptr(), scratch.data_ptr(), n, n_rows,
                                         n_heads, head_dim, value_dim, int(act), stream_ptr()))
+    return True
+
+
+def gated_chunks_scratch(n: int, n_rows: int, n_heads: int, head_dim: int, value_dim: int) -> int:
+    """fp32 numbers of scratch that ``gated_chunks_bf16`` needs for a step of ``n`` tokens in ``n_rows`` rows; 0: the kernels do not
+    cover the head sizes."""
+    handle = lib()
+    handle.ka_gated_chunks_scratch.restype = ctypes.c_long
+    if not handle.ka_gated_chunks_supported(int(head_dim), int(value_dim)):
+        return 0
+    return int(handle.ka_gated_chunks_scratch(int(n), int(n_rows), int(n_heads), int(head_dim), int(value_dim)))
+
+
+def gated_chunks_bf16(projected, offsets, pre, tau, q_scale, state, cu_q, row_slot, raw, n_heads, head_dim, value_dim, scratch) -> bool:
+    """``ops.core.gated_linear_attention`` for prompt portions on the matrix cores: the recurrence unrolled over chunks of 64 tokens, all
+    chunks at once in three launches (operands as there; ``scratch``: contiguous fp32 of at least ``gated_chunks_scratch`` numbers).
+    False: sizes or alignment not covered, nothing was run."""
+    handle = lib()
+    n = projected.shape[0]
+    if n == 0:
+        return True
+    n_rows = int(row_slot.numel())
+    if projected.dtype != torch.bfloat16 or not handle.ka_gated_chunks_supported(int(head_dim), int(value_dim)):
+        return False
+    oq, ok, ov = (int(o) for o in offsets)
+    size, base = projected.element_size(), projected.data_ptr()
+    stride = projected.stride(0) if n > 1 else max(projected.stride(0), projected.shape[1])
+    if base % 16 or stride % 8 or any(o % 8 for o in (oq, ok, ov)) or projected.stride(1) != 1 or state.stride(0) % 4 or state.data_ptr() % 16 \
+            or n // 64 + n_rows > 65535:
+        return False
+    need = gated_chunks_scratch(n, n_rows, n_heads, head_dim, value_dim)
+    for t, numbers, what in ((scratch, need, "scratch"), (raw, n * n_heads * value_dim, "read-outs"), (pre, n * n_heads * head_dim, "pre-activations")):
+        if t.dtype != torch.float32 or not t.is_contiguous() or t.numel() < numbers or not t.is_cuda:
+            raise KernelError(f"gated linear attention: the {what} must be contiguous fp32 of at least {numbers} numbers")
+    if max(oq + n_heads * head_dim, ok + n_heads * head_dim, ov + n_heads * value_dim) > projected.shape[1] or not tau > 0 \
+            or state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or state.shape[1] != n_heads * head_dim * value_dim \
+            or cu_q.dtype != torch.int32 or cu_q.numel() != n_rows + 1 or row_slot.dtype != torch.int32:
+        raise KernelError("gated linear attention: operands do not fit the head sizes")
+    _check(handle.ka_gated_chunks_bf16(base + oq * size, base + ok * size, base + ov * size, stride, pre.data_ptr(), float(tau), float(q_scale),
+                                       state.data_ptr(), state.stride(0), cu_q.data_ptr(), row_slot.data_ptr(), raw.data_ptr(), scratch.data_ptr(),
+                                       n, n_rows, n_heads, head_dim, value_dim, stream_ptr()))
     return True
 
 

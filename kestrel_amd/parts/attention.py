@@ -249,14 +249,13 @@ class PagedAttention(Mixer):
     def share_projections(self, in_weight, proj_weight) -> None:
         self.qkv_weight, self.proj_weight = in_weight, proj_weight
 
-    def fold_output_weight(self, weight: float) -> bool:
-        if weight == 1.0:
-            return True
-        if not self.taps:
-            return False
-        # the heads are weighted sums of values, and the values of what their taps weigh: fp32 numbers that take up any factor
-        self._taps[self.q_dim + self.kv_dim:] *= float(weight)
-        return True
+    def takes_output_weight(self, weight: float) -> bool:
+        return weight == 1.0 or bool(self.taps)
+
+    def fold_output_weight(self, weight: float) -> None:
+        if weight != 1.0:
+            # the heads are weighted sums of values, and the values of what their taps weigh: fp32 numbers that take up any factor
+            self._taps[self.q_dim + self.kv_dim:] *= float(weight)
 
     def _decodes_fused(self, batch, cache: LayerCache) -> bool:
         """One token per row in bf16 with a rotation by halves: the decode kernel then rotates q and

@@ -211,10 +211,13 @@ class Mixer(Part):
         """Hold these views of joint tensors instead of the mixer's own two weights (same values)."""
         raise NotImplementedError
 
-    def fold_output_weight(self, weight: float) -> bool:
-        """Whether what ``attend`` returns is ``weight`` times what it would be from now on, at no cost and no loss (a factor
-        that some fp32 constant of the mixer takes up)."""
+    def takes_output_weight(self, weight: float) -> bool:
+        """Whether ``fold_output_weight`` can take this weight up."""
         return weight == 1.0
+
+    def fold_output_weight(self, weight: float) -> None:
+        """What ``attend`` returns is ``weight`` times what it would be from now on, at no cost and no loss (a factor that some
+        fp32 constant of the mixer takes up)."""
 
 
 class FeedForward(Part):

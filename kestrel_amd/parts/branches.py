@@ -74,16 +74,11 @@ class Branches(Mixer):
             return
         if any(type(b).share_projections is Mixer.share_projections for b in self.branches):
             return
-        # (asked of all before any is changed: a weight that one branch folds must not be applied again)
-        weights = self.spec.weights
-        if not all(float(w) == 1.0 or type(b).fold_output_weight is not Mixer.fold_output_weight for b, w in zip(self.branches, weights)):
+        # (asked of all before any is changed: the weights are either all taken up or all applied to what the branches give)
+        if not all(b.takes_output_weight(float(w)) for b, w in zip(self.branches, self.spec.weights)):
             return
-        folded = [b.fold_output_weight(float(w)) for b, w in zip(self.branches, weights)]
-        if not all(folded):
-            for b, w, done in zip(self.branches, weights, folded):
-                if done and float(w) != 1.0:
-                    b.fold_output_weight(1.0 / float(w))
-            return
+        for b, w in zip(self.branches, self.spec.weights):
+            b.fold_output_weight(float(w))
         self.in_weight = torch.cat([stage[0] for stage in ins], dim=0).contiguous()
         self.proj_weight = torch.cat([stage[0] for stage in outs], dim=1).contiguous()
         self.in_cols, self.out_cols = [0], [0]

@@ -84,9 +84,11 @@ class GatedLinearAttention(Mixer):
     def share_projections(self, in_weight, proj_weight) -> None:
         self.in_weight, self.proj_weight = in_weight, proj_weight
 
-    def fold_output_weight(self, weight: float) -> bool:
-        self.gain = self.gain * float(weight)          # (the last factor of the heads before the gate, fp32)
+    def takes_output_weight(self, weight: float) -> bool:
         return True
+
+    def fold_output_weight(self, weight: float) -> None:
+        self.gain = self.gain * float(weight)          # (the last factor of the heads before the gate, fp32)
 
     def attend(self, projected, batch, cache: LayerCache, beside=None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
         """The recurrence over the step's tokens, normalised and gated: the input of the output projection."""
@@ -100,7 +102,16 @@ class GatedLinearAttention(Mixer):
         raw = ws.get("gated_attention.raw", (n, self.v_dim), torch.float32)
         sizes = (spec.n_heads, spec.head_dim, spec.value_dim)
         q_scale = float(spec.head_dim) ** -0.5
-        core.gated_linear_attention(projected, self.offsets, pre, float(spec.tau), q_scale, cache.state, batch.cu_q, batch.row_slot, raw, *sizes)
+        operands = (projected, self.offsets, pre, float(spec.tau), q_scale, cache.state, batch.cu_q, batch.row_slot, raw, *sizes)
+        done = False
+        if self.dtype == torch.bfloat16 and not batch.decode_only and n >= self.CHUNKS_FROM_TOKENS:
+            # (sized by the host side of the batch alone: the same for every replay of a captured step)
+            from ..ops import fast
+            need = fast.gated_chunks_scratch(n, batch.n_rows, *sizes)
+            if need:
+                done = fast.gated_chunks_bf16(*operands, ws.get("gated_attention.chunks", (need,), torch.float32))
+        if not done:
+            core.gated_linear_attention(*operands)
         if out is None:
             out = ws.get("gated_attention.out", (n, self.v_dim), self.dtype)
         core.heads_rmsnorm(raw, self.gain, projected[:, self.gate_at:self.gate_at + self.v_dim], out, spec.n_heads, spec.value_dim, float(spec.eps))
