@@ -24,7 +24,9 @@ layer of chunked attention beside a matrix memory) at sizes of its own (``BOGIVI
 ``--workload compare-letevik`` for the Letevik design (differential attention behind short convolutions and latent
 attention in a looped stretch of layers; ``LETEVIK_SIZES``), and ``--workload compare-vufolorn`` for the Vufolorn design (a
 linear recurrence with a decay per head, windowed latent attention, routed plain experts; ``VUFOLORN_SIZES``), which also
-has Bokorax, the design closest to it, beside it.
+has Bokorax, the design closest to it, beside it. ``--workload compare-gozatar`` does it for the Gozatar design (several
+residual streams, windowed attention beside gated linear attention in every layer, routed clamped experts;
+``GOZATAR_SIZES``), with Bogivik (the closest mixer) and Bokorax (the closest feed-forward) beside it.
 """
 
 from __future__ import annotations
@@ -254,7 +256,7 @@ def design_facts(net):
             # the shared rotated key part
             attention.append((spec.n_heads * (spec.head_dim + spec.rot_dim + spec.value_dim), spec.kv_rank + spec.rot_dim,
                               getattr(spec, "window", None), None, 0))
-        elif kind in ("matrix_memory", "linear_attention"):
+        elif kind in ("matrix_memory", "linear_attention", "gated_linear_attention"):
             memory.append((spec.n_heads, spec.head_dim, spec.value_dim))
         elif kind == "decayed_memory":
             memory.append((spec.n_heads, spec.head_dim, spec.head_dim))
@@ -426,6 +428,48 @@ def vufolorn_models(size: dict, positions: int):
                                             shared=e["shared"] * 2 // 3),
                                order=size["order"].replace("r", "w").replace("a", "1")), positions)
     return {"vufolorn": (vufolorn, "vufolorn"), **both}
+
+
+# Sizes at which Gozatar is measured beside Bogivik, whose parallel layers have the closest mixer (attention over the last keys
+# beside a recurrence), beside Bokorax, whose experts are the closest feed-forward (gated, in groups, with a shared one),
+# and beside the Moondream decoder: width, streams, attention's heads, kv heads and head size (keys and values), window, taps, the
+# recurrence's heads and head sizes, the rank of its decay, the experts (how many, their hidden size, choices per token, groups
+# and kept groups, the shared expert) and the order of layers by their feed-forward (d: a dense one of one and a half times `ff`, m:
+# the experts). Bogivik gets parallel layers alone, a matrix memory of its own head sizes with as many value channels and gated
+# feed-forwards of `ff`; Bokorax the same experts behind windowed attention and a decaying memory in turn.
+GOZATAR_SIZES = {
+    "w2048": dict(width=2048, ff=5632, streams=4, heads=32, kv_heads=8, head=64, window=1024, conv=4, recurrence=(16, 64, 128), rank=64,
+                  experts=dict(n=30, ff=704, top=4, groups=(5, 3), shared=704), memory=(8, 64, 256), order="dmmm"),
+    "w4096": dict(width=4096, ff=7168, streams=4, heads=32, kv_heads=8, head=128, window=2048, conv=4, recurrence=(32, 64, 128), rank=128,
+                  experts=dict(n=62, ff=896, top=6, groups=(2, 1), shared=1792), memory=(16, 64, 256), order="dmm"),
+}
+
+
+def gozatar_models(size: dict, positions: int):
+    """``{name: (config dict, registry name)}`` of Gozatar, Bogivik, Bokorax and the Moondream decoder at one size."""
+    w, h, g, d, e = size["width"], size["heads"], size["kv_heads"], size["head"], size["experts"]
+    rh, rd, rdv = size["recurrence"]
+    limits = {"limit": 7.0}
+    experts = {"kind": "moe", "expert": {"ff": e["ff"], **limits}, "shared": {"ff": e["shared"], **limits},
+               "router": {"experts": e["n"], "top": e["top"], "groups": dict(zip(("count", "keep"), e["groups"]))}}
+    mixer = {"left": {"heads": h, "kv_heads": g, "dim": d, "vdim": d, "scale": 1.0, "conv": size["conv"], "mask": {"size": size["window"]},
+                      "rot": {"base": 10000.0, "dims": d}},
+             "right": {"heads": rh, "dim": rd, "vdim": rdv, "tau": 16.0, "decay_rank": size["rank"]}, "left_scale": 0.8, "right_scale": 1.2}
+    layers = [{"type": "parallel", "mixer": mixer, "mlp": {"kind": "dense", "ff": size["ff"] * 3 // 2} if kind == "d" else experts}
+              for kind in size["order"]]
+    gozatar = {"architecture": "Gozatar", "vocab": COMPARE_VOCAB, "width": w, "streams": size["streams"], "norm": {"eps": 1e-5},
+               "max_positions": positions, "layers": layers}
+    count = len(size["order"])
+    first = bogivik_models(dict(width=w, ff=size["ff"], heads=h, kv_heads=g, head=d, chunk=size["window"], memory=size["memory"], order="p" * count), positions)
+    second = bokorax_models(dict(width=w, ff=size["ff"], heads=h, kv_heads=g, head=d, window=size["window"], memory=(rh * rd // 64 * 2, 64), rank=size["rank"],
+                                 experts=dict(n=e["n"], ff=e["ff"], top=e["top"], identity=0, groups=e["groups"], shared=e["shared"]),
+                                 order=("1w" * count)[:count]), positions)
+    return {"gozatar": (gozatar, "gozatar"), "bogivik": first["bogivik"], "bokorax": second["bokorax"], "moondream2": first["moondream2"]}
+
+
+def run_compare_gozatar(args, dtype, device) -> dict:
+    """Gozatar beside Bogivik, Bokorax and the Moondream decoder at equal sizes, through the same step function."""
+    return run_compare_design(args, dtype, device, "gozatar", GOZATAR_SIZES, gozatar_models)
 
 
 def run_compare_vufolorn(args, dtype, device) -> dict:
@@ -783,14 +827,14 @@ def main() -> int:
     parser.add_argument("--check", type=int, default=0,
                         help="with --workload: compare this many greedy requests with the plain implementation (for --layers 2)")
     parser.add_argument("--workload", default="decode", choices=["decode", "waves256", "mixed48", "compare-vimesun", "compare-bogivik", "compare-letevik", "compare-bokorax",
-                                                                     "compare-vufolorn"],
+                                                                     "compare-vufolorn", "compare-gozatar"],
                         help="decode: the benchmark's decode step (default); waves256 and mixed48 run requests through "
                              "InferenceEngine; compare-vimesun, compare-bogivik and compare-letevik measure that design beside the Moondream "
                              "decoder at equal sizes")
     parser.add_argument("--compare-sizes", default=None,
                         help="with --workload compare-*: which of its sizes, with commas between them "
                              "(default: all of them)")
-    parser.add_argument("--compare-model", default="both", choices=["both", "vimesun", "bogivik", "letevik", "bokorax", "vufolorn", "moondream2"],
+    parser.add_argument("--compare-model", default="both", choices=["both", "vimesun", "bogivik", "letevik", "bokorax", "vufolorn", "gozatar", "moondream2"],
                         help="with --workload compare-*: one of the two designs only (for profiling)")
     parser.add_argument("--compare-batches", default="1,8,64", help="with --workload compare-bogivik or compare-letevik: batch sizes of the decode steps")
     parser.add_argument("--skip-prefill", action="store_true", help="with --workload compare-bogivik or compare-letevik: decode steps only")
@@ -831,6 +875,9 @@ def main() -> int:
         return 0
     if args.workload == "compare-vufolorn":
         print(json.dumps(run_compare_vufolorn(args, dtype, device)))
+        return 0
+    if args.workload == "compare-gozatar":
+        print(json.dumps(run_compare_gozatar(args, dtype, device)))
         return 0
     if args.workload == "compare-letevik":
         print(json.dumps(run_compare_letevik(args, dtype, device)))

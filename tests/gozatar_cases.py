@@ -57,7 +57,7 @@ CONFIGS: Dict[str, dict] = {
     # three, one choice, decays that forget at once (tau below 1), a layer without a feed-forward
     "Q": _config(211, 100, 5, 1e-6, [
         parallel((3, 1, 12, 10, 0.35, 6, 7, 6, 100.0), (5, 10, 7, 0.3, 5), (1.2, 0.6), moe(6, 20, 0.7, 2, (2, 1))),
-        parallel((5, 5, 20, 6, 0.25, None, None, 20, 2000.0), (2, 1, 33, 16.0, 3), (0.9, -0.8), None),
+        parallel((5, 5, 20, 6, 0.25, None, None, 20, 2000.0), (2, 6, 33, 16.0, 3), (0.9, -0.8), None),
         parallel((4, 2, 18, 36, 0.3, 1, 11, 2, 7.0), (3, 22, 12, 1.0, 7), (-0.5, 1.1), moe(3, 24, 3.0, 1, None, (36, 0.5))),
         parallel((2, 1, 40, 18, 0.2, 5, 19, 12, 50.0), (1, 36, 20, 5.0, 9), (1.0, 0.9), dense(70)),
     ]),

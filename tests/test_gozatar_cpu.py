@@ -102,7 +102,7 @@ def test_streams_cache_groups_and_state():
     assert needs[0][1].shape == (3 * 320 + 3 * 32 * 40,) and needs[0][1].dtype == "float32"
     needs = DecoderModel(_plan("Q")).cache_needs()
     assert needs[0][1].shape == ((5 * (36 + 12 + 10) + 3) // 4 * 4 + (5 * 70 + 3) // 4 * 4,)
-    assert needs[1][1].shape == (2 * 33,) and needs[2][1].shape == (3 * 22 * 12,)       # no taps, or one: no rows to keep
+    assert needs[1][1].shape == (2 * 6 * 33,) and needs[2][1].shape == (3 * 22 * 12,)       # no taps, or one: no rows to keep
 
 
 def test_a_window_gives_its_pages_back():

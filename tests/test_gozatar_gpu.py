@@ -76,7 +76,7 @@ def _what_rounding_does(folder, ids):
 
 def _close(got, want, dtype, what, folder=None, ids=None):
     """Row by row: the root mean square of the difference over the vocabulary (mean taken off) as a share of the row's
-    spread: at most 5e-5 in float32, 4 % in bfloat16 or what rounding alone moves that row by if that is more
+    spread: at most 5e-5 in float32, 5 % in bfloat16 or what rounding alone moves that row by if that is more
     (``_what_rounding_does``), and no single value off by more than four times that."""
     got, want = got.detach().double().cpu(), want.detach().double().cpu()
     assert got.shape == want.shape, f"{what}: shape {tuple(got.shape)} vs {tuple(want.shape)}"
@@ -84,7 +84,7 @@ def _close(got, want, dtype, what, folder=None, ids=None):
     diff = diff - diff.mean(dim=-1, keepdim=True)
     spread = want.std(dim=-1, unbiased=False)
     rms, top = diff.pow(2).mean(dim=-1).sqrt() / spread, diff.abs().max(dim=-1).values / spread
-    bound = torch.full_like(rms, 5e-5 if dtype == torch.float32 else 0.04)
+    bound = torch.full_like(rms, 5e-5 if dtype == torch.float32 else 0.05)
     if dtype == torch.bfloat16 and folder is not None and not bool((rms <= bound).all() and (top <= 4 * bound).all()):
         bound = torch.maximum(bound, _what_rounding_does(folder, ids))
     worst = int(torch.argmax(rms / bound))
@@ -502,10 +502,19 @@ def test_every_layer(name, dtype):
     streams = []
     want = plain.forward(cases.config_of(folder), cases.stored_weights(folder), ids, streams)
     assert len(seen) == len(streams)
-    for layer, (a, b) in enumerate(zip(seen, streams)):
-        rms = ((a - b).pow(2).mean(dim=-1) / b.pow(2).mean(dim=-1)).sqrt()
-        assert float(rms.max()) <= (2e-5 if dtype == torch.float32 else 3e-2), f"{name} layer run {layer}: {float(rms.max()):.3g}"
-    _close(got["r"], want, dtype, f"{name} logits")
+    apart = lambda a, b: ((a - b).pow(2).mean(dim=-1) / b.pow(2).mean(dim=-1)).sqrt()  # noqa: E731
+    bounds = [torch.full((len(ids),), 2e-5 if dtype == torch.float32 else 3e-2, dtype=F64) for _ in streams]
+    if dtype == torch.bfloat16:                     # (or what rounding alone moves the row by, ``_what_rounding_does``)
+        gen = torch.Generator().manual_seed(98)
+        for _ in range(3):
+            moved = []
+            plain.forward(cases.config_of(folder), {k: v.double() * (1 + 2.0 ** -8 * torch.randn(v.shape, generator=gen, dtype=F64))
+                                                    for k, v in cases.stored_weights(folder).items()}, ids, moved)
+            bounds = [torch.maximum(bound, apart(a, b)) for bound, a, b in zip(bounds, moved, streams)]
+    for layer, (a, b, bound) in enumerate(zip(seen, streams, bounds)):
+        over = apart(a, b) / bound
+        assert float(over.max()) <= 1.0, f"{name} layer run {layer}: row {int(over.argmax())} is {float(over.max()):.3g} times its bound away"
+    _close(got["r"], want, dtype, f"{name} logits", folder, ids)
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=DTYPE_IDS)
@@ -594,7 +603,7 @@ def test_replayed_steps_of_any_shape(name, dtype):
         want = _expected(folder, req.ids)
         bound = None
         if dtype == torch.bfloat16:
-            bound = torch.clamp(_what_rounding_does(folder, req.ids)[places], min=0.04)
+            bound = torch.clamp(_what_rounding_does(folder, req.ids)[places], min=0.05)
         diff = torch.stack([got[tag][p] for p in places]).double().cpu() - want[places]
         diff = diff - diff.mean(dim=-1, keepdim=True)
         rms = diff.pow(2).mean(dim=-1).sqrt() / want[places].std(dim=-1, unbiased=False)
@@ -646,7 +655,7 @@ def test_a_far_key_and_the_windows_edges_in_the_model(dtype):
             runner = _runner(folder, dtype)
             reqs = {"r": Request("r", ids)}
             got = helpers.replay(runner, reqs, [[("r", head)]] + [[("r", 1)]] * (len(ids) - head))
-            _close(got["r"], want, dtype, f"distance {distance}, prompt of {head}")
+            _close(got["r"], want, dtype, f"distance {distance}, prompt of {head}", folder, ids)
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
