@@ -8,20 +8,13 @@
 #include "ka_rows.h"
 
 constexpr int EX_MAX_OUTPUTS = 512;             // router outputs a wave can hold (8 a lane)
-constexpr int EX_PER_LANE = EX_MAX_OUTPUTS / KA_WAVE;
 constexpr int EX_MAX_GROUPS = 64;
 
-// The largest value of a wave and the lowest index that holds it, in every lane.
-__device__ __forceinline__ void ex_wave_argmax(float& v, int& i) {
-#pragma unroll
-    for (int step = 1; step < KA_WAVE; step <<= 1) {
-        const float ov = __shfl_xor(v, step);
-        const int oi = __shfl_xor(i, step);
-        if (ov > v || (ov == v && oi < i)) {
-            v = ov;
-            i = oi;
-        }
-    }
+// The lowest index that holds the largest value of a wave (of at most `last`), in every lane.
+__device__ __forceinline__ int ex_wave_argmax(float v, int i, int last) {
+    const float best = ka_wave_max(v);
+    const int found = ka_lanes_reduce<1, KA_WAVE>(v == best ? i : 0x7fffffff, KaIntMin{});
+    return __builtin_amdgcn_readfirstlane(min(found, last));
 }
 
 // ----------------------------------------------------------------------------
@@ -36,19 +29,20 @@ __device__ __forceinline__ void ex_wave_argmax(float& v, int& i) {
 // chosen int32 [n, top], weights fp32 [n, top]; always >= 0: the rows are one longer and end in that output with weight 1 (a
 // feed-forward that every token uses, laid behind the experts).
 // ----------------------------------------------------------------------------
+template <int PER_LANE>          // outputs a lane holds
 __global__ void __launch_bounds__(KA_WAVE)
 route_kernel(const float* __restrict__ logits, long stride, const float* __restrict__ correction, int R, int top, int n_groups,
              int keep, int group_best, float scale, int mode, int always, int* __restrict__ chosen, float* __restrict__ weights) {
-    __shared__ float choice_s[EX_MAX_OUTPUTS];
+    __shared__ float choice_s[PER_LANE * KA_WAVE];
     __shared__ float group_s[EX_MAX_GROUPS];
     __shared__ int allowed_s[EX_MAX_GROUPS];
     const int t = blockIdx.x, lane = threadIdx.x;
     const bool by_logits = mode == 1, sigmoids = mode == 2;
     const float* z = logits + (size_t)t * stride;
-    float s[EX_PER_LANE], c[EX_PER_LANE];
+    float s[PER_LANE], c[PER_LANE];
     float top_z = -INFINITY;
 #pragma unroll
-    for (int q = 0; q < EX_PER_LANE; ++q) {
+    for (int q = 0; q < PER_LANE; ++q) {
         const int r = lane + q * KA_WAVE;
         s[q] = r < R ? z[r] : -INFINITY;
         top_z = fmaxf(top_z, s[q]);
@@ -56,7 +50,7 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
     top_z = ka_wave_max(top_z);
     float total = 0.f;
 #pragma unroll
-    for (int q = 0; q < EX_PER_LANE; ++q) {
+    for (int q = 0; q < PER_LANE; ++q) {
         c[q] = s[q];
         if (sigmoids) s[q] = lane + q * KA_WAVE < R ? 1.0f / (1.0f + expf(-s[q])) : 0.f;
         else s[q] = lane + q * KA_WAVE < R ? expf(s[q] - top_z) : 0.f;
@@ -64,7 +58,7 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
     }
     total = ka_wave_sum(total);
 #pragma unroll
-    for (int q = 0; q < EX_PER_LANE; ++q) {
+    for (int q = 0; q < PER_LANE; ++q) {
         const int r = lane + q * KA_WAVE;
         if (by_logits) continue;      // (the largest logit is among the chosen: e^(z - top) over their sum is their softmax)
         if (!sigmoids) s[q] = s[q] / total;
@@ -82,19 +76,17 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
                 best = fmaxf(best, v);
             }
             group_s[lane] = group_best == 2 && per > 1 ? best + second : best;
-            allowed_s[lane] = 0;
         }
         __syncthreads();
-        for (int turn = 0; turn < keep; ++turn) {
-            float v = lane < n_groups && !allowed_s[lane] ? group_s[lane] : -INFINITY;
-            int i = lane < n_groups && !allowed_s[lane] ? lane : 0x7fffffff;
-            ex_wave_argmax(v, i);
-            __syncthreads();
-            if (lane == 0 && i < n_groups) allowed_s[i] = 1;
-            __syncthreads();
+        if (lane < n_groups) {
+            const float own = group_s[lane];
+            int ahead = 0;              // groups that are kept before this one (the lower index wins a tie)
+            for (int g = 0; g < n_groups; ++g) ahead += group_s[g] > own || (group_s[g] == own && g < lane);
+            allowed_s[lane] = ahead < keep;
         }
+        __syncthreads();
 #pragma unroll
-        for (int q = 0; q < EX_PER_LANE; ++q) {
+        for (int q = 0; q < PER_LANE; ++q) {
             const int r = lane + q * KA_WAVE;
             if (r < R && !allowed_s[r / per]) c[q] = -INFINITY;
         }
@@ -107,22 +99,22 @@ route_kernel(const float* __restrict__ logits, long stride, const float* __restr
         float v = -INFINITY;
         int i = 0x7fffffff;
 #pragma unroll
-        for (int q = 0; q < EX_PER_LANE; ++q) {
+        for (int q = 0; q < PER_LANE; ++q) {
             const int r = lane + q * KA_WAVE;
             if (r < R && !(taken >> q & 1) && (c[q] > v || i == 0x7fffffff)) {
                 v = c[q];
                 i = r;
             }
         }
-        ex_wave_argmax(v, i);
+        i = ex_wave_argmax(v, i, R - 1);
         float sv = 0.f;
 #pragma unroll
-        for (int q = 0; q < EX_PER_LANE; ++q)
+        for (int q = 0; q < PER_LANE; ++q)
             if (lane + q * KA_WAVE == i) {
                 taken |= 1u << q;
                 sv = s[q];
             }
-        sv = ka_wave_sum(sv);    // (one lane holds it, the others 0)
+        sv = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(sv), i % KA_WAVE));       // (one lane holds it)
         sum += sv;
         if (lane == k % KA_WAVE) {
             // (more than a wave of choices would need more than one register a lane: the entry point refuses it)
@@ -152,8 +144,12 @@ KA_API int ka_route(const float* logits, long stride, const float* correction, i
              "%s: %d groups of which %d are kept do not divide %d outputs", who, n_groups, keep, R);
     KA_CHECK(n_groups == 0 || keep * (R / n_groups) >= top, "%s: %d kept groups hold fewer than %d outputs", who, keep, top);
     if (n == 0) return 0;
-    hipLaunchKernelGGL(route_kernel, dim3(n), dim3(KA_WAVE), 0, stream, logits, stride, correction, R, top, n_groups, keep, group_best,
-                       scale, mode, always, chosen, weights);
+#define EX_ROUTE(PER_LANE) \
+    hipLaunchKernelGGL(route_kernel<PER_LANE>, dim3(n), dim3(KA_WAVE), 0, stream, logits, stride, correction, R, top, n_groups, keep, group_best, scale, mode, always, chosen, weights)
+    if (R <= KA_WAVE) EX_ROUTE(1);
+    else if (R <= 2 * KA_WAVE) EX_ROUTE(2);
+    else EX_ROUTE(EX_MAX_OUTPUTS / KA_WAVE);
+#undef EX_ROUTE
     KA_LAUNCH_CHECK();
     return 0;
 }

@@ -118,10 +118,10 @@ struct ConvArgs {
     int normed;
     float eps;
     // the form of eight channels a thread: the tokens cut into runs of at most page_size (null: every token by itself), and
-    // whether every row brings one token (its thread then moves the state on as well)
+    // whether every row brings one token, row t token t (its thread then moves the state on as well)
     const int* run_first;
     const int* run_count;
-    int moves_state;
+    int single_tokens;
 };
 
 template <typename T>
@@ -247,12 +247,13 @@ __global__ void __launch_bounds__(SP_THREADS) conv_prepare_normed_kernel(ConvArg
 // The same for bf16 rows, up to SP_WIDE_TAPS taps, and query and key heads of 8 LPH channels, LPH a power of two: a thread
 // keeps eight neighbouring channels, their taps and the rows the taps still reach in registers and walks over the tokens of a
 // run, one 16-byte load a token; a head's sum of squares meets inside its LPH lanes, and the lanes of a rotated pair of
-// halves exchange their numbers. Grid (blocks of 2,048 channels: queries and keys, then values; runs). Values of a run that
-// fills a page leave as 32 bytes a channel. rot is a multiple of 16 for pairs of halves.
+// halves exchange their numbers. Grid (blocks of 2,048 channels: queries and keys, then values; runs; parts of a run). Eight values
+// of a channel that lie side by side in a page leave together. rot is a multiple of 16 for pairs of halves.
 typedef __attribute__((ext_vector_type(8))) __bf16 sp_bf16x8;
 typedef __attribute__((ext_vector_type(4))) float sp_floatx4;
 constexpr int SP_WIDE_TAPS = 4;
 constexpr int SP_WIDE_RUN = 16;                     // tokens of a run at most
+constexpr int SP_WIDE_QK = 4, SP_WIDE_V = 8;        // tokens of a run a workgroup takes, of queries and keys and of values
 constexpr int SP_WIDE_MAX_ROT = 256;
 
 // Whatever `back` = 1 .. SP_WIDE_TAPS - 1 rows before token t hold of channels c .. c + 7, into hist[back - 1].
@@ -276,46 +277,84 @@ __device__ __forceinline__ void sp_wide_history(const ConvArgs& a, int t, int lo
     }
 }
 
+// The taps of channels c .. c + 7 as w[back]: the tap that reads `back` rows before (0: behind the last). K numbers a channel, side
+// by side.
+template <int K>
+__device__ __forceinline__ void sp_wide_taps(const float* taps, int c, float (&w)[SP_WIDE_TAPS][8]) {
+    float flat[8 * K];
+    const float* src = taps + (size_t)c * K;
+#pragma unroll
+    for (int i = 0; i < 2 * K; ++i) {
+        const sp_floatx4 v = *reinterpret_cast<const sp_floatx4*>(src + 4 * i);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) flat[4 * i + e] = v[e];
+    }
+#pragma unroll
+    for (int back = 0; back < SP_WIDE_TAPS; ++back)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) w[back][e] = back < K ? flat[e * K + (back < K ? K - 1 - back : 0)] : 0.f;
+}
+
 template <int LPH>
 __global__ void __launch_bounds__(SP_THREADS) conv_prepare_wide_kernel(ConvArgs a) {
-    __shared__ float cs[SP_WIDE_RUN][SP_WIDE_MAX_ROT / 2], sn[SP_WIDE_RUN][SP_WIDE_MAX_ROT / 2];
+    __shared__ __attribute__((aligned(16))) float cs[SP_WIDE_QK][SP_WIDE_MAX_ROT / 2], sn[SP_WIDE_QK][SP_WIDE_MAX_ROT / 2];
+    __shared__ int row_s[SP_WIDE_V], at_s[SP_WIDE_V];
     constexpr int HD = 8 * LPH;
     const int tid = threadIdx.x;
     const int Cqk = (a.Hq + a.Hk) * HD, Cv = a.Hv * a.hdv;
     const int qk_blocks = (Cqk + 8 * SP_THREADS - 1) / (8 * SP_THREADS);
     const bool values = (int)blockIdx.x >= qk_blocks;
-    const int first = a.run_first ? a.run_first[blockIdx.y] : (int)blockIdx.y;
-    const int count = a.run_first ? min(a.run_count[blockIdx.y], SP_WIDE_RUN) : 1;
+    // this workgroup's tokens of the run
+    const int part = values ? SP_WIDE_V : SP_WIDE_QK;
+    const int first = (a.run_first ? a.run_first[blockIdx.y] : (int)blockIdx.y) + (int)blockIdx.z * part;
+    const int count = min((a.run_first ? min(a.run_count[blockIdx.y], SP_WIDE_RUN) : 1) - (int)blockIdx.z * part, part);
     if (count <= 0) return;
-    const int half = a.rot / 2;
-    if (a.freqs && !values) {
-        for (int e = tid; e < count * half; e += SP_THREADS)
-            sincosf((float)a.positions[first + e / half] * a.freqs[e % half], &sn[e / half][e % half], &cs[e / half][e % half]);
-        __syncthreads();
-    }
     // (threads behind the last channel do the work of the first ones and store nothing: all lanes of a wave stay together)
     const int mine = ((int)blockIdx.x - (values ? qk_blocks : 0)) * SP_THREADS + tid;
     const bool live = 8 * mine < (values ? Cv : Cqk);
     const int within = live ? 8 * mine : 8 * (tid % LPH);
     const int c = values ? Cqk + (live ? 8 * mine : 0) : within;
-    float w[SP_WIDE_TAPS][8];               // w[back]: the tap that reads `back` rows before
+    const bf16_t* u = reinterpret_cast<const bf16_t*>(a.u) + c;
+    sp_bf16x8 rows[SP_WIDE_V];
 #pragma unroll
-    for (int back = 0; back < SP_WIDE_TAPS; ++back)
-#pragma unroll
-        for (int e = 0; e < 8; ++e) w[back][e] = back < a.K ? a.taps[(size_t)(c + e) * a.K + (a.K - 1 - back)] : 0.f;
-    const bf16_t* u = reinterpret_cast<const bf16_t*>(a.u);
+    for (int i = 0; i < SP_WIDE_V; ++i)
+        if (i < count) rows[i] = *reinterpret_cast<const sp_bf16x8*>(u + (size_t)(first + i) * a.u_stride);
+    float w[SP_WIDE_TAPS][8];
+    switch (a.K) {
+        case 1: sp_wide_taps<1>(a.taps, c, w); break;
+        case 2: sp_wide_taps<2>(a.taps, c, w); break;
+        case 3: sp_wide_taps<3>(a.taps, c, w); break;
+        default: sp_wide_taps<4>(a.taps, c, w); break;
+    }
     float hist[SP_WIDE_TAPS - 1][8];
-    int row = -1, slot = -1;
-    // the rows before token t, where it is not the one behind the last token of its row
-    auto enter = [&](int t) {
-        const int r = a.token_row[t];
+    int row, slot;
+    if (a.single_tokens) {                          // (row t brings token t, its first)
+        row = first;
+        slot = a.row_slot[row];
+        sp_wide_history(a, first, 0, slot, c, hist);
+    } else {
+        row = a.token_row[first];
+        slot = a.row_slot[row];
+        sp_wide_history(a, first, first - a.cu_q[row], slot, c, hist);
+    }
+    const int half = a.rot / 2;
+    if (tid < count) {
+        row_s[tid] = a.single_tokens ? row : a.token_row[first + tid];
+        at_s[tid] = a.slots ? a.slots[first + tid] : -1;
+    }
+    if (a.freqs && !values)
+        for (int e = tid; e < count * half; e += SP_THREADS)
+            sincosf((float)a.positions[first + e / half] * a.freqs[e % half], &sn[e / half][e % half], &cs[e / half][e % half]);
+    __syncthreads();
+    // the rows before token i of the run, where it is not the one behind the last token of its row
+    auto enter = [&](int i) {
+        const int r = row_s[i];
         if (r == row) return;
         row = r;
         slot = a.row_slot[r];
-        sp_wide_history(a, t, t - a.cu_q[r], slot, c, hist);
+        sp_wide_history(a, first + i, first + i - a.cu_q[r], slot, c, hist);
     };
-    auto convolve = [&](int t, float (&y)[8]) {
-        const sp_bf16x8 x = *reinterpret_cast<const sp_bf16x8*>(u + (size_t)t * a.u_stride + c);
+    auto convolve = [&](const sp_bf16x8& x, float (&y)[8]) {
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
             float s = 0.f;
@@ -332,7 +371,7 @@ __global__ void __launch_bounds__(SP_THREADS) conv_prepare_wide_kernel(ConvArgs 
     };
     // (the row's only token: entry s of the state is now what stands K - 2 - s rows before the next token's predecessor)
     auto move_state = [&]() {
-        if (!a.moves_state || slot < 0 || !live) return;
+        if (!a.single_tokens || slot < 0 || !live) return;
         float* st = a.state + (size_t)slot * a.state_stride + c;
 #pragma unroll
         for (int back = 0; back < SP_WIDE_TAPS - 1; ++back) {
@@ -347,11 +386,17 @@ __global__ void __launch_bounds__(SP_THREADS) conv_prepare_wide_kernel(ConvArgs 
     if (!values) {
         const int head = within / HD, sub = within % HD / 8;
         const bool is_q = head < a.Hq;
-        for (int i = 0; i < count; ++i) {
-            const int t = first + i;
+        // (what a channel's rotation does is the same for every token)
+        const int apart = a.rot / 16;
+        const bool low = sub < apart, turned = a.freqs && !a.interleaved && sub < 2 * apart;
+        const int partner = (turned ? (tid % KA_WAVE) + (low ? apart : -apart) : tid % KA_WAVE);
+        const int j0 = (low ? sub : sub - apart) * 8;
+#pragma unroll
+        for (int i = 0; i < SP_WIDE_QK; ++i) {
+            if (i >= count) break;
             float y[8];
-            enter(t);
-            convolve(t, y);
+            enter(i);
+            convolve(rows[i], y);
             if (a.normed) {
                 float ss = 0.f;
 #pragma unroll
@@ -371,17 +416,16 @@ __global__ void __launch_bounds__(SP_THREADS) conv_prepare_wide_kernel(ConvArgs 
                     }
                 }
             } else if (a.freqs) {
-                const int apart = a.rot / 16;
-                const bool low = sub < apart, turned = sub < 2 * apart;
-                const int partner = (tid % KA_WAVE) + (low ? apart : -apart);
                 float other[8];
 #pragma unroll
-                for (int e = 0; e < 8; ++e) other[e] = __shfl(y[e], turned ? partner : tid % KA_WAVE);
+                for (int e = 0; e < 8; ++e) other[e] = __shfl(y[e], partner);
                 if (turned) {
+                    const sp_floatx4 c0 = *reinterpret_cast<const sp_floatx4*>(&cs[i][j0]), c1 = *reinterpret_cast<const sp_floatx4*>(&cs[i][j0 + 4]);
+                    const sp_floatx4 s0 = *reinterpret_cast<const sp_floatx4*>(&sn[i][j0]), s1 = *reinterpret_cast<const sp_floatx4*>(&sn[i][j0 + 4]);
 #pragma unroll
                     for (int e = 0; e < 8; ++e) {
-                        const int j = (low ? sub : sub - apart) * 8 + e;
-                        y[e] = low ? y[e] * cs[i][j] - other[e] * sn[i][j] : y[e] * cs[i][j] + other[e] * sn[i][j];
+                        const float co = e < 4 ? c0[e % 4] : c1[e % 4], si = e < 4 ? s0[e % 4] : s1[e % 4];
+                        y[e] = low ? y[e] * co - other[e] * si : y[e] * co + other[e] * si;
                     }
                 }
             }
@@ -390,9 +434,9 @@ __global__ void __launch_bounds__(SP_THREADS) conv_prepare_wide_kernel(ConvArgs 
             for (int e = 0; e < 8; ++e) o[e] = (bf16_t)y[e];
             if (!live) continue;
             if (is_q) {
-                *reinterpret_cast<sp_bf16x8*>(reinterpret_cast<bf16_t*>(a.q_out) + (size_t)t * a.q_stride + within) = o;
+                *reinterpret_cast<sp_bf16x8*>(reinterpret_cast<bf16_t*>(a.q_out) + (size_t)(first + i) * a.q_stride + within) = o;
             } else {
-                const int at = a.slots ? a.slots[t] : -1;
+                const int at = at_s[i];
                 if (at >= 0)
                     *reinterpret_cast<sp_bf16x8*>(reinterpret_cast<bf16_t*>(a.k_cache) + (((size_t)(at / a.page_size) * a.Hk + (head - a.Hq)) * a.page_size +
                                                   at % a.page_size) * HD + sub * 8) = o;
@@ -404,30 +448,29 @@ __global__ void __launch_bounds__(SP_THREADS) conv_prepare_wide_kernel(ConvArgs 
     if (!live) return;                              // (nothing below meets other lanes)
     const int vc = 8 * mine, vhead = vc / a.hdv, vd = vc % a.hdv;
     bf16_t* vbase = reinterpret_cast<bf16_t*>(a.v_cache);
-    const int at0 = a.slots ? a.slots[first] : -1;
-    if (count == SP_WIDE_RUN && a.page_size == SP_WIDE_RUN && at0 >= 0 && at0 % SP_WIDE_RUN == 0 && a.slots[first + SP_WIDE_RUN - 1] == at0 + SP_WIDE_RUN - 1) {
-        sp_bf16x8 page[8][2];
-        enter(first);
+    const int at0 = at_s[0];
+    if (count == SP_WIDE_V && a.page_size % SP_WIDE_V == 0 && at0 >= 0 && at0 % SP_WIDE_V == 0 && at_s[SP_WIDE_V - 1] == at0 + SP_WIDE_V - 1 &&
+        row_s[SP_WIDE_V - 1] == row_s[0]) {
+        sp_bf16x8 page[8];                          // (places side by side in a page: 16 bytes a channel)
 #pragma unroll
-        for (int i = 0; i < SP_WIDE_RUN; ++i) {
+        for (int i = 0; i < SP_WIDE_V; ++i) {
             float y[8];
-            convolve(first + i, y);
+            convolve(rows[i], y);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) page[e][i / 8][i % 8] = (bf16_t)y[e];
+            for (int e = 0; e < 8; ++e) page[e][i] = (bf16_t)y[e];
         }
-        bf16_t* dst = vbase + (((size_t)(at0 / SP_WIDE_RUN) * a.Hv + vhead) * a.hdv + vd) * SP_WIDE_RUN;
+        bf16_t* dst = vbase + (((size_t)(at0 / a.page_size) * a.Hv + vhead) * a.hdv + vd) * a.page_size + at0 % a.page_size;
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-            *reinterpret_cast<sp_bf16x8*>(dst + (size_t)e * SP_WIDE_RUN) = page[e][0];
-            *reinterpret_cast<sp_bf16x8*>(dst + (size_t)e * SP_WIDE_RUN + 8) = page[e][1];
-        }
+        for (int e = 0; e < 8; ++e) *reinterpret_cast<sp_bf16x8*>(dst + (size_t)e * a.page_size) = page[e];
         return;
     }
-    for (int i = 0; i < count; ++i) {
+#pragma unroll
+    for (int i = 0; i < SP_WIDE_V; ++i) {
+        if (i >= count) break;
         float y[8];
-        enter(first + i);
-        convolve(first + i, y);
-        const int at = a.slots ? a.slots[first + i] : -1;
+        enter(i);
+        convolve(rows[i], y);
+        const int at = at_s[i];
         if (at < 0) continue;
         bf16_t* dst = vbase + (((size_t)(at / a.page_size) * a.Hv + vhead) * a.hdv + vd) * a.page_size + at % a.page_size;
 #pragma unroll
@@ -444,7 +487,7 @@ static int sp_wide_lanes(const ConvArgs& a, int dtype, int n_runs) {
     if (a.freqs && (a.rot > SP_WIDE_MAX_ROT || (!a.interleaved && a.rot % 16 != 0))) return 0;
     if ((uintptr_t)a.u % 16 != 0 || a.u_stride % 8 != 0 || (uintptr_t)a.q_out % 16 != 0 || a.q_stride % 8 != 0) return 0;
     if ((uintptr_t)a.k_cache % 16 != 0 || (uintptr_t)a.v_cache % 16 != 0) return 0;
-    if (a.K > 1 && ((uintptr_t)a.state % 16 != 0 || a.state_stride % 4 != 0)) return 0;
+    if ((uintptr_t)a.taps % 16 != 0 || (a.K > 1 && ((uintptr_t)a.state % 16 != 0 || a.state_stride % 4 != 0))) return 0;
     return lanes;
 }
 
@@ -476,6 +519,7 @@ KA_API int ka_conv_prepare(const void* u, int dtype, long u_stride, const float*
                            const int* run_first, const int* run_count, int n_runs, int single_tokens, hipStream_t stream) {
     KA_CHECK(n >= 0 && n_rows >= 0 && Hq > 0 && Hk > 0 && hd > 0 && Hv > 0 && hdv > 0 && page_size > 0 && K >= 0 && eps >= 0.f, "ka_conv_prepare: bad sizes");
     KA_CHECK((run_first == nullptr) == (run_count == nullptr) && n_runs >= 0, "ka_conv_prepare: runs are two lists");
+    KA_CHECK(!single_tokens || n == n_rows, "ka_conv_prepare: a step of single tokens has as many rows as tokens");
     KA_CHECK(dtype == KA_F32 || dtype == KA_BF16, "ka_conv_prepare: unsupported dtype %d", dtype);
     KA_CHECK(K == 0 || taps != nullptr, "ka_conv_prepare: taps missing");
     KA_CHECK(K <= 1 || state != nullptr, "ka_conv_prepare: a convolution of %d taps needs its state", K);
@@ -491,7 +535,7 @@ KA_API int ka_conv_prepare(const void* u, int dtype, long u_stride, const float*
     a.freqs = freqs; a.rot = freqs ? rot : 0; a.interleaved = interleaved;
     a.state_stride = state_stride; a.normed = normed; a.eps = eps;
     KA_CHECK(K <= 1 || state_stride >= (long)(K - 1) * a.C, "ka_conv_prepare: the state's rows are too short");
-    a.run_first = nullptr; a.run_count = nullptr; a.moves_state = 0;
+    a.run_first = nullptr; a.run_count = nullptr; a.single_tokens = 0;
     if (n == 0) return 0;
     const int blocks = (a.C + SP_THREADS - 1) / SP_THREADS;
     KA_CHECK(blocks <= 65535, "ka_conv_prepare: too many channels %d", a.C);
@@ -501,9 +545,10 @@ KA_API int ka_conv_prepare(const void* u, int dtype, long u_stride, const float*
     const int wide = sp_wide_lanes(a, dtype, grid_runs);
     if (wide) {
         if (by_runs) { a.run_first = run_first; a.run_count = run_count; }
-        a.moves_state = K > 1 && single_tokens;
+        a.single_tokens = single_tokens;
         const int per = 8 * SP_THREADS;
-        const dim3 grid(ka_cdiv((long)(Hq + Hk) * hd, per) + ka_cdiv((long)Hv * hdv, per), grid_runs);
+        const dim3 grid(ka_cdiv((long)(Hq + Hk) * hd, per) + ka_cdiv((long)Hv * hdv, per), grid_runs,
+                        by_runs ? SP_WIDE_RUN / SP_WIDE_QK : 1);
         switch (wide) {
             case 2: hipLaunchKernelGGL(conv_prepare_wide_kernel<2>, grid, dim3(SP_THREADS), 0, stream, a); break;
             case 4: hipLaunchKernelGGL(conv_prepare_wide_kernel<4>, grid, dim3(SP_THREADS), 0, stream, a); break;
@@ -519,7 +564,7 @@ KA_API int ka_conv_prepare(const void* u, int dtype, long u_stride, const float*
     } else if (dtype == KA_F32) hipLaunchKernelGGL(conv_prepare_kernel<float>, dim3(n, n > SP_SPREAD_TOKENS ? 1 : blocks), dim3(SP_THREADS), 0, stream, a);
     else hipLaunchKernelGGL(conv_prepare_kernel<bf16_t>, dim3(n, n > SP_SPREAD_TOKENS ? 1 : blocks), dim3(SP_THREADS), 0, stream, a);
     KA_LAUNCH_CHECK();
-    if (K > 1 && n_rows > 0 && !a.moves_state) {
+    if (K > 1 && n_rows > 0 && !a.single_tokens) {
         if (dtype == KA_F32) hipLaunchKernelGGL(conv_state_kernel<float>, dim3(n_rows, blocks), dim3(SP_THREADS), 0, stream, a);
         else hipLaunchKernelGGL(conv_state_kernel<bf16_t>, dim3(n_rows, blocks), dim3(SP_THREADS), 0, stream, a);
         KA_LAUNCH_CHECK();

@@ -71,6 +71,9 @@ _SIGNATURES = {
     "ka_experts_gemm_supported": [_c_long, _c_int, _c_int, _c_long, _c_int, _c_int],
     "ka_experts_gemm_bf16": [_c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
                              _c_float, _c_float, _c_void_p, _c_long, _c_int, _c_int, _c_void_p],
+    "ka_experts_few_supported": [_c_int, _c_long, _c_int, _c_int, _c_int],
+    "ka_experts_few_bf16": [_c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float,
+                            _c_float, _c_void_p, _c_long, _c_int, _c_void_p],
     "ka_matrix_memory_chunks_bf16": [_c_void_p, _c_void_p, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_void_p, _c_void_p, _c_void_p,
                                      _c_void_p, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_float,
                                      _c_void_p, _c_int, _c_void_p],
@@ -948,6 +951,30 @@ def gated_chunks_bf16(projected, offsets, pre, tau, q_scale, state, cu_q, row_sl
     _check(handle.ka_gated_chunks_bf16(base + oq * size, base + ok * size, base + ov * size, stride, pre.data_ptr(), float(tau), float(q_scale),
                                        state.data_ptr(), state.stride(0), cu_q.data_ptr(), row_slot.data_ptr(), raw.data_ptr(), scratch.data_ptr(),
                                        n, n_rows, n_heads, head_dim, value_dim, stream_ptr()))
+    return True
+
+
+def experts_few_bf16(h, pairs, down, chosen, hidden, y, act, clamp=None) -> bool:
+    """Both linears of the chosen experts for a step of few pairs on the matrix cores, every chosen expert's weights read once: operands as
+    ``experts_feed_forward_bf16`` takes them, with ``hidden`` bf16 ``[n top, hidden]`` (the pairs' own rows). False: not covered, nothing was run."""
+    n, top = chosen.shape
+    n_experts, n_pair_rows, dim = pairs.shape
+    ff = down.shape[2]
+    handle = lib()
+    lda = h.stride(0) if n > 1 else max(h.stride(0), dim)
+    core._dev(h, pairs, down, chosen, hidden, y)
+    if h.dtype != torch.bfloat16 or h.data_ptr() % 16 or pairs.data_ptr() % 16 or down.data_ptr() % 16 or hidden.data_ptr() % 16 \
+            or not handle.ka_experts_few_supported(n * top, lda, n_pair_rows, dim, act) or not handle.ka_experts_few_supported(n * top, ff, dim, ff, 0):
+        return False
+    if tuple(down.shape) != (n_experts, dim, ff) or n_pair_rows != (2 * ff if act & 0x100 else ff) or pairs.dtype != torch.bfloat16 or down.dtype != torch.bfloat16:
+        raise KernelError("experts: weights of the two linears do not belong together")
+    if y.dtype != torch.float32 or tuple(y.shape) != (n * top, dim) or not y.is_contiguous() or chosen.dtype != torch.int32 or not chosen.is_contiguous() \
+            or hidden.dtype != torch.bfloat16 or tuple(hidden.shape) != (n * top, ff) or not hidden.is_contiguous():
+        raise KernelError("experts: fp32 outputs [pairs, dim], bf16 hidden rows [pairs, hidden] and int32 choices [n, top] expected")
+    _check(handle.ka_experts_few_bf16(h.data_ptr(), lda, top, pairs.data_ptr(), chosen.data_ptr(), n * top, n_experts, n_pair_rows, dim, act,
+                                      *core._clamp_args(clamp, act), hidden.data_ptr(), ff, 0, stream_ptr()))
+    _check(handle.ka_experts_few_bf16(hidden.data_ptr(), ff, 1, down.data_ptr(), chosen.data_ptr(), n * top, n_experts, dim, ff, 0,
+                                      *core._clamp_args(None, 0), y.data_ptr(), dim, 1, stream_ptr()))
     return True
 
 

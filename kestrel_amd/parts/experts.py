@@ -25,15 +25,17 @@ class RoutedExperts(FeedForward):
 
     When the weights are bound, the experts' ``gate`` and ``up`` rows are laid in pairs and the experts stacked
     (``[E, 2 hidden, dim]``, plain ones ``[E, hidden, dim]``; ``[E, dim, hidden]``). A step runs: the router's linear (fp32), the choice
-    (``ops.core.route``), the experts' two linears, and the weighted sum. In bf16 steps of at least
-    ``PAIRS_BY_EXPERT_FROM`` pairs, the pairs are listed by expert and each expert's pairs go through the matrix cores
-    together (``ops.fast.experts_feed_forward_bf16``); otherwise, and in fp32, every pair is computed by itself, its expert's
-    weights streamed once for it (``ops.core.experts_linear``). Measured at 48 pairs over 62 experts, where the lists hold
-    hardly more than a pair an expert: 1.28 ms a step by lists, 1.42 pair by pair. Either way a pair's result depends on
-    its own row alone."""
+    (``ops.core.route``), the experts' two linears, and the weighted sum. In bf16, by the number of pairs (token, choice): a
+    step of up to ``PAIR_BY_PAIR_TO`` computes every pair by itself, its expert's weights streamed for it
+    (``ops.core.experts_linear``; fp32 always does); up to ``FEW_PAIRS_TO`` every chosen expert's weights are streamed once past its pairs
+    (``ops.fast.experts_few_bf16``); beyond, the pairs are listed by expert first and each expert's go through the matrix cores in
+    tiles (``ops.fast.experts_feed_forward_bf16``). Measured, both linears, 31 experts of 2,048 x 704: 4 tokens of 5 pairs 38, 38 and 94
+    us in this order, 8 tokens 62, 52 and 98, 32 tokens 201, 72 and 106, 96 tokens (480 pairs) -, 118 and 119. Either way a
+    pair's result depends on its own row alone."""
 
     replays_every_step = True
-    PAIRS_BY_EXPERT_FROM = 33
+    PAIR_BY_PAIR_TO = 20
+    FEW_PAIRS_TO = 512
 
     def __init__(self, spec: RoutedExpertsSpec) -> None:
         super().__init__(spec)
@@ -133,9 +135,11 @@ class RoutedExperts(FeedForward):
         hidden = ws.get("experts.hidden", (n * top, spec.hidden_dim), self.dtype)
         y = ws.get("experts.y", (n * top, spec.dim), torch.float32)
         done = False
-        if self.dtype == torch.bfloat16 and n * top >= self.PAIRS_BY_EXPERT_FROM:
+        if self.dtype == torch.bfloat16 and n * top > self.PAIR_BY_PAIR_TO:
             from ..ops import fast
-            done = fast.experts_feed_forward_bf16(h, self.pairs, self.down, chosen, hidden, y, self.up_act, ws, clamp=self.clamp)
+            operands = (h, self.pairs, self.down, chosen, hidden, y, self.up_act)
+            done = n * top <= self.FEW_PAIRS_TO and fast.experts_few_bf16(*operands, clamp=self.clamp)
+            done = done or fast.experts_feed_forward_bf16(*operands, ws, clamp=self.clamp)
         if not done:
             flat = chosen.view(-1)
             core.experts_linear(h, top, self.pairs, flat, hidden, self.up_act, clamp=self.clamp)

@@ -335,6 +335,10 @@ def test_plain_experts_and_the_weighted_sum_kernels(n, dim, ff, n_experts, top, 
         y = torch.full((n * top, dim), float("nan"), device=DEV)
         assert fast.experts_feed_forward_bf16(h.to(DEV), up.to(DEV), down.to(DEV), chosen.to(DEV), None, y, act, Workspace(torch.device(DEV)))
         combined(y, "by expert")
+    if dtype == torch.bfloat16 and dim % 8 == 0 and ff % 8 == 0 and n * top <= 512:
+        y = torch.full((n * top, dim), float("nan"), device=DEV)
+        assert fast.experts_few_bf16(h.to(DEV), up.to(DEV), down.to(DEV), chosen.to(DEV), torch.zeros(n * top, ff, dtype=dtype, device=DEV), y, act)
+        combined(y, "few pairs")
 
 
 @pytest.mark.parametrize("kernel, dtype", [("generic", torch.float32), ("generic", torch.bfloat16), ("mfma", torch.bfloat16)],
@@ -491,7 +495,7 @@ def test_the_matrix_core_kernels_run_where_sizes_allow():
         for model in ("P", "R"):
             calls.clear()
             folder = cases.model_dir(model)
-            for length in (50, 80):              # (too short for its latents to be lifted, and long enough)
+            for length in (50, 270):             # (too short for its latents to be lifted and for lists of experts, and long enough)
                 helpers.replay(_runner(folder, torch.bfloat16), {"r": Request("r", _ids(folder, 900, length))}, [[("r", length)]])
             assert set(calls) == set(names) and all(bool(d) for done in calls.values() for d in done), (model, calls)
     finally:
