@@ -388,3 +388,151 @@ KA_API int ka_heads_rmsnorm(const float* raw, const float* gain, const void* gat
     KA_LAUNCH_CHECK();
     return 0;
 }
+
+// ----------------------------------------------------------------------------
+// One token of a recurrence that forgets channel by channel, from the projected row to the input of the output projection in
+// one launch: the decay's second linear z = W_a2 low + b and the decays, the head's state moved on by the token, the read-out, its
+// norm, gain and gate. A workgroup takes a head of a row; a group of 16 lanes takes value channels, NV times four key channels
+// a lane. The state is asked for before anything that it meets is computed. A row without a request gets zeros.
+// ----------------------------------------------------------------------------
+struct GatedStepArgs {
+    const void* row;            // [n, stride]: the projected rows (row r: the token of row r)
+    long stride;
+    int at_q, at_k, at_v, at_gate, at_low, rank;
+    const void* a2;             // [H d, rank]
+    const float* a2_bias;       // [H d]
+    const float* gain;          // [dv]
+    float* state;               // [slots, state_stride]: S [H, dv, d]
+    long state_stride;
+    const int* row_slot;
+    void* out;                  // [n, out_stride]
+    long out_stride;
+    int H, d, dv;
+    float per_tau, q_scale, eps;
+};
+
+constexpr int LS_MAX_D = 256, LS_MAX_DV = 512, LS_MAX_RANK = 1024;
+
+template <typename T, int NV>
+__global__ void __launch_bounds__(LA_THREADS) gated_step_kernel(GatedStepArgs a) {
+    constexpr int LANES = 16, GROUPS = LA_THREADS / LANES, AT_ONCE = 8 / NV;      // value channels of a group in flight
+    __shared__ __attribute__((aligned(16))) float q_s[LS_MAX_D], k_s[LS_MAX_D], w_s[LS_MAX_D];
+    __shared__ float low_s[LS_MAX_RANK], o_s[LS_MAX_DV], v_s[LS_MAX_DV], part[LA_THREADS / KA_WAVE];
+    const int head = blockIdx.x, r = blockIdx.y, tid = threadIdx.x;
+    const int d = a.d, dv = a.dv;
+    const T* row = reinterpret_cast<const T*>(a.row) + (size_t)r * a.stride;
+    T* out = reinterpret_cast<T*>(a.out) + (size_t)r * a.out_stride + (size_t)head * dv;
+    const int slot = a.row_slot[r];
+    if (slot < 0) {
+        for (int j = tid; j < dv; j += LA_THREADS) out[j] = ka_from_float<T>(0.f);
+        return;
+    }
+    const int group = tid / LANES, lane = tid % LANES;
+    float* S = a.state + (size_t)slot * a.state_stride + (size_t)head * d * dv;
+    float4 s[AT_ONCE][NV];
+    auto fetch = [&](int j0) {
+#pragma unroll
+        for (int m = 0; m < AT_ONCE; ++m)
+#pragma unroll
+            for (int u = 0; u < NV; ++u) {
+                const int j = j0 + m * GROUPS + group, i = (u * LANES + lane) * 4;
+                s[m][u] = j < dv && i < d ? *reinterpret_cast<const float4*>(S + (size_t)j * d + i) : make_float4(0.f, 0.f, 0.f, 0.f);
+            }
+    };
+    fetch(0);
+    for (int c = tid; c < a.rank; c += LA_THREADS) low_s[c] = ka_to_float(row[a.at_low + c]);
+    for (int i = tid; i < d; i += LA_THREADS) {
+        q_s[i] = ka_to_float(row[a.at_q + head * d + i]) * a.q_scale;
+        k_s[i] = ka_to_float(row[a.at_k + head * d + i]);
+    }
+    for (int j = tid; j < dv; j += LA_THREADS) v_s[j] = ka_to_float(row[a.at_v + head * dv + j]);
+    __syncthreads();
+    // (four lanes a key channel)
+    for (int i0 = 0; i0 < d; i0 += LA_THREADS / 4) {
+        const int i = min(i0 + tid / 4, d - 1);
+        const T* w = reinterpret_cast<const T*>(a.a2) + ((size_t)head * d + i) * a.rank;
+        float z = 0.f;
+#pragma unroll 8
+        for (int c = tid % 4; c < a.rank; c += 4) z = fmaf(ka_to_float(w[c]), low_s[c], z);
+        z = ka_lanes_reduce<1, 4>(z, KaSum{}) + a.a2_bias[head * d + i];
+        if (tid % 4 == 0) w_s[i] = ka_decay<sizeof(T) == 2>(z, a.per_tau);
+    }
+    __syncthreads();
+    float4 q[NV], k[NV], w[NV];
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+        const int i = min((u * LANES + lane) * 4, d - 4);
+        q[u] = *reinterpret_cast<const float4*>(q_s + i);
+        k[u] = *reinterpret_cast<const float4*>(k_s + i);
+        w[u] = *reinterpret_cast<const float4*>(w_s + i);
+    }
+    float ss = 0.f;
+    for (int j0 = 0; j0 < dv; j0 += AT_ONCE * GROUPS) {
+        if (j0 > 0) fetch(j0);
+#pragma unroll
+        for (int m = 0; m < AT_ONCE; ++m) {
+            const int j = j0 + m * GROUPS + group;
+            const float v = j < dv ? v_s[j] : 0.f;
+            float acc = 0.f;
+#pragma unroll
+            for (int u = 0; u < NV; ++u) {
+                const int i = (u * LANES + lane) * 4;
+                if (i >= d) continue;
+                float4& x = s[m][u];
+                x.x = fmaf(w[u].x, x.x, k[u].x * v);
+                x.y = fmaf(w[u].y, x.y, k[u].y * v);
+                x.z = fmaf(w[u].z, x.z, k[u].z * v);
+                x.w = fmaf(w[u].w, x.w, k[u].w * v);
+                acc = fmaf(q[u].x, x.x, acc);
+                acc = fmaf(q[u].y, x.y, acc);
+                acc = fmaf(q[u].z, x.z, acc);
+                acc = fmaf(q[u].w, x.w, acc);
+                if (j < dv) *reinterpret_cast<float4*>(S + (size_t)j * d + i) = x;
+            }
+            acc = ka_lanes_reduce<1, LANES>(acc, KaSum{});
+            if (lane == 0 && j < dv) {
+                o_s[j] = acc;
+                ss = fmaf(acc, acc, ss);
+            }
+        }
+    }
+    ss = ka_wave_sum(ss);
+    if (tid % KA_WAVE == 0) part[tid / KA_WAVE] = ss;
+    __syncthreads();
+    float total = 0.f;
+#pragma unroll
+    for (int v = 0; v < LA_THREADS / KA_WAVE; ++v) total += part[v];
+    const float scale = 1.0f / sqrtf(total / (float)dv + a.eps);
+    for (int j = tid; j < dv; j += LA_THREADS)
+        out[j] = ka_from_float<T>(o_s[j] * scale * a.gain[j] * la_act<T>(KA_ACT_SILU, ka_to_float(row[a.at_gate + head * dv + j])));
+}
+
+// Whether the kernel covers heads of these sizes: key channels in steps of four.
+KA_API int ka_gated_step_supported(int d, int dv, int rank) {
+    return d > 0 && d % 4 == 0 && d <= LS_MAX_D && dv > 0 && dv <= LS_MAX_DV && rank > 0 && rank <= LS_MAX_RANK ? 1 : 0;
+}
+
+KA_API int ka_gated_step(const void* row, long stride, int dtype, int at_q, int at_k, int at_v, int at_gate, int at_low, int rank, const void* a2,
+                         const float* a2_bias, const float* gain, float tau, float q_scale, float eps, float* state, long state_stride,
+                         const int* row_slot, void* out, long out_stride, int n, int H, int d, int dv, hipStream_t stream) {
+    const char* who = "ka_gated_step";
+    KA_CHECK(n >= 0 && n <= 65535 && H > 0 && ka_gated_step_supported(d, dv, rank), "%s: heads of %d x %d channels, a rank of %d are not covered", who, d, dv, rank);
+    KA_CHECK(dtype == KA_F32 || dtype == KA_BF16, "%s: unsupported dtype %d", who, dtype);
+    KA_CHECK(tau > 0.f && eps >= 0.f, "%s: a positive tau and an epsilon that is not negative", who);
+    const long ends[5] = {at_q + (long)H * d, at_k + (long)H * d, at_v + (long)H * dv, at_gate + (long)H * dv, at_low + (long)rank};
+    for (long end : ends) KA_CHECK(end <= stride, "%s: the projected rows are too short", who);
+    KA_CHECK(at_q >= 0 && at_k >= 0 && at_v >= 0 && at_gate >= 0 && at_low >= 0 && out_stride >= (long)H * dv, "%s: bad columns", who);
+    KA_CHECK(state_stride >= (long)H * d * dv && state_stride % 4 == 0 && (uintptr_t)state % 16 == 0, "%s: the state's rows must be 16-byte aligned", who);
+    if (n == 0) return 0;
+    const GatedStepArgs a{row, stride, at_q, at_k, at_v, at_gate, at_low, rank, a2, a2_bias, gain, state, state_stride, row_slot, out, out_stride,
+                          H, d, dv, 1.f / tau, q_scale, eps};
+#define LA_STEP(T)                                                                                                                            \
+    if (d <= 64) hipLaunchKernelGGL((gated_step_kernel<T, 1>), dim3(H, n), dim3(LA_THREADS), 0, stream, a);       \
+    else if (d <= 128) hipLaunchKernelGGL((gated_step_kernel<T, 2>), dim3(H, n), dim3(LA_THREADS), 0, stream, a); \
+    else hipLaunchKernelGGL((gated_step_kernel<T, 4>), dim3(H, n), dim3(LA_THREADS), 0, stream, a)
+    if (dtype == KA_F32) { LA_STEP(float); }
+    else { LA_STEP(bf16_t); }
+#undef LA_STEP
+    KA_LAUNCH_CHECK();
+    return 0;
+}

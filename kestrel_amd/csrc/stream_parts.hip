@@ -61,38 +61,50 @@ __device__ __forceinline__ void st_step_regs(const StreamArgs& a, Piece piece, f
     for (int s = 0; s < S; ++s) in[s] = a.into ? a.into[s] : 1.f;
     float4 u[PIECES];
     float sum = 0.f;
+    // (all that a few pieces need is asked for before anything is stored)
+    constexpr int AT_ONCE = PIECES < 4 ? PIECES : 4;
 #pragma unroll
-    for (int p = 0; p < PIECES; ++p) {
-        const int c = (p * ST_THREADS + tid) * 4;
-        u[p] = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (c < dim) {
-            float4 v[S];
+    for (int p0 = 0; p0 < PIECES; p0 += AT_ONCE) {
+        float4 v[AT_ONCE][S], y[AT_ONCE];
+#pragma unroll
+        for (int p = 0; p < AT_ONCE; ++p) {
+            const int c = ((p0 + p) * ST_THREADS + tid) * 4;
+            if (c >= dim) continue;
             if (a.embedded) {
-                const float4 e = *reinterpret_cast<const float4*>(a.embedded + (size_t)i * dim + c);
+                v[p][0] = *reinterpret_cast<const float4*>(a.embedded + (size_t)i * dim + c);
+            } else {
+#pragma unroll
+                for (int s = 0; s < S; ++s) v[p][s] = *reinterpret_cast<const float4*>(row + (size_t)s * dim + c);
+            }
+            if (writes) y[p] = piece(c);
+        }
+#pragma unroll
+        for (int p = 0; p < AT_ONCE; ++p) {
+            const int c = ((p0 + p) * ST_THREADS + tid) * 4;
+            float4& sums = u[p0 + p];
+            sums = make_float4(0.f, 0.f, 0.f, 0.f);
+            if (c >= dim) continue;
+            if (a.embedded) {
 #pragma unroll
                 for (int s = 0; s < S; ++s) {
-                    v[s] = e;
-                    *reinterpret_cast<float4*>(row + (size_t)s * dim + c) = e;
+                    v[p][s] = v[p][0];
+                    *reinterpret_cast<float4*>(row + (size_t)s * dim + c) = v[p][0];
                 }
-            } else {
-#pragma unroll
-                for (int s = 0; s < S; ++s) v[s] = *reinterpret_cast<const float4*>(row + (size_t)s * dim + c);
             }
             if (writes) {
-                const float4 y = piece(c);
 #pragma unroll
                 for (int t = 0; t < S; ++t) {
-                    float4 w = make_float4(o[t] * y.x, o[t] * y.y, o[t] * y.z, o[t] * y.w);
+                    float4 w = make_float4(o[t] * y[p].x, o[t] * y[p].y, o[t] * y[p].z, o[t] * y[p].w);
 #pragma unroll
-                    for (int s = 0; s < S; ++s) w = st_fma4(m[s][t], v[s], w);
+                    for (int s = 0; s < S; ++s) w = st_fma4(m[s][t], v[p][s], w);
                     *reinterpret_cast<float4*>(row + (size_t)t * dim + c) = w;
-                    u[p] = st_fma4(in[t], w, u[p]);
+                    sums = st_fma4(in[t], w, sums);
                 }
             } else {
 #pragma unroll
-                for (int s = 0; s < S; ++s) u[p] = st_fma4(in[s], v[s], u[p]);
+                for (int s = 0; s < S; ++s) sums = st_fma4(in[s], v[p][s], sums);
             }
-            sum += (u[p].x + u[p].y) + (u[p].z + u[p].w);
+            sum += (sums.x + sums.y) + (sums.z + sums.w);
         }
     }
     if (a.h == nullptr) return;
@@ -211,12 +223,20 @@ __global__ void __launch_bounds__(ST_THREADS) streams_experts_kernel(StreamArgs 
     if constexpr (S > 0) {
         st_step_regs<S, PIECES>(a, [&](int c) {
             float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
-            for (int k = 0; k < e.top; ++k) {
-                const float w = e.weights[(size_t)t * e.top + k];
-                float4 v;
-                if (e.chosen[(size_t)t * e.top + k] < e.E) v = *reinterpret_cast<const float4*>(e.pairs + ((size_t)t * e.top + k) * dim + c);
-                else v = make_float4(ka_to_float(hp[c]), ka_to_float(hp[c + 1]), ka_to_float(hp[c + 2]), ka_to_float(hp[c + 3]));
-                acc = st_fma4(w, v, acc);
+            // (four choices in flight; a choice without weights of its own has a row in `pairs` too, which is not used)
+            for (int k0 = 0; k0 < e.top; k0 += 4) {
+                float4 v[4];
+                float w[4];
+#pragma unroll
+                for (int k = 0; k < 4; ++k) {
+                    const size_t at = (size_t)t * e.top + min(k0 + k, e.top - 1);
+                    w[k] = e.weights[at];
+                    v[k] = *reinterpret_cast<const float4*>(e.pairs + at * dim + c);
+                    if (e.chosen[at] >= e.E) v[k] = make_float4(ka_to_float(hp[c]), ka_to_float(hp[c + 1]), ka_to_float(hp[c + 2]), ka_to_float(hp[c + 3]));
+                }
+#pragma unroll
+                for (int k = 0; k < 4; ++k)
+                    if (k0 + k < e.top) acc = st_fma4(w[k], v[k], acc);
             }
             if (e.shared) acc = st_fma4(sg, *reinterpret_cast<const float4*>(e.shared + (size_t)t * dim + c), acc);
             return acc;

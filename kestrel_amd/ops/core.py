@@ -79,6 +79,9 @@ _SIGNATURES = {
                            _c_void_p],
     "ka_gated_linear_attention": [_c_void_p, _c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_float, _c_float, _c_void_p, _c_long,
                                   _c_void_p, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p],
+    "ka_gated_step_supported": [_c_int, _c_int, _c_int],
+    "ka_gated_step": [_c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_void_p, _c_void_p, _c_void_p, _c_float, _c_float,
+                      _c_float, _c_void_p, _c_long, _c_void_p, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_void_p],
     "ka_heads_rmsnorm": [_c_void_p, _c_void_p, _c_void_p, _c_long, _c_void_p, _c_long, _c_int, _c_int, _c_int, _c_int, _c_float, _c_void_p],
     "ka_experts_combine": [_c_void_p, _c_void_p, _c_long, _c_int, _c_void_p, _c_void_p, _c_int, _c_int, _c_int, _c_void_p, _c_void_p,
                            _c_long, _c_void_p, _c_int, _c_int, _c_void_p],
@@ -564,6 +567,34 @@ def gated_linear_attention(projected: torch.Tensor, offsets, pre: torch.Tensor, 
                                            projected.stride(0) if n > 1 else projected.shape[1], code_of(projected.dtype), pre.data_ptr(),
                                            float(tau), float(q_scale), state.data_ptr(), state.stride(0), cu_q.data_ptr(), row_slot.data_ptr(),
                                            raw.data_ptr(), n, n_rows, n_heads, head_dim, value_dim, stream_ptr()))
+
+
+def gated_step(projected: torch.Tensor, offsets, a2: torch.Tensor, a2_bias: torch.Tensor, gain: torch.Tensor, tau: float, q_scale: float, eps: float,
+               state: torch.Tensor, row_slot: torch.Tensor, out: torch.Tensor, n_heads: int, head_dim: int, value_dim: int) -> bool:
+    """A step of single tokens (row ``r`` brings token ``r``) of gated linear attention in one launch: ``gated_linear_attention`` with ``pre = a2
+    low + a2_bias``, then ``heads_rmsnorm``. ``offsets``: the columns of q, k, v, gate and low in ``projected`` ``[n, ..]``; ``a2`` ``[H hd, rank]`` of
+    its type. False: sizes or alignment not covered, nothing was run."""
+    _dev(projected, a2, a2_bias, gain, state, row_slot, out)
+    n, rank = projected.shape[0], a2.shape[1]
+    who = "gated_step"
+    if not lib().ka_gated_step_supported(int(head_dim), int(value_dim), int(rank)) or state.stride(0) % 4 or state.data_ptr() % 16:
+        return False
+    _need(projected.dim() == 2 and projected.stride(1) == 1 and projected.dtype in (torch.float32, torch.bfloat16), f"{who}: projected rows [n, ..]")
+    _need(row_slot.dtype == torch.int32 and row_slot.numel() == n, f"{who}: as many rows as tokens")
+    _need(a2.dtype == projected.dtype and a2.is_contiguous() and a2.shape[0] == n_heads * head_dim, f"{who}: a2 [H hd, rank]")
+    _need(a2_bias.dtype == torch.float32 and a2_bias.is_contiguous() and a2_bias.numel() == n_heads * head_dim, f"{who}: the bias is fp32 [H hd]")
+    _need(gain.dtype == torch.float32 and gain.is_contiguous() and gain.numel() == value_dim, f"{who}: gain fp32 [dv]")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] == n_heads * head_dim * value_dim,
+          f"{who}: state fp32 [slots, H dv d]")
+    _need(out.dim() == 2 and tuple(out.shape) == (n, n_heads * value_dim) and out.stride(1) == 1 and out.dtype == projected.dtype, f"{who}: out [n, H dv]")
+    oq, ok, ov, og, ol = (int(o) for o in offsets)
+    _need(max(oq + n_heads * head_dim, ok + n_heads * head_dim, ov + n_heads * value_dim, og + n_heads * value_dim, ol + rank) <= projected.shape[1],
+          f"{who}: the projected rows are too short")
+    _check(lib().ka_gated_step(projected.data_ptr(), projected.stride(0) if n > 1 else max(projected.stride(0), projected.shape[1]),
+                               code_of(projected.dtype), oq, ok, ov, og, ol, rank, a2.data_ptr(), a2_bias.data_ptr(), gain.data_ptr(), float(tau),
+                               float(q_scale), float(eps), state.data_ptr(), state.stride(0), row_slot.data_ptr(), out.data_ptr(),
+                               out.stride(0) if n > 1 else max(out.stride(0), n_heads * value_dim), n, n_heads, head_dim, value_dim, stream_ptr()))
+    return True
 
 
 def heads_rmsnorm(raw: torch.Tensor, gain: torch.Tensor, gate: torch.Tensor, out: torch.Tensor, n_heads: int, value_dim: int, eps: float) -> None:

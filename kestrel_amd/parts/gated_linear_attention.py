@@ -24,11 +24,12 @@ class GatedLinearAttention(Mixer):
     Every head's ``o`` is divided by its root mean square (``eps``) and multiplied by the gain ``norm.weight`` ``[hdv]`` that the heads
     share; the concatenated heads are multiplied by ``silu(W_gate h)`` and go through the output projection.
 
-    One launch projects q | k | v | gate | a1 in the activation type; ``z`` comes from a linear of its own with fp32 output (what
-    enters the recurrence besides the projections is fp32). Steps of single tokens, steps of a few tokens, and fp32 runs walk
-    over every row's tokens in order (``ops.core.gated_linear_attention``); longer bf16 steps run on the matrix cores, the
-    recurrence unrolled over chunks of 64 tokens (``ops.fast.gated_chunks_bf16``). Either leaves the read-outs in fp32, which one
-    launch normalises and gates. Rows without a request (the padding of a replayed step) write zeros and touch no state."""
+    One launch projects q | k | v | gate | a1 in the activation type. A step of single tokens is one more launch up to the output
+    projection (``ops.core.gated_step``). Otherwise ``z`` comes from a linear of its own with fp32 output (what enters the recurrence
+    besides the projections is fp32); steps of a few tokens, and fp32 runs, walk over every row's tokens in order
+    (``ops.core.gated_linear_attention``), longer bf16 steps run on the matrix cores, the recurrence unrolled over chunks of 64
+    tokens (``ops.fast.gated_chunks_bf16``); either leaves the read-outs in fp32, which one launch normalises and gates. Rows
+    without a request (the padding of a replayed step) write zeros and touch no state."""
 
     replays_every_step = True
     # Tokens of a step from which the chunks' launches are run instead of the walk over tokens (a chain of that length at most)
@@ -97,11 +98,16 @@ class GatedLinearAttention(Mixer):
         ws = batch.workspace
         if cache.state is None:
             raise RuntimeError("gated linear attention needs its per-request state from the cache manager")
+        if out is None:
+            out = ws.get("gated_attention.out", (n, self.v_dim), self.dtype)
+        sizes = (spec.n_heads, spec.head_dim, spec.value_dim)
+        q_scale = float(spec.head_dim) ** -0.5
+        if batch.decode_only and core.gated_step(projected, (*self.offsets, self.gate_at, self.low_at), self.a2_weight, self.a2_bias, self.gain,
+                                                 float(spec.tau), q_scale, float(spec.eps), cache.state, batch.row_slot, out, *sizes):
+            return out
         pre = ws.get("gated_attention.pre", (n, self.qk_dim), torch.float32)
         linear(projected[:, self.low_at:self.low_at + self.rank], self.a2_weight, self.a2_bias, pre)
         raw = ws.get("gated_attention.raw", (n, self.v_dim), torch.float32)
-        sizes = (spec.n_heads, spec.head_dim, spec.value_dim)
-        q_scale = float(spec.head_dim) ** -0.5
         operands = (projected, self.offsets, pre, float(spec.tau), q_scale, cache.state, batch.cu_q, batch.row_slot, raw, *sizes)
         done = False
         if self.dtype == torch.bfloat16 and not batch.decode_only and n >= self.CHUNKS_FROM_TOKENS:
@@ -112,8 +118,6 @@ class GatedLinearAttention(Mixer):
                 done = fast.gated_chunks_bf16(*operands, ws.get("gated_attention.chunks", (need,), torch.float32))
         if not done:
             core.gated_linear_attention(*operands)
-        if out is None:
-            out = ws.get("gated_attention.out", (n, self.v_dim), self.dtype)
         core.heads_rmsnorm(raw, self.gain, projected[:, self.gate_at:self.gate_at + self.v_dim], out, spec.n_heads, spec.value_dim, float(spec.eps))
         return out
 

@@ -229,6 +229,44 @@ def test_many_rows_of_chunks():
 
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=DTYPE_IDS)
+@pytest.mark.parametrize("d, dv, heads, rank", [(64, 128, 3, 64), (16, 16, 1, 5), (4, 7, 2, 1), (36, 20, 5, 9), (128, 96, 2, 32), (256, 24, 1, 16), (100, 300, 2, 130),
+                                                 (224, 512, 1, 1000)])
+def test_a_token_of_the_recurrence_in_one_launch(d, dv, heads, rank, dtype):
+    """Four tokens in a row of three requests and a row without one, from the projected rows to the gated heads; the state goes
+    through three slots of wider rows, the output into columns of wider rows."""
+    from kestrel_amd.ops import core
+
+    gen = torch.Generator().manual_seed(d + dv)
+    H, tau, eps = heads, 0.7, 1e-4
+    a2 = (torch.randn(H * d, rank, generator=gen) / math.sqrt(rank)).to(dtype)
+    bias, gain = torch.randn(H * d, generator=gen), 1 + 0.3 * torch.randn(dv, generator=gen)
+    wide = torch.full((5, 4 + H * d * dv + 4), 7.0, device=DEV)
+    state = wide[:, 4:4 + H * d * dv]
+    state.fill_(float("nan"))
+    slots = [2, 0, -1, 3]
+    state[[2, 0, 3]] = 0.0
+    columns = 3 + 2 * H * d + 2 * H * dv + rank
+    rows = torch.randn(4, 4, columns, generator=gen).to(dtype)                 # [token, row]
+    offsets = [3, 3 + H * d, 3 + 2 * H * d, 3 + 2 * H * d + H * dv, 3 + 2 * H * d + 2 * H * dv]
+    got = []
+    for x in rows:
+        out = torch.full((4, H * dv + 5), 7.0, dtype=dtype, device=DEV)
+        assert core.gated_step(x.to(DEV), offsets, a2.to(DEV), bias.to(DEV), gain.to(DEV), tau, 0.3, eps, state, _i32(slots), out[:, 5:], H, d, dv)
+        assert bool((out[:, :5] == 7.0).all())
+        got.append(out[:, 5:].double().cpu())
+    for r, slot in enumerate(slots):
+        x = rows[:, r].double()
+        q, k = (x[:, o:o + H * d].reshape(4, H, d) for o in offsets[:2])
+        v, gate = (x[:, o:o + H * dv].reshape(4, H, dv) for o in offsets[2:4])
+        alpha = plain.decays(x[:, offsets[4]:] @ a2.double().T + bias.double(), tau).reshape(4, H, d)
+        want = (plain.rms(plain.gated_sum(q * 0.3, k, v, alpha), eps) * gain.double() * plain.silu(gate)).reshape(4, -1)
+        if slot < 0:
+            want = torch.zeros_like(want)
+        _near(torch.stack([g[r] for g in got]), want, dtype, f"row {r}", atol=1e-4 if dtype == torch.float32 else 2e-3, rtol=1e-4 if dtype == torch.float32 else 1e-2)
+    assert bool(torch.isnan(state[[1, 4]]).all()) and bool((wide[:, :4] == 7.0).all()) and bool((wide[:, 4 + H * d * dv:] == 7.0).all())
+
+
+@pytest.mark.parametrize("dtype", DTYPES, ids=DTYPE_IDS)
 @pytest.mark.parametrize("heads, dv", [(1, 4), (3, 7), (5, 64), (2, 128), (4, 33), (1, 300)])
 def test_norm_of_every_head_with_one_gain_kernel(heads, dv, dtype):
     from kestrel_amd.ops import core
