@@ -452,7 +452,7 @@ def gozatar_models(size: dict, positions: int):
     limits = {"limit": 7.0}
     experts = {"kind": "moe", "expert": {"ff": e["ff"], **limits}, "shared": {"ff": e["shared"], **limits},
                "router": {"experts": e["n"], "top": e["top"], "groups": dict(zip(("count", "keep"), e["groups"]))}}
-    mixer = {"left": {"heads": h, "kv_heads": g, "dim": d, "vdim": d, "scale": 1.0, "conv": size["conv"], "mask": {"size": size["window"]},
+    mixer = {"left": {"heads": h, "kv_heads": g, "dim": d, "vdim": d, "scale": d ** -0.5, "conv": size["conv"], "mask": {"size": size["window"]},
                       "rot": {"base": 10000.0, "dims": d}},
              "right": {"heads": rh, "dim": rd, "vdim": rdv, "tau": 16.0, "decay_rank": size["rank"]}, "left_scale": 0.8, "right_scale": 1.2}
     layers = [{"type": "parallel", "mixer": mixer, "mlp": {"kind": "dense", "ff": size["ff"] * 3 // 2} if kind == "d" else experts}
