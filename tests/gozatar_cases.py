@@ -44,8 +44,7 @@ def _config(vocab, width, streams, eps, layers):
 
 
 CONFIGS: Dict[str, dict] = {
-    # sizes the matrix-core kernels take; three streams; two windows, of two and a half pages and of one and a half, so two
-    # cache groups; a shared expert like the others and one with a size and a limit of its own
+    # sizes the matrix-core kernels take; three streams; two windows, of two and a half pages and of one and a half; a shared expert like the others and one with a size and a limit of its own
     "P": _config(300, 128, 3, 1e-5, [
         parallel((4, 2, 32, 64, 0.3, 4, 40, 16, 10000.0), (3, 32, 40, 8.0, 16), (0.8, 1.3), moe(8, 48, 1.2, 3, (4, 2), (48, 1.2))),
         parallel((2, 2, 64, 32, 0.2, 3, 24, 64, 500.0), (2, 48, 64, 4.0, 24), (1.4, -0.7), dense(176)),

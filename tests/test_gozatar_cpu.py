@@ -97,7 +97,7 @@ def test_streams_cache_groups_and_state():
     assert plan.streams == 3 and all(layer.arrangement == "streams" for layer in plan.layers) and not plan.tied_head
     needs = DecoderModel(plan).cache_needs()
     manager = CacheManager(needs, 16, 40, 3)
-    assert sorted(len(g.entries) for g in manager.groups) == [1, 1, 1, 1] or len(manager.groups) >= 2
+    assert [len(g.entries) for g in manager.groups] == [1, 1, 1, 1]         # (four sizes of keys, values and windows)
     # the convolution's last rows and the recurrence's state lie side by side in one tensor per layer, on 16-byte places
     assert needs[0][1].shape == (3 * 320 + 3 * 32 * 40,) and needs[0][1].dtype == "float32"
     needs = DecoderModel(_plan("Q")).cache_needs()
@@ -127,14 +127,13 @@ def test_plain_streams_by_hand():
 
 
 def test_plain_recurrence_by_hand():
-    one = torch.ones(1, 1, 1, dtype=F64)
     q = torch.tensor([[[1.0, 2.0]], [[3.0, 0.0]], [[1.0, 1.0]]], dtype=F64)
     k = torch.tensor([[[1.0, 1.0]], [[0.0, 1.0]], [[1.0, 0.0]]], dtype=F64)
     v = torch.tensor([[[10.0]], [[20.0]], [[30.0]]], dtype=F64)
     alpha = torch.tensor([[[0.1, 0.1]], [[0.5, 1.0]], [[0.5, 0.1]]], dtype=F64)
     # S: (10, 10); (5, 10 + 20); (2.5 + 30, 3)
     assert plain.gated_sum(q, k, v, alpha).flatten().tolist() == [30.0, 15.0, 35.5]
-    assert float(plain.decays(torch.tensor(0.0, dtype=F64), 2.0)) == pytest.approx(math.sqrt(0.5)) and one.shape == (1, 1, 1)
+    assert float(plain.decays(torch.tensor(0.0, dtype=F64), 2.0)) == pytest.approx(math.sqrt(0.5))
 
 
 def test_plain_convolution_rotation_and_window_by_hand():
